@@ -10,7 +10,8 @@
 //   s_j = cap tanh((q . k_j) scale temp[h] / cap), keys j with 0 <= p - j < window, ordinary softmax,
 //   o = sum_j p_j v_j.
 // The attention kernels also take a mask in chunks (a token sees the keys of its own chunk of `chunk`
-// positions counted from 0, up to itself), a penalty on distance, s_j -= a[h] ln(1 + b[h] (p - j)), a number per
+// positions counted from 0, up to itself), a penalty on distance, s_j -= a[h] ln(1 + b[h] (p - j)) or, without b,
+// s_j -= a[h] (p - j) (behind the cap, like everything that joins the score), a number per
 // head and distance that joins the score, s_j += bias[h][min(p - j, n_bias - 1)] (a table the host lays out by
 // distance, whatever rule groups the distances), and, with a window, the sequence's first `keep_first`
 // positions, which every later token goes on seeing (split 0 walks them before its own keys).
@@ -168,7 +169,7 @@ __global__ __launch_bounds__(256) void capped_attn_kernel(
 #pragma unroll
   for (int g = 0; g < MF_CAP_GC; ++g) {
     fa[g] = (far_a && g < gcount) ? far_a[h0 + g] : 0.f;
-    fb[g] = (far_a && g < gcount) ? far_b[h0 + g] : 0.f;
+    fb[g] = (far_b && g < gcount) ? far_b[h0 + g] : 0.f;
   }
   const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
   __syncthreads();
@@ -211,7 +212,7 @@ __global__ __launch_bounds__(256) void capped_attn_kernel(
       for (int g = 0; g < MF_CAP_GC; ++g) {
         float x = s[g] * tm[g];
         if (cap > 0.f) x = cap * tanhf(x * inv_cap);
-        if (far_a && valid) x -= fa[g] * log1pf(fb[g] * (float)(p - j));
+        if (far_a && valid) x -= fa[g] * (far_b ? log1pf(fb[g] * (float)(p - j)) : (float)(p - j));
         if (bias && valid && g < gcount) x += bias[(size_t)(h0 + g) * n_bias + min(p - j, n_bias - 1)];
         sc[g * MF_CAP_KEYS + threadIdx.x] = valid ? x : -INFINITY;
       }
@@ -360,7 +361,7 @@ MF_API int mf_capped_attn(const void* q, const void* kc, const void* vc, const i
                           int n_bias, int n_splits, int split_len, hipStream_t stream) {
   if (n_tok <= 0) return 0;
   if (nk <= 0 || nh % nk || D <= 0 || D > 512 || V <= 0 || V > 256 || n_splits < 1 || n_splits > 64 ||
-      split_len < 1 || (n_splits > 1 && !part) || !temp || chunk < 0 || (far_a != nullptr) != (far_b != nullptr) ||
+      split_len < 1 || (n_splits > 1 && !part) || !temp || chunk < 0 || (far_b && !far_a) ||
       keep_first < 0 || (keep_first > 0 && chunk > 0) || (bias && n_bias < 1))
     return (int)hipErrorInvalidValue;
   int VP = 1;

@@ -3,7 +3,7 @@
 // compile time: the library is built for a model's sizes).  Semantics as `capped_attn_kernel`:
 // s = cap tanh(q . k scale temp[h] / cap), keys j with 0 <= p - j < window, softmax, o = sum p_j v_j; with
 // `chunk`, a token sees the keys of its own chunk of that many positions only; with `far_a`, `far_b`,
-// s -= far_a[h] ln(1 + far_b[h] (p - j)); with `bias`, s += bias[h][min(p - j, n_bias - 1)]; with a window and
+// s -= far_a[h] ln(1 + far_b[h] (p - j)), and with `far_a` alone s -= far_a[h] (p - j); with `bias`, s += bias[h][min(p - j, n_bias - 1)]; with a window and
 // `keep_first`, every token also sees the sequence's first `keep_first` keys: the wave of split 0 walks their
 // half pages first and then jumps to the half page of its window's first key.
 //
@@ -128,7 +128,7 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
 #pragma unroll
   for (int r = 0; r < RB; ++r) {
     fa[r] = far_a ? far_a[h0 + r] : 0.f;
-    fb[r] = far_a ? far_b[h0 + r] : 0.f;
+    fb[r] = far_b ? far_b[h0 + r] : 0.f;
   }
   const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
 
@@ -207,7 +207,7 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
       for (int j = 0; j < 8; ++j) {
         float y = (j < 4 ? s0[j] : s1[j - 4]) * sc[r];
         if (cap > 0.f) y = cap * fast_tanh(y * inv_cap);
-        if (far_a) y -= fa[r] * __logf(1.0f + fb[r] * dist[j]);
+        if (far_a) y -= fa[r] * (far_b ? __logf(1.0f + fb[r] * dist[j]) : dist[j]);
         if (bias) y += j < 4 ? add_lo[j] : add_hi[j - 4];
         x[j] = seen[j] ? y : -INFINITY;
         mx = fmaxf(mx, x[j]);
@@ -298,7 +298,7 @@ MF_API int mf_capped_mfma(const void* q, const void* kc, const void* vc, const i
   if (n_tiles <= 0) return 0;
   if (d != D || v != V || nk <= 0 || nh % nk || !temp || n_splits < 1 || n_splits > 64 ||
       (n_splits > 1 && (!part || split_len < 32 || split_len % 32)) || chunk < 0 ||
-      (far_a != nullptr) != (far_b != nullptr) || keep_first < 0 || (keep_first > 0 && chunk > 0) || (bias && n_bias < 1))
+      (far_b && !far_a) || keep_first < 0 || (keep_first > 0 && chunk > 0) || (bias && n_bias < 1))
     return (int)hipErrorInvalidValue;
   if (!bias) n_bias = 1;
   const int G = nh / nk;

@@ -14,6 +14,11 @@
 //   the attention's result per head is rotated back by the query token's angles (`unrotate_kernel`),
 //   multiplied by a scale and rounded to the run type.
 //
+// `qk_row_prep_kernel`: queries and keys normed over the whole projection, all heads at once, each with a gain as
+// long as the projection, and a query temperature that grows with the position,
+//   q <- q (1 + coef ln(floor((p + 1) / every) + 1)).
+// A workgroup per (token, part of q | k | v) sums the squares of its part's row and writes it.
+//
 // `qk_norm_prep_kernel`: a workgroup per (token, head of q, k or v): the head in LDS, the sum of squares
 // over the workgroup, then norm, rotation, the cache write (pages as every attention kernel reads them)
 // and q rounded to the run type.  All arithmetic is 32-bit.
@@ -83,6 +88,43 @@ __global__ __launch_bounds__(128) void qk_norm_prep_kernel(
   }
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void qk_row_prep_kernel(
+    const float* __restrict__ qkv, const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
+    float temp_coef, int temp_every, const int* __restrict__ seq_of_tok, const int* __restrict__ positions,
+    const int* __restrict__ page_table, int pt_stride, T* __restrict__ q_out, T* __restrict__ kc, T* __restrict__ vc, int H,
+    int G, int D, int V, int write_cache) {
+  __shared__ float scratch[4];
+  const int t = blockIdx.x, kind = blockIdx.y;      // query, key, value
+  const int n = kind == 0 ? H * D : (kind == 1 ? G * D : G * V);
+  const int C = H * D + G * D + G * V;
+  const float* row = qkv + (size_t)t * C + (kind == 0 ? 0 : (kind == 1 ? H * D : H * D + G * D));
+  const int p = positions[t];
+  if (kind > 0 && !write_cache) return;
+  const int page = kind > 0 ? page_table[(size_t)seq_of_tok[t] * pt_stride + p / MF_PAGE] : 0;
+  const int in_page = p % MF_PAGE;
+  if (kind == 2) {
+    for (int i = threadIdx.x; i < n; i += 256) {
+      const int head = i / V, e = i % V;
+      if (sizeof(T) == 2)      // bfloat16 pages keep V transposed in two halves of 32 keys
+        vc[((((size_t)page * G + head) * 2 + in_page / 32) * V + e) * 32 + in_page % 32] = from_f32<T>(row[i]);
+      else
+        vc[(((size_t)page * G + head) * MF_PAGE + in_page) * V + e] = from_f32<T>(row[i]);
+    }
+    return;
+  }
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < n; i += 256) ss = fmaf(row[i], row[i], ss);
+  float r = 1.0f / sqrtf(block_sum<256>(ss, scratch) / (float)n + eps);
+  if (kind == 0 && temp_every > 0) r *= 1.0f + temp_coef * logf((float)((p + 1) / temp_every) + 1.0f);
+  const float* gain = kind == 0 ? q_gain : k_gain;
+  for (int i = threadIdx.x; i < n; i += 256) {
+    const T v = from_f32<T>(row[i] * r * gain[i]);
+    if (kind == 0) q_out[(size_t)t * n + i] = v;
+    else kc[(((size_t)page * G + i / D) * MF_PAGE + in_page) * D + i % D] = v;
+  }
+}
+
 // rows [tokens][heads][V] of the run type, in place: pair m of every head turns by minus the token's angle m,
 // and everything is multiplied by `scale`
 template <typename T>
@@ -140,5 +182,24 @@ MF_API int mf_unrotate(void* rows, int is_bf16, const float* cos_v, const float*
     unrotate_kernel<bf16><<<grid, 256, 0, stream>>>((bf16*)rows, cos_v, sin_v, positions, H, V, scale);
   else
     unrotate_kernel<float><<<grid, 256, 0, stream>>>((float*)rows, cos_v, sin_v, positions, H, V, scale);
+  return mf_launch_status();
+}
+
+// q_gain float32 [H D], k_gain float32 [G D]; temp_every 0: no query temperature
+MF_API int mf_qk_row_prep(const float* qkv, const float* q_gain, const float* k_gain, float eps, float temp_coef,
+                          int temp_every, const int* seq_of_tok, const int* positions, const int* page_table, int pt_stride,
+                          void* q_out, void* kc, void* vc, int is_bf16, int n_tok, int H, int G, int D, int V, int write_cache,
+                          hipStream_t stream) {
+  if (n_tok <= 0) return 0;
+  if (H <= 0 || G <= 0 || D <= 0 || V <= 0 || !q_gain || !k_gain || temp_every < 0) return (int)hipErrorInvalidValue;
+  const dim3 grid(n_tok, 3);
+  if (is_bf16)
+    qk_row_prep_kernel<bf16><<<grid, 256, 0, stream>>>(qkv, q_gain, k_gain, eps, temp_coef, temp_every, seq_of_tok, positions,
+                                                        page_table, pt_stride, (bf16*)q_out, (bf16*)kc, (bf16*)vc, H, G, D, V,
+                                                        write_cache);
+  else
+    qk_row_prep_kernel<float><<<grid, 256, 0, stream>>>(qkv, q_gain, k_gain, eps, temp_coef, temp_every, seq_of_tok, positions,
+                                                         page_table, pt_stride, (float*)q_out, (float*)kc, (float*)vc, H, G, D, V,
+                                                         write_cache);
   return mf_launch_status();
 }

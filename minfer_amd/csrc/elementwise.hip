@@ -6,12 +6,12 @@
 #include "random_normal.h"
 
 // ---------------------------------------------------------------- embedding
-// h[t][:] = table[ids[t]][:], no scaling (src/graph/cpu_backend.rs:269-285).  The host
-// checks ids before upload; an id outside the table gives a row of NaN so that it shows.
+// h[t][:] = table[ids[t]][:] (src/graph/cpu_backend.rs:269-285), times a scale where a design has
+// one.  The host checks ids before upload; an id outside the table gives a row of NaN so that it shows.
 template <typename TT>
 __global__ __launch_bounds__(256) void embed_kernel(const TT* __restrict__ table,
                                                     const int* __restrict__ ids,
-                                                    float* __restrict__ out, int d, int vocab) {
+                                                    float* __restrict__ out, int d, int vocab, float scale) {
   const int row = blockIdx.x;
   const int id = ids[row];
   float* o = out + (size_t)row * d;
@@ -20,16 +20,16 @@ __global__ __launch_bounds__(256) void embed_kernel(const TT* __restrict__ table
     return;
   }
   const TT* src = table + (size_t)id * d;
-  for (int i = threadIdx.x; i < d; i += 256) o[i] = to_f32(src[i]);
+  for (int i = threadIdx.x; i < d; i += 256) o[i] = to_f32(src[i]) * scale;
 }
 
 MF_API int mf_embed(const void* table, int table_is_bf16, const int* ids, float* out, int rows,
-                    int d, int vocab, hipStream_t stream) {
+                    int d, int vocab, float scale, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (table_is_bf16)
-    embed_kernel<bf16><<<rows, 256, 0, stream>>>((const bf16*)table, ids, out, d, vocab);
+    embed_kernel<bf16><<<rows, 256, 0, stream>>>((const bf16*)table, ids, out, d, vocab, scale);
   else
-    embed_kernel<float><<<rows, 256, 0, stream>>>((const float*)table, ids, out, d, vocab);
+    embed_kernel<float><<<rows, 256, 0, stream>>>((const float*)table, ids, out, d, vocab, scale);
   return mf_launch_status();
 }
 
@@ -725,5 +725,210 @@ __global__ __launch_bounds__(256) void add_rows_kernel(float* __restrict__ h, co
 MF_API int mf_add_rows(float* h, const float* x, size_t n, hipStream_t stream) {
   if (n == 0) return 0;
   add_rows_kernel<<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(h, x, n);
+  return mf_launch_status();
+}
+
+// ---------------------------------------------------------------- square of relu
+template <typename OT>
+__global__ __launch_bounds__(256) void relu2_kernel(const float* __restrict__ x, OT* __restrict__ out, size_t n) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) {
+    const float z = fmaxf(x[i], 0.f);
+    out[i] = from_f32<OT>(z * z);
+  }
+}
+// the same, four values a thread
+template <typename OT>
+__global__ __launch_bounds__(256) void relu2_vec_kernel(const float* __restrict__ x, OT* __restrict__ out, size_t n4) {
+  typedef OT out4 __attribute__((ext_vector_type(4)));
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n4) {
+    const float4 v = ((const float4*)x)[i];
+    const float a = fmaxf(v.x, 0.f), b = fmaxf(v.y, 0.f), c = fmaxf(v.z, 0.f), d = fmaxf(v.w, 0.f);
+    ((out4*)out)[i] = out4{from_f32<OT>(a * a), from_f32<OT>(b * b), from_f32<OT>(c * c), from_f32<OT>(d * d)};
+  }
+}
+
+MF_API int mf_relu2(const float* x, void* out, int out_is_bf16, size_t n, hipStream_t stream) {
+  if (n == 0) return 0;
+  if (n % 4 == 0) {
+    const unsigned blocks = (unsigned)((n / 4 + 255) / 256);
+    if (out_is_bf16)
+      relu2_vec_kernel<bf16><<<blocks, 256, 0, stream>>>(x, (bf16*)out, n / 4);
+    else
+      relu2_vec_kernel<float><<<blocks, 256, 0, stream>>>(x, (float*)out, n / 4);
+    return mf_launch_status();
+  }
+  const unsigned blocks = (unsigned)((n + 255) / 256);
+  if (out_is_bf16)
+    relu2_kernel<bf16><<<blocks, 256, 0, stream>>>(x, (bf16*)out, n);
+  else
+    relu2_kernel<float><<<blocks, 256, 0, stream>>>(x, (float*)out, n);
+  return mf_launch_status();
+}
+
+// ---------------------------------------------------------------- layer norm, alone or behind a scaled sum
+// u = x[row] (JOIN: alpha x[row] + y[row]); out = (u - mean(u)) / sqrt(mean((u - mean(u))^2) + eps) * w.  JOIN
+// writes the 32-bit stream, which may be x itself, and with `cast_out` its rounded copy.  A row of at most
+// 256 * 4 * KEEP values, a multiple of 4 of them, stays in registers; other rows are read once per pass (each
+// thread reads and writes its own values only, so in place is fine).
+template <typename OT, bool JOIN, int KEEP>
+__global__ __launch_bounds__(256) void layernorm_kernel(const float* x, const float* __restrict__ y, float alpha,
+                                                        const int* __restrict__ row_idx, const float* __restrict__ w,
+                                                        OT* out, bf16* __restrict__ cast_out, int d, float eps) {
+  __shared__ float scratch[4];
+  const int row = blockIdx.x;
+  const float* xr = x + (size_t)(row_idx ? row_idx[row] : row) * d;
+  const float* yr = JOIN ? y + (size_t)row * d : nullptr;
+  OT* o = out + (size_t)row * d;
+  bf16* co = cast_out ? cast_out + (size_t)row * d : nullptr;
+  if (KEEP > 0) {
+    typedef OT out4 __attribute__((ext_vector_type(4)));
+    float4 v[KEEP > 0 ? KEEP : 1];
+    float s = 0.f;
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      v[c] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (i < d) {
+        v[c] = *reinterpret_cast<const float4*>(xr + i);
+        if (JOIN) {
+          const float4 b = *reinterpret_cast<const float4*>(yr + i);
+          v[c].x = fmaf(alpha, v[c].x, b.x);
+          v[c].y = fmaf(alpha, v[c].y, b.y);
+          v[c].z = fmaf(alpha, v[c].z, b.z);
+          v[c].w = fmaf(alpha, v[c].w, b.w);
+        }
+      }
+      s += (v[c].x + v[c].y) + (v[c].z + v[c].w);
+    }
+    const float mean = block_sum<256>(s, scratch) / (float)d;
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      if ((c * 256 + (int)threadIdx.x) * 4 < d) {
+        v[c].x -= mean;
+        v[c].y -= mean;
+        v[c].z -= mean;
+        v[c].w -= mean;
+      }
+      ss = fmaf(v[c].x, v[c].x, ss);
+      ss = fmaf(v[c].y, v[c].y, ss);
+      ss = fmaf(v[c].z, v[c].z, ss);
+      ss = fmaf(v[c].w, v[c].w, ss);
+    }
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, scratch) / (float)d + eps);
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < d) {
+        const float4 g = *reinterpret_cast<const float4*>(w + i);
+        const float4 z = make_float4(v[c].x * r * g.x, v[c].y * r * g.y, v[c].z * r * g.z, v[c].w * r * g.w);
+        *reinterpret_cast<out4*>(o + i) = out4{from_f32<OT>(z.x), from_f32<OT>(z.y), from_f32<OT>(z.z), from_f32<OT>(z.w)};
+        if (co) *reinterpret_cast<bf16x4*>(co + i) = bf16x4{(bf16)z.x, (bf16)z.y, (bf16)z.z, (bf16)z.w};
+      }
+    }
+    return;
+  }
+  auto value = [&](int i) { return JOIN ? fmaf(alpha, xr[i], yr[i]) : xr[i]; };
+  float s = 0.f;
+  for (int i = threadIdx.x; i < d; i += 256) s += value(i);
+  const float mean = block_sum<256>(s, scratch) / (float)d;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < d; i += 256) {
+    const float c = value(i) - mean;
+    ss = fmaf(c, c, ss);
+  }
+  const float r = 1.0f / sqrtf(block_sum<256>(ss, scratch) / (float)d + eps);
+  for (int i = threadIdx.x; i < d; i += 256) {
+    const float z = (value(i) - mean) * r * w[i];
+    o[i] = from_f32<OT>(z);
+    if (co) co[i] = (bf16)z;
+  }
+}
+
+template <typename OT, bool JOIN>
+static int launch_layernorm(const float* x, const float* y, float alpha, const int* row_idx, const float* w, OT* out,
+                            bf16* cast_out, int rows, int d, float eps, hipStream_t stream) {
+#define MF_GO(KEEP) \
+  layernorm_kernel<OT, JOIN, KEEP><<<rows, 256, 0, stream>>>(x, y, alpha, row_idx, w, out, cast_out, d, eps)
+  if (d % 4 != 0 || d > 8192) MF_GO(0);
+  else if (d <= 1024) MF_GO(1);
+  else if (d <= 2048) MF_GO(2);
+  else if (d <= 4096) MF_GO(4);
+  else MF_GO(8);
+#undef MF_GO
+  return mf_launch_status();
+}
+
+MF_API int mf_layernorm(const float* x, const int* row_idx, const float* w, void* out, int out_is_bf16, int rows, int d,
+                        float eps, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (d <= 0) return (int)hipErrorInvalidValue;
+  if (out_is_bf16)
+    return launch_layernorm<bf16, false>(x, nullptr, 1.f, row_idx, w, (bf16*)out, nullptr, rows, d, eps, stream);
+  return launch_layernorm<float, false>(x, nullptr, 1.f, row_idx, w, (float*)out, nullptr, rows, d, eps, stream);
+}
+
+// h <- layernorm(alpha h + y) in place; cast_out (bfloat16, or null) gets the new rows rounded
+MF_API int mf_layernorm_join(float* h, const float* y, float alpha, const float* w, void* cast_out, int rows, int d, float eps,
+                             hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (d <= 0) return (int)hipErrorInvalidValue;
+  return launch_layernorm<float, true>(h, y, alpha, nullptr, w, h, (bf16*)cast_out, rows, d, eps, stream);
+}
+
+// ---------------------------------------------------------------- two normed rows, summed
+// out[r] (+)= scale (a[r] / rms(a[r]) wa + b[r] / rms(b[r]) wb), rms with eps inside the root
+template <int KEEP>
+__global__ __launch_bounds__(256) void rmsnorm_pair_kernel(const float* __restrict__ a, const float* __restrict__ wa,
+                                                           const float* __restrict__ b, const float* __restrict__ wb,
+                                                           float* __restrict__ out, int d, float eps, float scale, int add) {
+  __shared__ float scratch[4];
+  const size_t at = (size_t)blockIdx.x * d;
+  float va[KEEP > 0 ? KEEP : 1], vb[KEEP > 0 ? KEEP : 1];
+  float sa = 0.f, sb = 0.f;
+  if (KEEP > 0) {
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = c * 256 + threadIdx.x;
+      va[c] = i < d ? a[at + i] : 0.f;
+      vb[c] = i < d ? b[at + i] : 0.f;
+      sa = fmaf(va[c], va[c], sa);
+      sb = fmaf(vb[c], vb[c], sb);
+    }
+  } else {
+    for (int i = threadIdx.x; i < d; i += 256) {
+      sa = fmaf(a[at + i], a[at + i], sa);
+      sb = fmaf(b[at + i], b[at + i], sb);
+    }
+  }
+  const float ra = scale / sqrtf(block_sum<256>(sa, scratch) / (float)d + eps);
+  const float rb = scale / sqrtf(block_sum<256>(sb, scratch) / (float)d + eps);
+  auto put = [&](int i, float x, float z) {
+    const float v = x * ra * wa[i] + z * rb * wb[i];
+    out[at + i] = add ? out[at + i] + v : v;
+  };
+  if (KEEP > 0) {
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = c * 256 + threadIdx.x;
+      if (i < d) put(i, va[c], vb[c]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < d; i += 256) put(i, a[at + i], b[at + i]);
+  }
+}
+
+MF_API int mf_rmsnorm_pair(const float* a, const float* wa, const float* b, const float* wb, float* out, int rows, int d,
+                           float eps, float scale, int add, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (d <= 0) return (int)hipErrorInvalidValue;
+  if (d <= 2048)
+    rmsnorm_pair_kernel<8><<<rows, 256, 0, stream>>>(a, wa, b, wb, out, d, eps, scale, add);
+  else if (d <= 4096)
+    rmsnorm_pair_kernel<16><<<rows, 256, 0, stream>>>(a, wa, b, wb, out, d, eps, scale, add);
+  else
+    rmsnorm_pair_kernel<0><<<rows, 256, 0, stream>>>(a, wa, b, wb, out, d, eps, scale, add);
   return mf_launch_status();
 }

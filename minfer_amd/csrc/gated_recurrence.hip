@@ -1,12 +1,21 @@
-// Linear attention whose forget gate, one per key channel and token, sets the input gate as well
-// (the HGRN2 recurrence), over the ragged batch of a step, state in 32-bit per sequence slot.
+// Linear attention with a decay per key channel and token, over the ragged batch of a step, state in 32-bit per
+// sequence slot.  Two ways to the decay and to what enters the state:
 //
+// A forget gate that sets the input gate as well (the HGRN2 recurrence; MF_GR_FORGET).
 // Per head, with q_t = silu(q projection) (dim values), v_t the value projection (vdim values) and
 //   a_t = l + (1 - l) sigmoid(f projection + bias)      (dim values, l the learned lower bounds),
 //   S_t = diag(a_t) S_(t-1) + (1 - a_t) v_t^T           (dim x vdim),      o_t = S_t^T q_t.
 // Every head's o_t is then RMS-normed over its vdim values with a gain vector shared by the heads,
 // multiplied by a scale and rounded once (`head_rmsnorm_kernel`).  q | f | v arrive as one 32-bit row per
 // token (the bias already added); gates, state, products and sums are 32-bit throughout.
+//
+// Keys of their own and a decay through a low-rank product (gated linear attention; MF_GR_LOW_RANK, and
+// MF_GR_DECAYS where the decays were formed before).  With q_t, k_t, v_t as projected (q times a scale) and
+// r_t the token's `rank` values,
+//   a_t = sigmoid(A2 r_t + b)^(1/tau)                   (dim values),
+//   S_t = diag(a_t) S_(t-1) + k_t v_t^T,                o_t = S_t^T q_t.
+// q | k | v | ... | r | ... arrive as one 32-bit row per token.  The passes over a prompt read every decay
+// several times, so `low_rank_decay_kernel` forms them once in front; a short walk forms them on the way into LDS.
 //
 // `gated_scan_kernel`: a workgroup owns (segment, head, 64 value columns) and walks the segment's
 // tokens in order; its 256 threads are 4 slices of the key dimension times 64 columns, a thread keeping its
@@ -24,21 +33,39 @@
 
 __device__ __forceinline__ float gr_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
 
+#define MF_GR_FORGET 0
+#define MF_GR_LOW_RANK 1
+#define MF_GR_DECAYS 2
+
+struct LowRankGate {
+  const float* a2;        // [H D][rank]
+  const float* bias;      // [H D]
+  const float* decays;    // [tokens][H D] (MF_GR_DECAYS)
+  int rank, off_r;
+  float inv_tau, q_scale;
+};
+
+// sigmoid(z)^(1/tau)
+__device__ __forceinline__ float root_sigmoid(float z, float inv_tau) {
+  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+}
+
 #define MF_GR_SEQUENCES 0
 #define MF_GR_REDUCE 1
 #define MF_GR_APPLY 2
 
-// proj row: q [H D] | f [H D] | v [H V].  chunk table: int32 [4][n_chunks] = first token, tokens, sequence, last of
+// proj row: q [H D] | f or k [H D] | v [H V] | ....  chunk table: int32 [4][n_chunks] = first token, tokens, sequence, last of
 // its sequence or not.
-template <int DS, int MODE>
+template <int DS, int MODE, int GATE>
 __global__ __launch_bounds__(256) void gated_scan_kernel(const float* __restrict__ proj, int row_len,
                                                          const float* __restrict__ lower,
                                                          const int* __restrict__ cu_seqlens,
                                                          const int* __restrict__ chunks, int n_chunks,
                                                          const int* __restrict__ slot_ids, float* __restrict__ state,
                                                          float* __restrict__ ws, float* __restrict__ ws_a,
-                                                         float* __restrict__ out, int H, int D, int V) {
+                                                         float* __restrict__ out, int H, int D, int V, LowRankGate lr) {
   __shared__ float sq[MF_GR_TT][4 * DS], sa[MF_GR_TT][4 * DS];
+  __shared__ float sk[GATE == MF_GR_FORGET ? 1 : MF_GR_TT][4 * DS];
   __shared__ float partial[MF_GR_TT][4][64];
   const int seg = blockIdx.x, h = blockIdx.y;
   const int col = blockIdx.z * 64 + (threadIdx.x & 63), slice = threadIdx.x >> 6;
@@ -73,14 +100,29 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(const float* __restrict
     for (int i = threadIdx.x; i < nt * 4 * DS; i += 256) {
       const int tt = i / (4 * DS), d = i % (4 * DS);
       const float* row = proj + (size_t)(tb + tt) * row_len + h * D + d;
-      float qv = 0.f, av = 1.f;
+      float qv = 0.f, av = 1.f, kv = 0.f;
       if (d < D) {
-        const float l = lower[h * D + d];
-        av = l + (1.0f - l) * gr_sigmoid(row[off_f]);
-        if (MODE != MF_GR_REDUCE) { const float z = row[0]; qv = z * gr_sigmoid(z); }
+        if (GATE == MF_GR_FORGET) {
+          const float l = lower[h * D + d];
+          av = l + (1.0f - l) * gr_sigmoid(row[off_f]);
+          if (MODE != MF_GR_REDUCE) { const float z = row[0]; qv = z * gr_sigmoid(z); }
+        } else {
+          if (MODE != MF_GR_REDUCE) qv = row[0] * lr.q_scale;
+          kv = row[off_f];                   // the keys stand where the other kind has its gates
+          if (GATE == MF_GR_DECAYS) {
+            av = lr.decays[(size_t)(tb + tt) * H * D + h * D + d];
+          } else {
+            const float* r = proj + (size_t)(tb + tt) * row_len + lr.off_r;
+            const float* w = lr.a2 + (size_t)(h * D + d) * lr.rank;
+            float z = lr.bias[h * D + d];
+            for (int i2 = 0; i2 < lr.rank; ++i2) z = fmaf(w[i2], r[i2], z);
+            av = root_sigmoid(z, lr.inv_tau);
+          }
+        }
       }
       sq[tt][d] = qv;
       sa[tt][d] = av;
+      if (GATE != MF_GR_FORGET) sk[tt][d] = kv;
     }
     __syncthreads();
     for (int tt = 0; tt < nt; ++tt) {
@@ -90,7 +132,7 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(const float* __restrict
       for (int i = 0; i < DS; ++i) {
         const int d = slice * DS + i;
         const float a = sa[tt][d];
-        S[i] = fmaf(a, S[i], (1.0f - a) * vv);
+        S[i] = fmaf(a, S[i], (GATE == MF_GR_FORGET ? 1.0f - a : sk[tt][d]) * vv);
         if (MODE == MF_GR_REDUCE) A[i] *= a;
         else o = fmaf(S[i], sq[tt][d], o);
       }
@@ -159,6 +201,39 @@ __global__ __launch_bounds__(256) void head_rmsnorm_kernel(const float* __restri
   }
 }
 
+// decays[t][d] = sigmoid(bias[d] + a2[d][:] . r_t)^(1/tau) for MF_GR_LR_TOKENS tokens a workgroup, a thread a
+// channel; r_t is the columns off_r .. of the token's row
+#define MF_GR_LR_TOKENS 16
+#define MF_GR_LR_RANK 64      // values of r staged together
+__global__ __launch_bounds__(256) void low_rank_decay_kernel(const float* __restrict__ proj, int row_len, LowRankGate lr,
+                                                             float* __restrict__ decays, int n_tok, int C) {
+  __shared__ float sr[MF_GR_LR_TOKENS][MF_GR_LR_RANK + 1];
+  const int t0 = blockIdx.x * MF_GR_LR_TOKENS, d = blockIdx.y * 256 + threadIdx.x;
+  const int nt = min(MF_GR_LR_TOKENS, n_tok - t0);
+  float z[MF_GR_LR_TOKENS];
+#pragma unroll
+  for (int t = 0; t < MF_GR_LR_TOKENS; ++t) z[t] = d < C ? lr.bias[d] : 0.f;
+  for (int r0 = 0; r0 < lr.rank; r0 += MF_GR_LR_RANK) {
+    const int nr = min(MF_GR_LR_RANK, lr.rank - r0);
+    __syncthreads();
+    for (int i = threadIdx.x; i < MF_GR_LR_TOKENS * nr; i += 256) {
+      const int t = i / nr, r = i % nr;
+      sr[t][r] = t < nt ? proj[(size_t)(t0 + t) * row_len + lr.off_r + r0 + r] : 0.f;
+    }
+    __syncthreads();
+    if (d < C)
+      for (int r = 0; r < nr; ++r) {
+        const float w = lr.a2[(size_t)d * lr.rank + r0 + r];
+#pragma unroll
+        for (int t = 0; t < MF_GR_LR_TOKENS; ++t) z[t] = fmaf(w, sr[t][r], z[t]);
+      }
+  }
+  if (d >= C) return;
+#pragma unroll
+  for (int t = 0; t < MF_GR_LR_TOKENS; ++t)
+    if (t < nt) decays[(size_t)(t0 + t) * C + d] = root_sigmoid(z[t], lr.inv_tau);
+}
+
 #define MF_GR_DISPATCH(CALL)  \
   if (D <= 32) { CALL(8) }    \
   else if (D <= 64) { CALL(16) } \
@@ -167,33 +242,28 @@ __global__ __launch_bounds__(256) void head_rmsnorm_kernel(const float* __restri
 
 MF_API int mf_gr_chunk(void) { return MF_GR_CHUNK; }
 
-// proj float32 [tokens][2 H D + H V]; lower float32 [H D]; state float32 [slots][H][D][V]; out float32 [tokens][H V]
-MF_API int mf_gated_scan(const float* proj, const float* lower, const int* cu_seqlens, const int* slot_ids, float* state,
-                         float* out, int n_seqs, int H, int D, int V, hipStream_t stream) {
-  if (n_seqs <= 0) return 0;
-  if (H <= 0 || D <= 0 || V <= 0 || D > 256) return (int)hipErrorInvalidValue;
-  const int row_len = 2 * H * D + H * V;
+namespace {
+
+template <int GATE>
+int gated_sequences(const float* proj, int row_len, const float* lower, const int* cu_seqlens, const int* slot_ids,
+                    float* state, float* out, int n_seqs, int H, int D, int V, const LowRankGate& lr, hipStream_t stream) {
   dim3 grid(n_seqs, H, (V + 63) / 64);
 #define MF_CALL(DS)                                                                                                    \
-  gated_scan_kernel<DS, MF_GR_SEQUENCES><<<grid, 256, 0, stream>>>(proj, row_len, lower, cu_seqlens, nullptr, 0, slot_ids, \
-                                                                    state, nullptr, nullptr, out, H, D, V);
+  gated_scan_kernel<DS, MF_GR_SEQUENCES, GATE><<<grid, 256, 0, stream>>>(proj, row_len, lower, cu_seqlens, nullptr, 0, \
+                                                                         slot_ids, state, nullptr, nullptr, out, H, D, V, lr);
   MF_GR_DISPATCH(MF_CALL)
 #undef MF_CALL
   return mf_launch_status();
 }
 
-// chunks int32 [4][n_chunks]; seq_first_chunk int32 [n_seqs + 1]; ws float32 [n_chunks][H][D][V] and ws_a
-// float32 [n_chunks][H][D], both scratch
-MF_API int mf_gated_scan_chunked(const float* proj, const float* lower, const int* chunks, int n_chunks,
-                                 const int* seq_first_chunk, const int* slot_ids, float* state, float* ws, float* ws_a,
-                                 float* out, int n_seqs, int H, int D, int V, hipStream_t stream) {
-  if (n_seqs <= 0 || n_chunks <= 0) return 0;
-  if (H <= 0 || D <= 0 || V <= 0 || D > 256 || !ws || !ws_a) return (int)hipErrorInvalidValue;
-  const int row_len = 2 * H * D + H * V;
+template <int GATE>
+int gated_chunks(const float* proj, int row_len, const float* lower, const int* chunks, int n_chunks,
+                 const int* seq_first_chunk, const int* slot_ids, float* state, float* ws, float* ws_a, float* out, int n_seqs,
+                 int H, int D, int V, const LowRankGate& lr, hipStream_t stream) {
   dim3 grid(n_chunks, H, (V + 63) / 64);
 #define MF_CALL(DS)                                                                                                    \
-  gated_scan_kernel<DS, MF_GR_REDUCE><<<grid, 256, 0, stream>>>(proj, row_len, lower, nullptr, chunks, n_chunks, slot_ids, \
-                                                                 state, ws, ws_a, nullptr, H, D, V);
+  gated_scan_kernel<DS, MF_GR_REDUCE, GATE><<<grid, 256, 0, stream>>>(proj, row_len, lower, nullptr, chunks, n_chunks, \
+                                                                      slot_ids, state, ws, ws_a, nullptr, H, D, V, lr);
   MF_GR_DISPATCH(MF_CALL)
 #undef MF_CALL
   int rc = mf_launch_status();
@@ -203,11 +273,55 @@ MF_API int mf_gated_scan_chunked(const float* proj, const float* lower, const in
   rc = mf_launch_status();
   if (rc) return rc;
 #define MF_CALL(DS)                                                                                                    \
-  gated_scan_kernel<DS, MF_GR_APPLY><<<grid, 256, 0, stream>>>(proj, row_len, lower, nullptr, chunks, n_chunks, slot_ids, \
-                                                                state, ws, ws_a, out, H, D, V);
+  gated_scan_kernel<DS, MF_GR_APPLY, GATE><<<grid, 256, 0, stream>>>(proj, row_len, lower, nullptr, chunks, n_chunks, \
+                                                                     slot_ids, state, ws, ws_a, out, H, D, V, lr);
   MF_GR_DISPATCH(MF_CALL)
 #undef MF_CALL
   return mf_launch_status();
+}
+
+}  // namespace
+
+// proj float32 [tokens][2 H D + H V]; lower float32 [H D]; state float32 [slots][H][D][V]; out float32 [tokens][H V]
+MF_API int mf_gated_scan(const float* proj, const float* lower, const int* cu_seqlens, const int* slot_ids, float* state,
+                         float* out, int n_seqs, int H, int D, int V, hipStream_t stream) {
+  if (n_seqs <= 0) return 0;
+  if (H <= 0 || D <= 0 || V <= 0 || D > 256) return (int)hipErrorInvalidValue;
+  return gated_sequences<MF_GR_FORGET>(proj, 2 * H * D + H * V, lower, cu_seqlens, slot_ids, state, out, n_seqs, H, D, V,
+                                       LowRankGate{}, stream);
+}
+
+// chunks int32 [4][n_chunks]; seq_first_chunk int32 [n_seqs + 1]; ws float32 [n_chunks][H][D][V] and ws_a
+// float32 [n_chunks][H][D], both scratch
+MF_API int mf_gated_scan_chunked(const float* proj, const float* lower, const int* chunks, int n_chunks,
+                                 const int* seq_first_chunk, const int* slot_ids, float* state, float* ws, float* ws_a,
+                                 float* out, int n_seqs, int H, int D, int V, hipStream_t stream) {
+  if (n_seqs <= 0 || n_chunks <= 0) return 0;
+  if (H <= 0 || D <= 0 || V <= 0 || D > 256 || !ws || !ws_a) return (int)hipErrorInvalidValue;
+  return gated_chunks<MF_GR_FORGET>(proj, 2 * H * D + H * V, lower, chunks, n_chunks, seq_first_chunk, slot_ids, state, ws, ws_a,
+                                    out, n_seqs, H, D, V, LowRankGate{}, stream);
+}
+
+// rows of row_len floats: q [H D] | k [H D] | v [H V] | ..., the gate's r in the columns off_r ..; a2 float32
+// [H D][rank]; n_chunks 0: every sequence in one walk; decays float32 [tokens][H D], scratch of the chunked form
+MF_API int mf_low_rank_scan(const float* proj, int row_len, const float* a2, const float* bias, int rank, int off_r,
+                            float inv_tau, float q_scale, const int* cu_seqlens, const int* chunks, int n_chunks,
+                            const int* seq_first_chunk, const int* slot_ids, float* state, float* ws, float* ws_a,
+                            float* decays, float* out, int n_tok, int n_seqs, int H, int D, int V, hipStream_t stream) {
+  if (n_tok <= 0 || n_seqs <= 0) return 0;
+  if (H <= 0 || D <= 0 || V <= 0 || D > 256 || rank <= 0 || off_r < 0 || off_r + rank > row_len || row_len < 2 * H * D + H * V ||
+      !a2 || !bias)
+    return (int)hipErrorInvalidValue;
+  LowRankGate lr{a2, bias, decays, rank, off_r, inv_tau, q_scale};
+  if (n_chunks <= 0)
+    return gated_sequences<MF_GR_LOW_RANK>(proj, row_len, nullptr, cu_seqlens, slot_ids, state, out, n_seqs, H, D, V, lr, stream);
+  if (!ws || !ws_a || !decays) return (int)hipErrorInvalidValue;
+  low_rank_decay_kernel<<<dim3((n_tok + MF_GR_LR_TOKENS - 1) / MF_GR_LR_TOKENS, (H * D + 255) / 256), 256, 0, stream>>>(
+      proj, row_len, lr, decays, n_tok, H * D);
+  const int rc = mf_launch_status();
+  if (rc) return rc;
+  return gated_chunks<MF_GR_DECAYS>(proj, row_len, nullptr, chunks, n_chunks, seq_first_chunk, slot_ids, state, ws, ws_a, out,
+                                    n_seqs, H, D, V, lr, stream);
 }
 
 MF_API int mf_head_rmsnorm(const float* o, const float* w, void* y, int y_is_bf16, int rows, int H, int V, float eps,

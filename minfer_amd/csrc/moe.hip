@@ -11,11 +11,16 @@
 // scores for the choice of groups and experts only (the weights take the scores themselves); a group's score is
 // the sum of its `group_top` best (corrected) scores instead of its best; the weights are multiplied by a scale.
 //
+// A table in a router's place (`moe_table_kernel`): row id of the table names the experts of token id, all of one
+// weight.
+//
 // Expert: g = min(gate, limit), u = clamp(up, -limit, limit), y = g sigmoid(1.702 g) (u + 1); or, with
 // `act` 1, the plain gated form y = silu(gate) up.
 // `moe_act_kernel` applies it to the gate|up sums of every expert and multiplies by the token's
 // weight for that expert (0 where it was not chosen), so that one product with the experts' down
 // matrices side by side gives the weighted sum of the chosen experts' outputs.
+// `gated_expert_act_kernel`: an expert that every token takes, weighed by a sigmoid of its own per token:
+// y = silu(gate) up sigmoid(z), from one row gate [F] | up [F] | z | padding.
 // `moe_sparse_*`: for steps of few tokens, only the chosen experts' matrices are read: a wave per
 // output row of a (token, choice) pair.
 #include "common.h"
@@ -160,6 +165,20 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
   }
 }
 
+// chosen[t][:] = table[ids[rows[t]]][:] (rows: which tokens of the step, or all in order), weights all `weight`.
+// The host checks the table's entries and the ids; an id outside the table takes expert 0.
+__global__ __launch_bounds__(256) void moe_table_kernel(const int* __restrict__ table, const int* __restrict__ ids,
+                                                        const int* __restrict__ rows, int* __restrict__ chosen,
+                                                        float* __restrict__ weights, int n_pairs, int top, int vocab,
+                                                        float weight) {
+  const int p = blockIdx.x * 256 + threadIdx.x;
+  if (p >= n_pairs) return;
+  const int t = p / top;
+  const int id = ids[rows ? rows[t] : t];
+  chosen[p] = id >= 0 && id < vocab ? table[(size_t)id * top + p % top] : 0;
+  weights[p] = weight;
+}
+
 #define MF_MOE_ACT_CLAMPED 0
 #define MF_MOE_ACT_SILU 1
 
@@ -183,6 +202,17 @@ __global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ 
     if (wgt != 0.f) v = wgt * expert_act(row[(size_t)e * 2 * F + f], row[(size_t)e * 2 * F + F + f], limit, act);
     y[(size_t)t * E * F + i] = from_f32<OT>(v);
   }
+}
+
+// gu [tokens][row_len]: gate [F] | up [F] | z | ...; y [tokens][F] = silu(gate) up sigmoid(z)
+template <typename OT>
+__global__ __launch_bounds__(256) void gated_expert_act_kernel(const float* __restrict__ gu, int row_len, OT* __restrict__ y,
+                                                               int F) {
+  const int t = blockIdx.x;
+  const float* row = gu + (size_t)t * row_len;
+  const float s = 1.0f / (1.0f + expf(-row[2 * F]));
+  for (int f = blockIdx.y * 256 + threadIdx.x; f < F; f += gridDim.y * 256)
+    y[(size_t)t * F + f] = from_f32<OT>(expert_act(row[f], row[F + f], 0.f, MF_MOE_ACT_SILU) * s);
 }
 
 // ------------------------------------------------------------------ few tokens: the chosen experts only
@@ -443,5 +473,28 @@ MF_API int mf_moe_combine(const float* rows, const int* chosen, const int* rank,
                           float* out, int n_tok, int top, int N, int add, hipStream_t stream) {
   if (n_tok <= 0) return 0;
   moe_combine_kernel<<<dim3(n_tok, (N + 255) / 256), 256, 0, stream>>>(rows, chosen, rank, offsets, weights, out, top, N, add);
+  return mf_launch_status();
+}
+
+// table int32 [vocab][top]; ids int32; rows int32 [n_tok] or null; chosen, weights [n_tok][top]
+MF_API int mf_moe_table(const int* table, const int* ids, const int* rows, int* chosen, float* weights, int n_tok, int top,
+                        int vocab, float weight, hipStream_t stream) {
+  if (n_tok <= 0) return 0;
+  if (top <= 0 || vocab <= 0) return (int)hipErrorInvalidValue;
+  const int pairs = n_tok * top;
+  moe_table_kernel<<<(pairs + 255) / 256, 256, 0, stream>>>(table, ids, rows, chosen, weights, pairs, top, vocab, weight);
+  return mf_launch_status();
+}
+
+MF_API int mf_gated_expert_act(const float* gu, int row_len, void* y, int y_is_bf16, int n_tok, int F, hipStream_t stream) {
+  if (n_tok <= 0 || F <= 0) return 0;
+  if (row_len < 2 * F + 1) return (int)hipErrorInvalidValue;
+  int by = (F + 255) / 256;
+  if (by > 64) by = 64;
+  const dim3 grid(n_tok, by);
+  if (y_is_bf16)
+    gated_expert_act_kernel<bf16><<<grid, 256, 0, stream>>>(gu, row_len, (bf16*)y, F);
+  else
+    gated_expert_act_kernel<float><<<grid, 256, 0, stream>>>(gu, row_len, (float*)y, F);
   return mf_launch_status();
 }

@@ -34,6 +34,8 @@ class StepContext:
     # slot a sequence lives in is not among them: slots are addressed through `slot_ids` only.
     host_new: List[int] = field(default_factory=list)        # new tokens of each sequence
     host_start: Optional[List[int]] = None                   # tokens each held before (None in a decode step)
+    host_tokens: object = None                               # token ids (numpy), None in a decode step
+    host_rows: object = None                                 # `logit_rows` on the host (numpy), None for all rows
     new_lengths: Dict[int, int] = field(default_factory=dict)   # slot -> tokens held after the step
     # between a product that adds into the residual stream and the norm that reads it next (see
     # `parts.base.announce_norm`): the norm the running part's output meets, the norm that follows
@@ -41,6 +43,9 @@ class StepContext:
     norm_next: object = None
     norm_after_block: object = None
     norm_ahead: object = None
+    # the rows (int32 indices on the device) that go on behind the running block, whose feed-forward sees those
+    # alone; None: all of them
+    kept_rows: Optional[torch.Tensor] = None
     _memo: Dict = field(default_factory=dict, repr=False)
 
     def page_table(self, group) -> torch.Tensor:

@@ -237,7 +237,8 @@ class Engine:
             cache=self.cache, n_tokens=n_tok, n_seqs=n_seq, token_ids=views[0], positions=views[1],
             seq_of_tok=views[2], cu_seqlens=views[3], start_pos=views[4], slot_ids=views[5],
             logit_rows=None if rows is None else views[6], page_tables=tables, max_len=max_len,
-            max_new=max(n_new), all_decode=all(n == 1 for n in n_new), host_new=n_new, host_start=start)
+            max_new=max(n_new), all_decode=all(n == 1 for n in n_new), host_new=n_new, host_start=start,
+            host_tokens=flat, host_rows=rows)
         ctx.new_lengths = new_len
         return ctx
 

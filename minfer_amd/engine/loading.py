@@ -18,7 +18,7 @@ from ..kernels import ops
 from ..registry import config_from_dict
 from ..weights.loader import FolderWeights, WeightError
 from ..weights.safetensors_io import SafetensorsError, open_model_files
-from ..weights.random_init import tensor_seed
+from ..weights.random_init import random_table, tensor_seed
 from .model import DecoderModel
 
 DTYPES = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32,
@@ -110,6 +110,8 @@ def random_model(config: Union[Dict[str, Any], Any], seed: int = 0, dtype="bfloa
 
     def get(name: str) -> torch.Tensor:
         ts = expected[name]
+        if ts.below is not None:
+            return random_table(seed, name, ts).to(device)
         if ts.init == "ones":
             return torch.ones(ts.shape, dtype=dt, device=device)
         if ts.init == "zeros":

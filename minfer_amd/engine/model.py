@@ -39,10 +39,10 @@ def _build_block(bs: BlockSpec, rt: Runtime):
              None if bs.feed_forward is None else make_part(FEED_FORWARDS, bs.feed_forward, rt, "feed-forward"),
              {name: make_part(NORMS, spec, rt, "norm") for name, spec in bs.norms.items()}, rt)
     if bs.combiner is None:
-        return cls(*parts)
+        return cls(*parts, **bs.params)
     if not cls.takes_combiner:
         raise ValueError(f"{where}: this arrangement takes no combiner")
-    return cls(*parts, combiner=make_part(COMBINERS, bs.combiner, rt, "combiner"))
+    return cls(*parts, combiner=make_part(COMBINERS, bs.combiner, rt, "combiner"), **bs.params)
 
 
 class DecoderModel:
@@ -141,6 +141,7 @@ class DecoderModel:
         ctx.norm_ahead = None
         for n, e in enumerate(s.schedule):
             keep = rows if (n == last and rows is not None) else None
+            ctx.kept_rows = keep                 # which of the step's tokens the block's feed-forward sees
             # the norm that reads the stream behind this block: the next block's first one, or the final one
             ctx.norm_after_block = (self.final_norm if n == last else
                                     None if s.schedule[n + 1].adds_embedding else

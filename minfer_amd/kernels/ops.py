@@ -29,7 +29,7 @@ class KernelError(RuntimeError):
 _P = c_void_p
 _PROTOTYPES = {
     "elementwise": {
-        "mf_embed": [_P, c_int, _P, _P, c_int, c_int, c_int, _P],
+        "mf_embed": [_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_rmsnorm": [_P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_rmsnorm_cols": [_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_gather_rows": [_P, _P, _P, c_int, c_int, _P],
@@ -49,12 +49,22 @@ _PROTOTYPES = {
         "mf_softcap": [_P, c_float, c_size_t, _P],
         "mf_weighted_sum": [_P, c_int, c_int, _P, _P, _P, c_int, c_int, _P],
         "mf_add_rows": [_P, _P, c_size_t, _P],
+        "mf_relu2": [_P, _P, c_int, c_size_t, _P],
+        "mf_layernorm": [_P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
+        "mf_layernorm_join": [_P, _P, c_float, _P, _P, c_int, c_int, c_float, _P],
+        "mf_rmsnorm_pair": [_P, _P, _P, _P, _P, c_int, c_int, c_float, c_float, c_int, _P],
     },
     "linear_attention": {
         "mf_la_chunk": [],
         "mf_lightning_scan": [_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
         "mf_lightning_scan_chunked": [_P, _P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
         "mf_gated_rmsnorm": [_P, _P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P],
+        "mf_memory_gate_bytes": [],
+        "mf_retention_scan": [_P, c_int, _P, _P, c_int, _P, _P, _P, c_float, c_float, _P, _P, c_int, _P, _P, _P, _P, c_int,
+                              c_int, c_int, c_int, c_int, _P],
+        "mf_memory_scan": [_P, c_int, _P, _P, c_int, _P, _P, c_float, c_float, c_int, c_int, c_float, _P, _P, _P, _P, _P, _P,
+                           _P, _P, c_int, c_int, c_int, c_int, _P],
+        "mf_gated_head_norm": [_P, _P, _P, _P, c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_float, _P],
     },
     "attn_capped": {
         "mf_qkv_conv_prep": [_P, _P, c_int, _P, _P, _P, _P, _P, _P, _P, c_int, c_float, _P, _P, _P, c_int, _P, _P, _P,
@@ -71,18 +81,24 @@ _PROTOTYPES = {
         "mf_qk_norm_prep": [_P, _P, _P, c_float, c_int, _P, _P, _P, _P, c_int, c_int, c_int, _P, _P, c_int, _P, c_int, _P, _P, _P,
                             c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P],
         "mf_unrotate": [_P, c_int, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
+        "mf_qk_row_prep": [_P, _P, _P, c_float, c_float, c_int, _P, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int,
+                           c_int, c_int, c_int, _P],
     },
     "gated_recurrence": {
         "mf_gr_chunk": [],
         "mf_gated_scan": [_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
         "mf_gated_scan_chunked": [_P, _P, _P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
         "mf_head_rmsnorm": [_P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_float, _P],
+        "mf_low_rank_scan": [_P, c_int, _P, _P, c_int, c_int, c_float, c_float, _P, _P, c_int, _P, _P, _P, _P, _P, _P, _P,
+                             c_int, c_int, c_int, c_int, c_int, _P],
     },
     "moe": {
         "mf_moe_route": [_P, c_int, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_float, _P],
         "mf_moe_act": [_P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P],
         "mf_moe_sparse": [_P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
                           _P],
+        "mf_moe_table": [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
+        "mf_gated_expert_act": [_P, c_int, _P, c_int, c_int, c_int, _P],
         "mf_moe_group": [_P, c_int, c_int, _P, _P, _P],
         "mf_moe_gather": [_P, c_int, _P, _P, _P, _P, c_int, c_int, c_int, _P],
         "mf_moe_combine": [_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
@@ -343,13 +359,14 @@ def note_replaced_buffer(old: Optional[torch.Tensor] = None) -> None:
 
 
 # ------------------------------------------------------------------ element-wise
-def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor) -> None:
+def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> None:
+    """out[t] = table[ids[t]] * scale, in 32-bit."""
     _need(table, "embed.table", _FLOATS)
     _need(ids, "embed.ids", torch.int32)
     n, d = ids.numel(), table.shape[1]
     _need(out, "embed.out", torch.float32, (n, d))
     _check(_fn("elementwise", "mf_embed")(_ptr(table), _is_bf16(table), _ptr(ids), _ptr(out), n, d,
-                                           table.shape[0], _stream()), "embed")
+                                           table.shape[0], float(scale), _stream()), "embed")
 
 
 def rmsnorm(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out: torch.Tensor,
@@ -613,6 +630,56 @@ def add_rows(h: torch.Tensor, x: torch.Tensor) -> None:
     _check(_fn("elementwise", "mf_add_rows")(_ptr(h), _ptr(x), h.numel(), _stream()), "add_rows")
 
 
+def relu2(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = max(x, 0)^2; x float32, out run type."""
+    _need(x, "relu2.x", torch.float32)
+    _need(out, "relu2.out", _FLOATS, tuple(x.shape))
+    _check(_fn("elementwise", "mf_relu2")(_ptr(x), _ptr(out), _is_bf16(out), x.numel(), _stream()), "relu2")
+
+
+def layernorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
+              row_idx: Optional[torch.Tensor] = None) -> None:
+    """out = (x - mean) / sqrt(variance + eps) * weight, row by row (row r reads x[row_idx[r]] where given); the
+    variance is the mean of the squared deviations.  x float32, out run type."""
+    _need(x, "layernorm.x", torch.float32)
+    rows, d = out.shape[0], x.shape[-1]
+    _need(out, "layernorm.out", _FLOATS, (rows, d))
+    _need(weight, "layernorm.weight", torch.float32, (d,))
+    if row_idx is not None:
+        _need(row_idx, "layernorm.row_idx", torch.int32, (rows,))
+    elif x.shape[0] != rows:
+        raise KernelError(f"layernorm: x has {x.shape[0]} rows, out has {rows}")
+    _check(_fn("elementwise", "mf_layernorm")(_ptr(x), _ptr(row_idx), _ptr(weight), _ptr(out), _is_bf16(out), rows, d,
+                                               float(eps), _stream()), "layernorm")
+
+
+def layernorm_join(h: torch.Tensor, y: torch.Tensor, alpha: float, weight: torch.Tensor, eps: float,
+                   cast_out: Optional[torch.Tensor] = None) -> None:
+    """h <- layernorm(alpha h + y) * weight, in place (float32 rows both); `cast_out` (bfloat16), where given, also
+    gets the new rows rounded."""
+    _need(h, "layernorm_join.h", torch.float32)
+    rows, d = h.shape
+    _need(y, "layernorm_join.y", torch.float32, (rows, d))
+    _need(weight, "layernorm_join.weight", torch.float32, (d,))
+    if cast_out is not None:
+        _need(cast_out, "layernorm_join.cast_out", torch.bfloat16, (rows, d))
+    _check(_fn("elementwise", "mf_layernorm_join")(_ptr(h), _ptr(y), float(alpha), _ptr(weight), _ptr(cast_out), rows, d,
+                                                    float(eps), _stream()), "layernorm_join")
+
+
+def rmsnorm_pair(a: torch.Tensor, wa: torch.Tensor, b: torch.Tensor, wb: torch.Tensor, eps: float, scale: float,
+                 out: torch.Tensor, accumulate: bool = False) -> None:
+    """out (+)= scale (a / rms(a) * wa + b / rms(b) * wb), row by row, all float32."""
+    rows, d = a.shape
+    _need(a, "rmsnorm_pair.a", torch.float32)
+    _need(b, "rmsnorm_pair.b", torch.float32, (rows, d))
+    _need(wa, "rmsnorm_pair.wa", torch.float32, (d,))
+    _need(wb, "rmsnorm_pair.wb", torch.float32, (d,))
+    _need(out, "rmsnorm_pair.out", torch.float32, (rows, d))
+    _check(_fn("elementwise", "mf_rmsnorm_pair")(_ptr(a), _ptr(wa), _ptr(b), _ptr(wb), _ptr(out), rows, d, float(eps),
+                                                  float(scale), 1 if accumulate else 0, _stream()), "rmsnorm_pair")
+
+
 # ------------------------------------------------------------------ gated linear recurrence
 GR_CHUNK = 64            # tokens of a chunk of the chunked form (MF_GR_CHUNK in csrc/gated_recurrence.hip)
 
@@ -667,6 +734,42 @@ def gated_scan(proj: torch.Tensor, lower: torch.Tensor, cu_seqlens: torch.Tensor
         _ptr(proj), _ptr(lower), _ptr(table), n_chunks, c_void_p(table.data_ptr() + 16 * n_chunks), _ptr(slot_ids),
         _ptr(state), _ptr(ws), c_void_p(ws.data_ptr() + 4 * n_chunks * per), _ptr(out), n_seqs, n_heads, dim, v_dim,
         _stream()), "gated_scan_chunked")
+
+
+def low_rank_scan(proj: torch.Tensor, a2: torch.Tensor, bias: torch.Tensor, off_r: int, tau: float, q_scale: float,
+                  cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n_heads: int,
+                  dim: int, v_dim: int, chunks=None) -> None:
+    """Gated linear attention, S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t q_scale, with
+    a_t = sigmoid(a2 r_t + bias)^(1/tau), over a ragged step.  `proj` float32 rows that begin with q `[H dim]` |
+    k `[H dim]` | v `[H v_dim]` and hold r in the columns `off_r ..`; `a2` float32 `[H dim][rank]`; the rest as
+    `gated_scan`."""
+    n_tok, row_len = proj.shape
+    n_seqs, rank = slot_ids.numel(), a2.shape[1]
+    _need(proj, "low_rank_scan.proj", torch.float32)
+    _need(a2, "low_rank_scan.a2", torch.float32, (n_heads * dim, rank))
+    _need(bias, "low_rank_scan.bias", torch.float32, (n_heads * dim,))
+    _need(cu_seqlens, "low_rank_scan.cu_seqlens", torch.int32, (n_seqs + 1,))
+    _need(slot_ids, "low_rank_scan.slot_ids", torch.int32, (n_seqs,))
+    _need(state, "low_rank_scan.state", torch.float32)
+    if tuple(state.shape[1:]) != (n_heads, dim, v_dim):
+        raise KernelError(f"low_rank_scan: state {tuple(state.shape)} for {n_heads} heads of {dim} x {v_dim}")
+    _need(out, "low_rank_scan.out", torch.float32, (n_tok, n_heads * v_dim))
+    if dim > 256 or row_len < n_heads * (2 * dim + v_dim) or not 0 <= off_r <= row_len - rank:
+        raise KernelError(f"low_rank_scan: rows of {row_len}, {n_heads} heads of {dim} (at most 256) and {v_dim}, the gate's "
+                          f"{rank} values from {off_r}")
+    table, n_chunks, first, ws, ws_a, decays = None, 0, None, None, None, None
+    if chunks is not None:
+        table, n_chunks = chunks
+        _need(table, "low_rank_scan.chunks", torch.int32, (4 * n_chunks + n_seqs + 1,))
+        first = c_void_p(table.data_ptr() + 16 * n_chunks)
+        per = n_heads * dim * v_dim
+        buf = workspace("gr_chunks", n_chunks * (per + n_heads * dim) + n_tok * n_heads * dim, proj.device)
+        ws, ws_a = _ptr(buf), c_void_p(buf.data_ptr() + 4 * n_chunks * per)
+        decays = c_void_p(buf.data_ptr() + 4 * n_chunks * (per + n_heads * dim))
+    _check(_fn("gated_recurrence", "mf_low_rank_scan")(
+        _ptr(proj), row_len, _ptr(a2), _ptr(bias), rank, int(off_r), 1.0 / float(tau), float(q_scale), _ptr(cu_seqlens),
+        _ptr(table), n_chunks, first, _ptr(slot_ids), _ptr(state), ws, ws_a, decays, _ptr(out), n_tok, n_seqs, n_heads, dim,
+        v_dim, _stream()), "low_rank_scan" if chunks is None else "low_rank_scan_chunked")
 
 
 def head_rmsnorm(o: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out: torch.Tensor, n_heads: int,
@@ -732,6 +835,30 @@ def qk_norm_prep(qkv: torch.Tensor, q_gain: Optional[torch.Tensor], k_gain: Opti
         1 if v_from_k else 0, _ptr(page_table),
         page_table.shape[1], _ptr(q_out), _ptr(kcache), _ptr(vcache), _is_bf16(q_out), n_tok, n_heads, n_kv_heads, dim,
         v_dim, 1 if write_cache else 0, _stream()), "qk_norm_prep")
+
+
+def qk_row_prep(qkv: torch.Tensor, q_gain: torch.Tensor, k_gain: torch.Tensor, eps: float, temperature,
+                seq_of_tok: torch.Tensor, positions: torch.Tensor, page_table: torch.Tensor, q_out: torch.Tensor,
+                kcache: torch.Tensor, vcache: torch.Tensor, n_heads: int, n_kv_heads: int, dim: int, v_dim: int,
+                write_cache: bool = True) -> None:
+    """From the 32-bit q|k|v rows of one product: q and k over their root mean square, all heads of a token at once,
+    times the gains `q_gain` `[n_heads dim]` and `k_gain` `[n_kv_heads dim]`; with `temperature` = (coef, every)
+    q further times 1 + coef ln(floor((position + 1) / every) + 1); k and v into the cache pages, q rounded into
+    `q_out`."""
+    n_tok = positions.numel()
+    _need(qkv, "qk_row_prep.qkv", torch.float32, (n_tok, n_heads * dim + n_kv_heads * (dim + v_dim)))
+    _need(q_gain, "qk_row_prep.q_gain", torch.float32, (n_heads * dim,))
+    _need(k_gain, "qk_row_prep.k_gain", torch.float32, (n_kv_heads * dim,))
+    _need(q_out, "qk_row_prep.q_out", _FLOATS, (n_tok, n_heads * dim))
+    _need_kv_pages("qk_row_prep", kcache, vcache, q_out.dtype, n_kv_heads, dim, v_dim)
+    _need(page_table, "qk_row_prep.page_table", torch.int32)
+    _need(seq_of_tok, "qk_row_prep.seq_of_tok", torch.int32, (n_tok,))
+    _need(positions, "qk_row_prep.positions", torch.int32, (n_tok,))
+    coef, every = (0.0, 0) if temperature is None else (float(temperature[0]), int(temperature[1]))
+    _check(_fn("attn_normed", "mf_qk_row_prep")(
+        _ptr(qkv), _ptr(q_gain), _ptr(k_gain), float(eps), coef, every, _ptr(seq_of_tok), _ptr(positions), _ptr(page_table),
+        page_table.shape[1], _ptr(q_out), _ptr(kcache), _ptr(vcache), _is_bf16(q_out), n_tok, n_heads, n_kv_heads, dim, v_dim,
+        1 if write_cache else 0, _stream()), "qk_row_prep")
 
 
 def unrotate(rows: torch.Tensor, value_tables, positions: torch.Tensor, n_heads: int, scale: float = 1.0) -> None:
@@ -806,6 +933,123 @@ def lightning_scan(proj: torch.Tensor, cu_seqlens: torch.Tensor, slot_ids: torch
     _check(_fn("linear_attention", "mf_lightning_scan_chunked")(
         _ptr(proj), _ptr(table), n_chunks, first, _ptr(slot_ids), _ptr(decays), _ptr(state), _ptr(ws), _ptr(out),
         n_seqs, n_heads, dim, v_dim, _stream()), "lightning_scan_chunked")
+
+
+def _la_chunk_args(what: str, chunks, n_seqs: int, dim: int):
+    """(chunk table, its number of chunks, pointer to the sequences' first chunks), or (None, 0, None) for one walk
+    a sequence."""
+    if chunks is None or dim > LA_CHUNKED_MAX_DIM:
+        return None, 0, None
+    table, n_chunks = chunks
+    _need(table, what + ".chunks", torch.int32, (2 * n_chunks + n_seqs + 1,))
+    return table, n_chunks, c_void_p(table.data_ptr() + 8 * n_chunks)
+
+
+def _need_la(what: str, proj, cu_seqlens, slot_ids, state, state_shape, out, n_heads: int, dim: int, v_dim: int):
+    n_tok, n_seqs = proj.shape[0], slot_ids.numel()
+    _need(proj, what + ".proj", torch.float32)
+    _need(cu_seqlens, what + ".cu_seqlens", torch.int32, (n_seqs + 1,))
+    _need(slot_ids, what + ".slot_ids", torch.int32, (n_seqs,))
+    _need(state, what + ".state", torch.float32)
+    if tuple(state.shape[1:]) != tuple(state_shape):
+        raise KernelError(f"{what}: state {tuple(state.shape)}, expected [slots] + {list(state_shape)}")
+    _need(out, what + ".out", torch.float32, (n_tok, n_heads * v_dim))
+    if dim > 256 or proj.shape[1] < n_heads * (2 * dim + v_dim):
+        raise KernelError(f"{what}: rows of {proj.shape[1]} for {n_heads} heads of {dim} (at most 256) and {v_dim}")
+
+
+def retention_scan(proj: torch.Tensor, cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, decays: torch.Tensor,
+                   tables, positions: torch.Tensor, q_scale: float, k_scale: float, state: torch.Tensor, out: torch.Tensor,
+                   n_heads: int, dim: int, v_dim: int, chunks=None) -> None:
+    """S_t = decay S_(t-1) + k_t v_t^T, o_t = S_t^T q_t over a ragged step, with q and k turned in halves by the
+    token's angles (`tables` = (cos, sin) `[positions][rot / 2]`, or None) and times `q_scale`, `k_scale`.  `proj`
+    float32 rows that begin with q | k | v; the chunked form turns their q and k in place.  State, out and chunks
+    as `lightning_scan`."""
+    _need_la("retention_scan", proj, cu_seqlens, slot_ids, state, (n_heads, dim, v_dim), out, n_heads, dim, v_dim)
+    n_tok, row_len = proj.shape
+    n_seqs = slot_ids.numel()
+    _need(decays, "retention_scan.decays", torch.float32, (n_heads,))
+    _need(positions, "retention_scan.positions", torch.int32, (n_tok,))
+    cos = sin = None
+    rot = 0
+    if tables is not None:
+        cos, sin = tables
+        _need(cos, "retention_scan.cos", torch.float32)
+        _need(sin, "retention_scan.sin", torch.float32, tuple(cos.shape))
+        rot = 2 * cos.shape[1]
+        if rot > dim:
+            raise KernelError(f"retention_scan: {rot} rotated values in heads of {dim}")
+    table, n_chunks, first = _la_chunk_args("retention_scan", chunks, n_seqs, dim)
+    ws = workspace("la_chunks", n_chunks * n_heads * dim * v_dim, proj.device) if n_chunks else None
+    _check(_fn("linear_attention", "mf_retention_scan")(
+        _ptr(proj), row_len, _ptr(cu_seqlens), _ptr(table), n_chunks, first, _ptr(slot_ids), _ptr(decays), float(q_scale),
+        float(k_scale), _ptr(cos), _ptr(sin), rot, _ptr(positions), _ptr(state), _ptr(ws), _ptr(out), n_tok, n_seqs, n_heads,
+        dim, v_dim, _stream()), "retention_scan_chunked" if n_chunks else "retention_scan")
+
+
+MEMORY_GATE_FLOATS = 4       # floats of a token's and head's entry in the gates' scratch (MemoryGate)
+
+
+def memory_state_len(n_heads: int, dim: int, v_dim: int) -> int:
+    """Floats of a slot's state of the matrix memory: S `[H][dim][v_dim]`, n `[H][dim]`, m `[H]`."""
+    return n_heads * (dim * v_dim + dim + 1)
+
+
+def memory_scan(proj: torch.Tensor, off_i: int, off_f: int, cap: float, q_scale: float, cu_seqlens: torch.Tensor,
+                slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, den: torch.Tensor, floor: torch.Tensor,
+                n_heads: int, dim: int, v_dim: int, chunks=None) -> None:
+    """The matrix memory with exponential gates over a ragged step: with i = cap tanh(zi / cap),
+    f = logsigmoid(cap tanh(zf / cap)) from the columns `off_i + h`, `off_f + h` of the rows (which begin with q |
+    k | v) and m_t = max(f + m_(t-1), i),  S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k_t v_t^T, n_t
+    likewise with k alone; `out` = S_t^T q_t q_scale, `den` `[tokens][H]` = n_t . q_t q_scale, `floor` = exp(-m_t).
+    `state` float32 `[slots][memory_state_len]`; chunks as `lightning_scan`."""
+    _need_la("memory_scan", proj, cu_seqlens, slot_ids, state, (memory_state_len(n_heads, dim, v_dim),), out, n_heads, dim, v_dim)
+    n_tok, row_len = proj.shape
+    n_seqs = slot_ids.numel()
+    _need(den, "memory_scan.den", torch.float32, (n_tok, n_heads))
+    _need(floor, "memory_scan.floor", torch.float32, (n_tok, n_heads))
+    for name, off in (("off_i", off_i), ("off_f", off_f)):
+        if not 0 <= off <= row_len - n_heads:
+            raise KernelError(f"memory_scan: {name} {off} with {n_heads} heads in rows of {row_len}")
+    table, n_chunks, first = _la_chunk_args("memory_scan", chunks, n_seqs, dim)
+    gates = decay = n_ws = ws = None
+    if n_chunks:
+        g, s, n = MEMORY_GATE_FLOATS * n_tok * n_heads, n_chunks * n_heads * dim * v_dim, n_chunks * n_heads * dim
+        buf = workspace("la_memory", g + s + n + n_chunks * n_heads, proj.device)
+        at = buf.data_ptr()
+        gates, ws, n_ws, decay = (c_void_p(at), c_void_p(at + 4 * g), c_void_p(at + 4 * (g + s)), c_void_p(at + 4 * (g + s + n)))
+    _check(_fn("linear_attention", "mf_memory_scan")(
+        _ptr(proj), row_len, _ptr(cu_seqlens), _ptr(table), n_chunks, first, _ptr(slot_ids), float(q_scale), 1.0, int(off_i),
+        int(off_f), float(cap), _ptr(state), gates, decay, n_ws, ws, _ptr(out), _ptr(den), _ptr(floor), n_seqs, n_heads, dim,
+        v_dim, _stream()), "memory_scan_chunked" if n_chunks else "memory_scan")
+
+
+def gated_head_norm(o: torch.Tensor, proj: torch.Tensor, gate_offset: int, weight: Optional[torch.Tensor], eps: float,
+                    out: torch.Tensor, n_heads: int, act: str, den: Optional[torch.Tensor] = None,
+                    floor: Optional[torch.Tensor] = None) -> None:
+    """out[t][h] = u / sqrt(mean(u^2) + eps) * weight * act(gate[t][h]) with u = o[t][h], or with `den` and `floor`
+    `[tokens][H]` u = o[t][h] / (max(|den|, floor) + 1e-6); the gate is the columns `gate_offset ..` of the 32-bit
+    rows `proj`, `act` "silu" or "sigmoid"; `weight`: None, one vector for all heads, or as long as a row."""
+    rows, n = o.shape
+    _need(o, "gated_head_norm.o", torch.float32)
+    _need(proj, "gated_head_norm.proj", torch.float32)
+    if n % n_heads or proj.shape[0] != rows or not 0 <= gate_offset <= proj.shape[1] - n or act not in ("silu", "sigmoid"):
+        raise KernelError(f"gated_head_norm: rows of {n} values, {n_heads} heads, gate columns {gate_offset}..{gate_offset + n} of "
+                          f"rows {tuple(proj.shape)}, act {act!r}")
+    per_head = 0
+    if weight is not None:
+        per_head = int(weight.numel() == n and n_heads > 1)
+        _need(weight, "gated_head_norm.weight", torch.float32, (n if per_head else n // n_heads,))
+    if (den is None) != (floor is None):
+        raise KernelError("gated_head_norm: den and floor come together")
+    if den is not None:
+        _need(den, "gated_head_norm.den", torch.float32, (rows, n_heads))
+        _need(floor, "gated_head_norm.floor", torch.float32, (rows, n_heads))
+    _need(out, "gated_head_norm.out", _FLOATS, (rows, n))
+    _check(_fn("linear_attention", "mf_gated_head_norm")(
+        _ptr(o), _ptr(den), _ptr(floor), c_void_p(proj.data_ptr() + 4 * gate_offset), proj.shape[1], _ptr(weight), per_head,
+        _ptr(out), _is_bf16(out), rows, n_heads, n // n_heads, 1 if act == "silu" else 0, float(eps), _stream()),
+        "gated_head_norm")
 
 
 def gated_rmsnorm(o: torch.Tensor, proj: torch.Tensor, gate_offset: int, weight: torch.Tensor, eps: float,
@@ -911,7 +1155,8 @@ def capped_attn(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, pag
     """Each query token attends to its sequence's cache rows lo..position with
     s = cap tanh(q . k scale temp[head] / cap) (no cap where `cap` is 0), ordinary softmax; keys of
     `dim` and values of `v_dim` values.  `chunk`: a token sees only the keys of its own chunk of that many
-    positions, counted from 0.  `far` = (a, b), float32 per head: s -= a[h] ln(1 + b[h] (position - key)).
+    positions, counted from 0.  `far` = (a, b), float32 per head: s -= a[h] ln(1 + b[h] (position - key)); with b
+    None, s -= a[h] (position - key).
     `keep_first`: with a window, the sequence's first so many positions stay in sight of every later token.
     `bias` float32 `[heads][n]`: s += bias[h][min(position - key, n - 1)]."""
     n_tok = positions.numel()
@@ -962,12 +1207,14 @@ def _kept_and_bias(what: str, keep_first, window, chunk, bias: Optional[torch.Te
 
 
 def _far_pair(what: str, far, n_heads: int):
-    """The two per-head vectors of the penalty on distance, checked; (None, None) without one."""
+    """The two per-head vectors of the penalty on distance (the second may be None: a penalty in proportion to the
+    distance), checked; (None, None) without one."""
     if far is None:
         return None, None
     a, b = far
     _need(a, what + ".far[0]", torch.float32, (n_heads,))
-    _need(b, what + ".far[1]", torch.float32, (n_heads,))
+    if b is not None:
+        _need(b, what + ".far[1]", torch.float32, (n_heads,))
     return a, b
 
 
@@ -1997,6 +2244,36 @@ def probe_mfma(rounds: int, blocks: Optional[int] = None, device="cuda") -> floa
     sink = workspace("probe", blocks, device)
     _check(_fn("probe", "mf_probe_mfma")(int(rounds), _ptr(sink), blocks, _stream()), "probe_mfma")
     return float(blocks) * 8 * rounds * 8 * 2 * 32 * 32 * 16
+
+
+def moe_table(table: torch.Tensor, ids: torch.Tensor, rows: Optional[torch.Tensor], chosen: torch.Tensor,
+              weights: torch.Tensor, weight: float) -> None:
+    """chosen[t] = table[ids[rows[t]]] (`rows`: which of the step's tokens the t are; None: all, in order), every
+    weight `weight`.  `table` int32 `[vocab][top]`; its entries are the caller's to check."""
+    n_tok, top = chosen.shape
+    _need(table, "moe_table.table", torch.int32)
+    if table.dim() != 2 or table.shape[1] != top:
+        raise KernelError(f"moe_table: table {tuple(table.shape)} for {top} choices a token")
+    _need(ids, "moe_table.ids", torch.int32)
+    if rows is not None:
+        _need(rows, "moe_table.rows", torch.int32, (n_tok,))
+    elif ids.numel() != n_tok:
+        raise KernelError(f"moe_table: {ids.numel()} token ids for {n_tok} rows")
+    _need(chosen, "moe_table.chosen", torch.int32)
+    _need(weights, "moe_table.weights", torch.float32, (n_tok, top))
+    _check(_fn("moe", "mf_moe_table")(_ptr(table), _ptr(ids), _ptr(rows), _ptr(chosen), _ptr(weights), n_tok, top, table.shape[0],
+                                       float(weight), _stream()), "moe_table")
+
+
+def gated_expert_act(gu: torch.Tensor, out: torch.Tensor) -> None:
+    """out[t][f] = silu(gate) up sigmoid(z) from float32 rows gate `[F]` | up `[F]` | z | padding, F = out's columns."""
+    n_tok, F = out.shape
+    _need(gu, "gated_expert_act.gu", torch.float32)
+    if gu.shape[0] != n_tok or gu.shape[1] < 2 * F + 1:
+        raise KernelError(f"gated_expert_act: rows {tuple(gu.shape)} for {n_tok} tokens of {F} values")
+    _need(out, "gated_expert_act.out", _FLOATS, (n_tok, F))
+    _check(_fn("moe", "mf_gated_expert_act")(_ptr(gu), gu.shape[1], _ptr(out), _is_bf16(out), n_tok, F, _stream()),
+           "gated_expert_act")
 
 
 def moe_group(chosen: torch.Tensor, n_experts: int, rank: torch.Tensor, counts: torch.Tensor) -> None:

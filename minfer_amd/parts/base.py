@@ -75,6 +75,11 @@ class Norm(Part):
         if cast_out is not None:
             cast_out.copy_(h)
 
+    def join_normed(self, y: torch.Tensor, h: torch.Tensor, scale: float, cast_out: Optional[torch.Tensor] = None) -> None:
+        """h <- norm(scale h + y), for arrangements that norm the stream itself behind every branch (float32 rows
+        both); `cast_out` as in `add_normed`.  Norms with a kernel for it provide this."""
+        raise NotImplementedError(f"{type(self).__name__} does not norm a scaled sum")
+
 
 @dataclass
 class NormAhead:

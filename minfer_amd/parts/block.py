@@ -87,11 +87,14 @@ class BranchNormBlock(Block):
         ops.convert(h, x)
         return x
 
+    def _norm_into(self, norm, y, h, copy) -> None:
+        norm.add_normed(y, h, cast_out=copy)
+
     def _join(self, norm, y, h, ctx, want_copy: bool):
         copy = None
         if want_copy and self.rt.dtype == torch.bfloat16:
             copy = torch.empty(h.shape, dtype=torch.bfloat16, device=h.device)
-        norm.add_normed(y, h, cast_out=copy)
+        self._norm_into(norm, y, h, copy)
         ctx.stream_copy = None if copy is None else (h, copy)
 
     @staticmethod
@@ -118,6 +121,21 @@ class BranchNormBlock(Block):
             y = self._run(self.feed_forward, self._input(h, ctx), h.shape[0], h.shape[1], ctx)
             self._join(self.norms["feed_forward_out"], y, h, ctx, want_copy=keep_rows is None)
         return h
+
+
+@register_block("postnorm")
+class PostNormBlock(BranchNormBlock):
+    """h <- N1(a h + mixer(h)); h <- N2(a h + feed_forward(h)): the branches read the stream itself and the stream is
+    normed behind every sum; `stream_scale` is the a.  norms: "mixer_out" behind the mixer's sum, "feed_forward_out"
+    behind the feed-forward's; a block without one branch has neither that branch nor its norm.  The norm is one that
+    takes a scaled sum (`Norm.join_normed`), whose kernel also leaves the rounded stream the next branch reads."""
+
+    def __init__(self, mixer, feed_forward, norms, rt, stream_scale: float = 1.0):
+        super().__init__(mixer, feed_forward, norms, rt)
+        self.stream_scale = float(stream_scale)
+
+    def _norm_into(self, norm, y, h, copy) -> None:
+        norm.join_normed(y, h, self.stream_scale, cast_out=copy)
 
 
 @register_block("sandwich")

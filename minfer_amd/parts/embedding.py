@@ -15,11 +15,12 @@ from .linear import Linear
 
 @register_embedding("token_embedding")
 class TokenEmbedding(Embedding):
-    """params: name (tensor), vocab_size, hidden_size."""
+    """params: name (tensor), vocab_size, hidden_size, scale (of the rows, default 1)."""
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
         self.name = spec.params["name"]
+        self.scale = float(spec.params.get("scale", 1.0))
         self.vocab, self.hidden = int(spec.params["vocab_size"]), int(spec.params["hidden_size"])
         self.weight = None
 
@@ -33,7 +34,7 @@ class TokenEmbedding(Embedding):
         return self.weight
 
     def forward(self, token_ids, out, ctx=None) -> None:
-        ops.embed(self.weight, token_ids, out)
+        ops.embed(self.weight, token_ids, out, self.scale)
 
 
 @register_embedding("normed_token_embedding")
@@ -53,7 +54,7 @@ class NormedTokenEmbedding(TokenEmbedding):
         self.norm.load(get)
 
     def forward(self, token_ids, out, ctx=None) -> None:
-        ops.embed(self.weight, token_ids, out)
+        ops.embed(self.weight, token_ids, out, self.scale)
         self.norm.forward(out, out=out)       # in place, 32-bit rows
 
 
@@ -117,6 +118,8 @@ class TokenPositionEmbedding(TokenEmbedding):
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
+        if self.scale != 1.0:
+            raise ValueError("token_position_embedding: the rows are not scaled")
         self.pos_name, self.max_positions = spec.params["positions"], int(spec.params["max_positions"])
         self.pos = None
 

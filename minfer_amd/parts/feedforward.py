@@ -128,6 +128,10 @@ class DenseGelu(FeedForward):
     """down(gelu(up x)) without biases, gelu in its tanh form, from the up product's 32-bit sums and
     rounded once.  params: hidden_size, intermediate_size, up, down (tensor names)."""
 
+    @staticmethod
+    def activation(u, y):
+        ops.gelu_tanh(u, y)
+
     takes_normed = True
     can_overwrite = True
 
@@ -151,5 +155,15 @@ class DenseGelu(FeedForward):
     def forward(self, x, h, ctx, accumulate: bool = True) -> None:
         u = self.up(x, out_dtype=torch.float32)
         y = torch.empty((u.shape[0], self.inter), dtype=self.rt.dtype, device=u.device)
-        ops.gelu_tanh(u, y)
+        self.activation(u, y)
         self.down(y, out=h, accumulate=accumulate)
+
+
+@register_feed_forward("dense_relu2")
+class DenseRelu2(DenseGelu):
+    """down(relu(up x)^2) without biases, from the up product's 32-bit sums and rounded once.  params: hidden_size,
+    intermediate_size, up, down (tensor names)."""
+
+    @staticmethod
+    def activation(u, y):
+        ops.relu2(u, y)

@@ -1,4 +1,5 @@
-"""Mixture-of-experts feed-forward with a router that first keeps the best groups of experts.
+"""Mixture-of-experts feed-forwards: with a router that first keeps the best groups of experts, or with a table in
+the router's place; and an expert that every token takes besides, where a design has one.
 
 Router: z = Wr x in 32-bit, scores = softmax(z) over all experts; the experts form `groups` equal
 groups of neighbours, a group's score is its best expert's, and only experts of the `keep` best groups
@@ -11,22 +12,30 @@ Expert (no biases): g = min(Wg x, limit), u = clamp(Wu x, -limit, limit), y = g 
 output Wd y; or, with `act` "silu", the plain gated form y = silu(Wg x) (Wu x).  The result is the weighted sum
 of the chosen experts' outputs.
 
+Table: the token's id picks its experts from a table `[vocab][top]` of expert numbers, each weighing 1 / top; the
+stream plays no part in the choice, so the host knows it too and a prompt's step waits for nothing.
+
+Shared expert: silu(Wg x) (Wu x) times one number per token, sigmoid(w x), then Wd; added to the chosen experts'
+sum.  The gate, the up matrix and w are one product.
+
 Two forms, both of which read or multiply only what was chosen.  Steps of few tokens and decode steps (which
 may be captured, so nothing may wait for the host): `ops.moe_sparse`, up to 16 tokens a launch, reads every
 chosen expert's matrices once.  Steps of many tokens: the (token, choice) pairs are grouped by expert
 (`ops.moe_group`; the host reads the experts' counts, the one wait of the step), the tokens' rows are put side by
 side expert by expert, every expert with tokens runs its two products over its rows, and the rows' results are
-added into the stream with the tokens' weights, a token's choices in their order.
+added into the stream with the tokens' weights, a token's choices in their order.  (With a table nothing waits:
+the host counts the experts' pairs itself.)
 
 A step whose context carries a list under `_memo["route_log"]` gets every routed layer's choices
 (`[rows][top]` expert numbers, on the device) appended to it, in run order.
 """
 from __future__ import annotations
 
+import numpy as np
 import torch
 
 from ..kernels import ops
-from ..weights.loader import TensorSpec
+from ..weights.loader import TensorSpec, WeightError
 from .base import FeedForward, register_feed_forward
 from .linear import Linear
 
@@ -34,13 +43,44 @@ from .linear import Linear
 SPARSE_UP_TO = ops.MOE_SPARSE_TOKENS
 
 
-@register_feed_forward("grouped_moe")
-class GroupedMoE(FeedForward):
-    """params: hidden_size, intermediate_size (of one expert), n_experts, top, groups and keep (default 1: no
-    groups), act ("clamped_swish", the default, with `limit`; or "silu"), router (tensor name), router_bias
-    (tensor name, or None), score ("softmax", the default, or "sigmoid"), correction (tensor name, or None),
-    group_top (default 1), weight_scale (default 1.0), expert (format of an expert's tensor stem, e.g. "mlp.e{}";
-    its matrices are stem + ".gate", ".up", ".down")."""
+class SharedExpert:
+    """The expert every token takes, weighed by a sigmoid of its own (plain silu form; widths of its own).
+    `spec`: dict(stem, weight, intermediate_size); the matrices are stem + ".gate", ".up", ".down"."""
+
+    PAD = 16        # the product's rows are filled up to a multiple of this
+
+    def __init__(self, spec, hidden: int, rt):
+        self.hidden, self.rt = hidden, rt
+        self.inter, self.stem, self.weight_name = int(spec["intermediate_size"]), spec["stem"], spec["weight"]
+        self.up = self.down = None
+
+    def tensor_specs(self):
+        return {self.stem + ".gate": TensorSpec((self.inter, self.hidden)), self.stem + ".up": TensorSpec((self.inter, self.hidden)),
+                self.stem + ".down": TensorSpec((self.hidden, self.inter)), self.weight_name: TensorSpec((1, self.hidden))}
+
+    def load(self, get):
+        rows = [get(self.stem + ".gate"), get(self.stem + ".up"), get(self.weight_name)]
+        fill = -(2 * self.inter + 1) % self.PAD
+        if fill:
+            rows.append(torch.zeros((fill, self.hidden), dtype=rows[0].dtype, device=rows[0].device))
+        self.up = Linear.stacked(rows)
+        self.down = Linear(get(self.stem + ".down"))
+
+    def decode_copies(self, make: bool, min_row_length: int = 0) -> int:
+        return self.up.decode_copy(make, min_row_length) + self.down.decode_copy(make, min_row_length)
+
+    def forward(self, x, h, accumulate: bool) -> None:
+        gu = self.up(x, out_dtype=torch.float32)
+        y = torch.empty((x.shape[0], self.inter), dtype=self.rt.dtype, device=x.device)
+        ops.gated_expert_act(gu, y)
+        self.down(y, out=h, accumulate=accumulate)
+
+
+class Experts(FeedForward):
+    """The experts and their two forms; who takes which is a subclass's `choose`.  params: hidden_size,
+    intermediate_size (of one expert), n_experts, top, act ("clamped_swish", the default, with `limit`; or "silu"),
+    expert (format of an expert's tensor stem, e.g. "mlp.e{}"; its matrices are stem + ".gate", ".up", ".down"),
+    shared (None, or dict(stem, weight, intermediate_size): the expert every token takes)."""
 
     can_overwrite = True
 
@@ -49,65 +89,61 @@ class GroupedMoE(FeedForward):
         p = spec.params
         self.hidden, self.inter, self.ne, self.top = (
             int(p[k]) for k in ("hidden_size", "intermediate_size", "n_experts", "top"))
-        self.groups, self.keep = int(p.get("groups", 1)), int(p.get("keep", p.get("groups", 1)))
         act = p.get("act", "clamped_swish")
         if act not in ops.MOE_ACTS:
-            raise ValueError(f"grouped_moe: activation {act!r} is not one of {sorted(ops.MOE_ACTS)}")
+            raise ValueError(f"{spec.kind}: activation {act!r} is not one of {sorted(ops.MOE_ACTS)}")
         self.act = ops.MOE_ACTS[act]
         self.limit = float(p["limit"]) if act == "clamped_swish" else 0.0
-        self.router_name, self.expert_name = p["router"], p["expert"]
-        self.bias_name = p.get("router_bias")
-        self.correction_name = p.get("correction")
-        self.score, self.group_top = p.get("score", "softmax"), int(p.get("group_top", 1))
-        self.weight_scale = float(p.get("weight_scale", 1.0))
-        if self.score not in ops.MOE_SCORES or self.group_top < 1:
-            raise ValueError(f"grouped_moe: scores {self.score!r} (one of {sorted(ops.MOE_SCORES)}), group_top {self.group_top}")
-        per = self.ne // max(1, self.groups)
-        if self.ne % self.groups or not 1 <= self.keep <= self.groups or not 1 <= self.top <= min(64, self.keep * per) \
-                or self.ne > ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"grouped_moe: {self.ne} experts in {self.groups} groups, {self.keep} kept, {self.top} chosen")
-        self.router = self.router_bias = self.correction = self.gate_up = self.down = None
+        self.expert_name = p["expert"]
+        self.shared = None if p.get("shared") is None else SharedExpert(p["shared"], self.hidden, rt)
+        if not 1 <= self.top <= min(64, self.ne) or self.ne > ops.MOE_MAX_EXPERTS:
+            raise ValueError(f"{spec.kind}: {self.top} of {self.ne} experts chosen (at most 64 of at most {ops.MOE_MAX_EXPERTS})")
+        self.gate_up = self.down = None
 
     def tensor_specs(self):
-        s = {self.router_name: TensorSpec((self.ne, self.hidden))}
-        if self.bias_name is not None:
-            s[self.bias_name] = TensorSpec((self.ne,))
-        if self.correction_name is not None:
-            s[self.correction_name] = TensorSpec((self.ne,))
+        s = {}
         for e in range(self.ne):
             stem = self.expert_name.format(e)
             s[stem + ".gate"] = TensorSpec((self.inter, self.hidden))
             s[stem + ".up"] = TensorSpec((self.inter, self.hidden))
             s[stem + ".down"] = TensorSpec((self.hidden, self.inter))
+        if self.shared is not None:
+            s.update(self.shared.tensor_specs())
         return s
 
     def load(self, get):
-        self.router = get(self.router_name).to(torch.float32).contiguous()   # the router's product is 32-bit
-        if self.bias_name is not None:
-            self.router_bias = get(self.bias_name).to(torch.float32).contiguous()
-        if self.correction_name is not None:
-            self.correction = get(self.correction_name).to(torch.float32).contiguous()
         stems = [self.expert_name.format(e) for e in range(self.ne)]
         # [experts][gate | up][hidden] and [experts][hidden][inter]: an expert's matrices are contiguous slices
         self.gate_up = torch.stack([torch.cat([get(s + ".gate"), get(s + ".up")], dim=0) for s in stems]).contiguous()
         self.down = torch.stack([get(s + ".down") for s in stems]).contiguous()
         self.experts = [(Linear(self.gate_up[e]), Linear(self.down[e])) for e in range(self.ne)]
+        if self.shared is not None:
+            self.shared.load(get)
 
     def decode_copies(self, make: bool, min_row_length: int = 0) -> int:
-        return 0
+        return 0 if self.shared is None else self.shared.decode_copies(make, min_row_length)
+
+    def choose(self, x, ctx, chosen: torch.Tensor, weights: torch.Tensor) -> None:
+        """Fills `chosen` (int32) and `weights` (float32), `[rows][top]`, for the rows x."""
+        raise NotImplementedError
+
+    def host_counts(self, ctx):
+        """How many of the rows' choices fall on each expert, where the host knows it without waiting, else None."""
+        return None
 
     def forward(self, x, h, ctx, accumulate: bool = True) -> None:
         n, dev = x.shape[0], x.device
         chosen = torch.empty((n, self.top), dtype=torch.int32, device=dev)
         weights = torch.empty((n, self.top), dtype=torch.float32, device=dev)
-        ops.moe_route(x, self.router, None, chosen, weights, self.groups, self.keep, bias=self.router_bias,
-                      score=self.score, correction=self.correction, group_top=self.group_top,
-                      weight_scale=self.weight_scale)
+        self.choose(x, ctx, chosen, weights)
         log = ctx._memo.get("route_log") if ctx is not None else None
         if log is not None:                  # a caller that wants to know: every routed layer's choices, in run order
             log.append(chosen)
         if n == 0:
             return
+        if self.shared is not None:
+            self.shared.forward(x, h, accumulate)
+            accumulate = True
         few = min(SPARSE_UP_TO, max(1, ops.MOE_SPARSE_PAIRS // self.top))
         if (n <= few or (ctx is not None and ctx.all_decode)) and x.dtype == self.gate_up.dtype:
             if not accumulate:
@@ -119,11 +155,14 @@ class GroupedMoE(FeedForward):
         rank = torch.empty_like(chosen)
         counts = torch.empty(self.ne, dtype=torch.int32, device=dev)
         ops.moe_group(chosen, self.ne, rank, counts)
-        per_expert = [int(c) for c in counts.cpu()]          # the step waits for the host here
+        per_expert = self.host_counts(ctx)
+        if per_expert is None:
+            per_expert = [int(c) for c in counts.cpu()]      # the step waits for the host here
         starts = [0]
         for c in per_expert:
             starts.append(starts[-1] + c)
-        offsets = torch.tensor(starts[:-1], dtype=torch.int32).to(dev)
+        # from pinned memory the copy does not wait for what the stream still has to do
+        offsets = torch.tensor(starts[:-1], dtype=torch.int32, pin_memory=dev.type == "cuda").to(dev, non_blocking=True)
         pairs = n * self.top
         xs = torch.empty((pairs, self.hidden), dtype=x.dtype, device=dev)
         ops.moe_gather(x, chosen, rank, offsets, xs)
@@ -145,3 +184,81 @@ class GroupedMoE(FeedForward):
         if have is None or have.shape[0] < n:
             have = self._ones_buf = torch.ones((max(n, 4096), 1), dtype=torch.float32, device=dev)
         return have[:n]
+
+
+@register_feed_forward("grouped_moe")
+class GroupedMoE(Experts):
+    """params: those of `Experts`, and groups and keep (default 1: no groups), router (tensor name), router_bias
+    (tensor name, or None), score ("softmax", the default, or "sigmoid"), correction (tensor name, or None),
+    group_top (default 1), weight_scale (default 1.0)."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        p = spec.params
+        self.groups, self.keep = int(p.get("groups", 1)), int(p.get("keep", p.get("groups", 1)))
+        self.router_name = p["router"]
+        self.bias_name = p.get("router_bias")
+        self.correction_name = p.get("correction")
+        self.score, self.group_top = p.get("score", "softmax"), int(p.get("group_top", 1))
+        self.weight_scale = float(p.get("weight_scale", 1.0))
+        if self.score not in ops.MOE_SCORES or self.group_top < 1:
+            raise ValueError(f"grouped_moe: scores {self.score!r} (one of {sorted(ops.MOE_SCORES)}), group_top {self.group_top}")
+        per = self.ne // max(1, self.groups)
+        if self.ne % self.groups or not 1 <= self.keep <= self.groups or not self.top <= self.keep * per:
+            raise ValueError(f"grouped_moe: {self.ne} experts in {self.groups} groups, {self.keep} kept, {self.top} chosen")
+        self.router = self.router_bias = self.correction = None
+
+    def tensor_specs(self):
+        s = {self.router_name: TensorSpec((self.ne, self.hidden))}
+        if self.bias_name is not None:
+            s[self.bias_name] = TensorSpec((self.ne,))
+        if self.correction_name is not None:
+            s[self.correction_name] = TensorSpec((self.ne,))
+        s.update(super().tensor_specs())
+        return s
+
+    def load(self, get):
+        self.router = get(self.router_name).to(torch.float32).contiguous()   # the router's product is 32-bit
+        if self.bias_name is not None:
+            self.router_bias = get(self.bias_name).to(torch.float32).contiguous()
+        if self.correction_name is not None:
+            self.correction = get(self.correction_name).to(torch.float32).contiguous()
+        super().load(get)
+
+    def choose(self, x, ctx, chosen, weights) -> None:
+        ops.moe_route(x, self.router, None, chosen, weights, self.groups, self.keep, bias=self.router_bias,
+                      score=self.score, correction=self.correction, group_top=self.group_top,
+                      weight_scale=self.weight_scale)
+
+
+@register_feed_forward("table_moe")
+class TableMoE(Experts):
+    """Experts that a table picks by the token's id, each weighing 1 / top.  params: those of `Experts`, and table
+    (tensor name of int32 `[vocab_size][top]`), vocab_size."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.table_name, self.vocab = spec.params["table"], int(spec.params["vocab_size"])
+        self.table = self.host_table = None
+
+    def tensor_specs(self):
+        return dict(super().tensor_specs(), **{self.table_name: TensorSpec((self.vocab, self.top), below=self.ne)})
+
+    def load(self, get):
+        self.table = get(self.table_name).to(torch.int32).contiguous()
+        self.host_table = self.table.cpu().numpy()
+        ranked = np.sort(self.host_table, axis=1)
+        if ranked.size and (ranked.min() < 0 or ranked.max() >= self.ne):
+            raise WeightError(f"{self.table_name}: expert numbers {ranked.min()}..{ranked.max()}, the layer has {self.ne}")
+        if (ranked[:, 1:] == ranked[:, :-1]).any():
+            raise WeightError(f"{self.table_name}: a row names an expert twice")
+        super().load(get)
+
+    def choose(self, x, ctx, chosen, weights) -> None:
+        ops.moe_table(self.table, ctx.token_ids, ctx.kept_rows, chosen, weights, 1.0 / self.top)
+
+    def host_counts(self, ctx):
+        if ctx.host_tokens is None:
+            return None
+        tokens = ctx.host_tokens if ctx.kept_rows is None else ctx.host_tokens[ctx.host_rows]
+        return np.bincount(self.host_table[tokens].reshape(-1), minlength=self.ne).tolist()

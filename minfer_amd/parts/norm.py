@@ -103,3 +103,31 @@ class OffsetRMSNorm(GroupRMSNorm):
 
     def load(self, get):
         self.weight = (get(self.name).to(torch.float32) + 1.0).contiguous()
+
+
+@register_norm("layernorm")
+class LayerNorm(Norm):
+    """Layer norm without a bias: (x - mean) / sqrt(variance + eps) * w, the variance being the mean of the squared
+    deviations.  params: size, eps, weight (tensor name)."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.size, self.eps, self.name = int(spec.params["size"]), float(spec.params["eps"]), spec.params["weight"]
+        self.weight = None
+
+    def tensor_specs(self):
+        return {self.name: TensorSpec((self.size,), init="ones")}
+
+    def load(self, get):
+        self.weight = get(self.name).to(torch.float32).contiguous()
+
+    def forward(self, h, out: Optional[torch.Tensor] = None, row_idx: Optional[torch.Tensor] = None):
+        rows = h.shape[0] if row_idx is None else row_idx.numel()
+        if out is None:
+            out = torch.empty((rows, self.size), dtype=self.rt.dtype, device=h.device)
+        ops.layernorm(h, self.weight, self.eps, out, row_idx)
+        return out
+
+    def join_normed(self, y, h, scale: float, cast_out: Optional[torch.Tensor] = None) -> None:
+        """h <- norm(scale h + y) in one kernel; `cast_out` (bfloat16) also gets the new rows rounded."""
+        ops.layernorm_join(h, y, scale, self.weight, self.eps, cast_out)

@@ -16,9 +16,13 @@ Further parameters: no norm at all (`qk_norm` False); a rotation in halves inste
 served by the same order); with a window, the sequence's first `keep_first` positions, which stay in sight of
 every later token; a learned number per (bucket of the distance, head) that joins the scaled score, with the
 buckets of `distance_buckets`; and `shared_kv`: the layer has no key and value matrices and reads the keys and
-values another layer's run left in its cache entry (the run order gives it that entry, not written by it).
+values another layer's run left in its cache entry (the run order gives it that entry, not written by it);
+biases on all four projections; `row_norm`: q and k over the root mean square of the whole projection, all heads at
+once, with gains as long as the projections (no rotation then); a query temperature that grows with the position,
+q <- q (1 + coef ln(floor((p + 1) / every) + 1)); a cap on the scaled score, cap tanh(s / cap); a penalty in proportion
+to the distance, slopes[h] (i - j), behind the cap.
 
-The attention itself runs in the kernels of the capped attention (temperatures of one, no cap).
+The attention itself runs in the kernels of the capped attention (temperatures of one).
 """
 from __future__ import annotations
 
@@ -57,7 +61,10 @@ class NormedAttention(Mixer):
     None), values_from_keys, value_rotation (PartSpec of a rotation in pairs over v_dim values, or None), window,
     chunk (None or int each), distance (None, or the names of the penalty's two per-head tensors), out_scale,
     qk_norm (default True), keep_first (None or int; needs a window), distance_bias (None, or dict(table: tensor
-    name of `[rows][heads]`, rows, far)), shared_kv (default False), q, k, v, o, q_norm, k_norm (tensor names)."""
+    name of `[rows][heads]`, rows, far)), shared_kv (default False), biases (default False; a bias is its
+    projection's name + ".b"), row_norm (default False; q_norm and k_norm name the gains), q_temperature (None, or
+    dict(coef, every); needs row_norm), cap (None or a number), slopes (None, or one number per head), q, k, v, o,
+    q_norm, k_norm (tensor names)."""
 
     takes_normed = True
     can_overwrite = True
@@ -77,6 +84,20 @@ class NormedAttention(Mixer):
         self.keep_first = int(p.get("keep_first") or 0)
         self.bias_spec = p.get("distance_bias")
         self.shared_kv = bool(p.get("shared_kv", False))
+        self.biases, self.row_norm = bool(p.get("biases", False)), bool(p.get("row_norm", False))
+        self.q_temperature = None
+        if p.get("q_temperature") is not None:
+            self.q_temperature = (float(p["q_temperature"]["coef"]), int(p["q_temperature"]["every"]))
+        self.cap = float(p.get("cap") or 0.0)
+        self.slopes = p.get("slopes")
+        if self.row_norm and (self.gains or not self.normed or self.v_from_k or self.shared_kv or p.get("position") is not None
+                              or p.get("value_rotation") is not None):
+            raise ValueError("normed_attention: a norm over whole projections goes with keys and values of the layer's own "
+                             "and no rotation")
+        if self.q_temperature is not None and (not self.row_norm or self.q_temperature[1] < 1):
+            raise ValueError("normed_attention: a query temperature goes with row_norm and needs 'every' of at least 1")
+        if self.slopes is not None and (len(self.slopes) != self.nh or self.distance is not None):
+            raise ValueError(f"normed_attention: {len(self.slopes)} slopes for {self.nh} heads, or a second penalty on distance")
         if self.keep_first and (self.window is None or self.chunk is not None):
             raise ValueError("normed_attention: kept first positions go with a window (and no chunks)")
         if self.gains and not self.normed:
@@ -109,6 +130,10 @@ class NormedAttention(Mixer):
                                  "queries and keys, in halves (half_tables)")
         self.halves = self.position is not None and not hasattr(self.position, "pair_tables")
         self.qkv = self.o = self.q_gain = self.k_gain = self.far = self.ones = self.bias = None
+        self.bias_names = [n + ".b" for n in (self.names["q"], self.names["k"], self.names["v"], self.names["o"])] \
+            if self.biases else []
+        if self.biases and (self.shared_kv or self.v_from_k):
+            raise ValueError("normed_attention: biases go with keys and values of the layer's own")
 
     def tensor_specs(self):
         n = self.names
@@ -123,6 +148,11 @@ class NormedAttention(Mixer):
         if self.gains:
             s[n["q_norm"]] = TensorSpec((self.dim,), init="ones")
             s[n["k_norm"]] = TensorSpec((self.dim,), init="ones")
+        if self.row_norm:
+            s[n["q_norm"]] = TensorSpec((self.nh * self.dim,), init="ones")
+            s[n["k_norm"]] = TensorSpec((self.nk * self.dim,), init="ones")
+        for name, rows in zip(self.bias_names, (self.nh * self.dim, self.nk * self.dim, self.nk * self.vdim, self.hidden)):
+            s[name] = TensorSpec((rows,))
         if self.distance is not None:
             # random weights: positive numbers, or the logarithm has no value
             s[self.distance[0]] = TensorSpec((self.nh,), init="halves")
@@ -132,18 +162,21 @@ class NormedAttention(Mixer):
     def load(self, get):
         n = self.names
         self.qkv = Linear.stacked([get(n[k]) for k in (("q",) if self.shared_kv else ("q", "k") if self.v_from_k
-                                                       else ("q", "k", "v"))])
+                                                       else ("q", "k", "v"))],
+                                  [get(name) for name in self.bias_names[:3]] if self.biases else None)
         if self.bias_spec is not None:
             # the table by distance, a row a head: what the kernels look up
             table = get(self.bias_spec["table"]).to(torch.float32)
             rows = torch.tensor(self.bias_rows, dtype=torch.long, device=table.device)
             self.bias = table[rows].t().contiguous()
-        self.o = Linear(get(n["o"]))
-        if self.gains:
+        self.o = Linear(get(n["o"]), get(self.bias_names[3]) if self.biases else None)
+        if self.gains or self.row_norm:
             self.q_gain = get(n["q_norm"]).to(torch.float32).contiguous()
             self.k_gain = get(n["k_norm"]).to(torch.float32).contiguous()
         if self.distance is not None:
             self.far = tuple(get(name).to(torch.float32).contiguous() for name in self.distance)
+        if self.slopes is not None:
+            self.far = (torch.tensor([float(s) for s in self.slopes], dtype=torch.float32, device=self.o.weight.device), None)
         self.ones = torch.ones(self.nh, dtype=torch.float32, device=self.o.weight.device)
 
     def cache_request(self):
@@ -171,18 +204,22 @@ class NormedAttention(Mixer):
                                                   else self.position.pair_tables)(ctx.max_len)
         vrot = None if self.value_position is None else self.value_position.pair_tables(ctx.max_len)
         q = torch.empty((n, self.nh * self.dim), dtype=self.rt.dtype, device=dev)
-        ops.qk_norm_prep(qkv, self.q_gain, self.k_gain, self.eps, self.normed, ctx.seq_of_tok, ctx.positions, rot, vrot,
-                         self.v_from_k, table, q, kc, vc, self.nh, self.nk, self.dim, self.vdim, writes_cache,
-                         halves=self.halves, q_only=self.shared_kv)
+        if self.row_norm:
+            ops.qk_row_prep(qkv, self.q_gain, self.k_gain, self.eps, self.q_temperature, ctx.seq_of_tok, ctx.positions, table,
+                            q, kc, vc, self.nh, self.nk, self.dim, self.vdim, writes_cache)
+        else:
+            ops.qk_norm_prep(qkv, self.q_gain, self.k_gain, self.eps, self.normed, ctx.seq_of_tok, ctx.positions, rot, vrot,
+                             self.v_from_k, table, q, kc, vc, self.nh, self.nk, self.dim, self.vdim, writes_cache,
+                             halves=self.halves, q_only=self.shared_kv)
         o = torch.empty((n, self.nh * self.vdim), dtype=self.rt.dtype, device=dev)
         window = 0 if self.window is None else int(self.window)
         chunk = 0 if self.chunk is None else int(self.chunk)
         if ops.capped_mfma_takes(self.rt.dtype, self.dim, self.vdim):
             ops.capped_attn_prefill(q, kc, vc, table, ctx, self.ones, o, self.nh, self.nk, self.dim, self.vdim, self.scale,
-                                    0.0, window, chunk=chunk, far=self.far, keep_first=self.keep_first, bias=self.bias)
+                                    self.cap, window, chunk=chunk, far=self.far, keep_first=self.keep_first, bias=self.bias)
         else:
             ops.capped_attn(q, kc, vc, table, ctx.positions, ctx.seq_of_tok, self.ones, o, self.nh, self.nk, self.dim,
-                            self.vdim, self.scale, 0.0, window, ctx.max_len, chunk=chunk, far=self.far,
+                            self.vdim, self.scale, self.cap, window, ctx.max_len, chunk=chunk, far=self.far,
                             keep_first=self.keep_first, bias=self.bias)
         if vrot is not None or self.out_scale != 1.0:
             ops.unrotate(o, vrot, ctx.positions, self.nh, self.out_scale)

@@ -42,6 +42,7 @@ class BlockSpec:
     feed_forward_norm: Optional[PartSpec] = None
     norms: Mapping[str, PartSpec] = field(default_factory=dict)
     combiner: Optional[PartSpec] = None       # what goes on to the next block, where not the block's result itself
+    params: Mapping[str, Any] = field(default_factory=dict)       # constants of the arrangement itself
 
     def __post_init__(self):
         norms = dict(self.norms)

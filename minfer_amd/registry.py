@@ -50,6 +50,8 @@ def _register_builtin() -> None:
     register_architecture(nodutar.ARCHITECTURE, nodutar.NodutarConfig)
     from .config import katarax
     register_architecture(katarax.ARCHITECTURE, katarax.KataraxConfig)
+    from .config import rofizen
+    register_architecture(rofizen.ARCHITECTURE, rofizen.RofizenConfig)
 
 
 _register_builtin()

@@ -12,7 +12,7 @@ widens everything floating to float32 (exact for bfloat16 and float16).
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Dict, Tuple
+from typing import Dict, Optional, Tuple
 
 import torch
 
@@ -27,9 +27,11 @@ class WeightError(ValueError):
 class TensorSpec:
     """What a part expects of one tensor: its shape, and how random weights fill it
     ('normal': N(0, std) of the configuration; 'ones': norm gains; 'zeros': gains stored around
-    zero; 'halves': bounds that lie between 0 and 1)."""
+    zero; 'halves': bounds that lie between 0 and 1).  With `below` it is a table of integers from 0 to
+    below - 1 that differ within a row (random weights fill it so, whatever `init` says)."""
     shape: Tuple[int, ...]
     init: str = "normal"
+    below: Optional[int] = None
 
 
 def storage_dtype(stored: torch.dtype, run_dtype: torch.dtype) -> torch.dtype:
@@ -48,8 +50,10 @@ def check_against(expected: Dict[str, TensorSpec], found: Dict[str, Tuple[Tuple[
     shapes = sorted(f"{n}: expected {list(expected[n].shape)}, found {list(found[n][0])}"
                     for n in expected if n in found and tuple(found[n][0]) != tuple(expected[n].shape))
     dtypes = sorted(f"{n}: {found[n][1]}" for n in expected
-                    if n in found and not found[n][1].is_floating_point)
-    if not (missing or unexpected or shapes or dtypes):
+                    if n in found and expected[n].below is None and not found[n][1].is_floating_point)
+    floats = sorted(f"{n}: {found[n][1]}" for n in expected
+                    if n in found and expected[n].below is not None and found[n][1].is_floating_point)
+    if not (missing or unexpected or shapes or dtypes or floats):
         return
     lines = [f"weights in {where} do not match the model:"]
     if missing:
@@ -60,6 +64,8 @@ def check_against(expected: Dict[str, TensorSpec], found: Dict[str, Tuple[Tuple[
         lines.append(f"  wrong shapes ({len(shapes)}): " + "; ".join(shapes))
     if dtypes:
         lines.append(f"  not floating point ({len(dtypes)}): " + "; ".join(dtypes))
+    if floats:
+        lines.append(f"  not integers ({len(floats)}): " + "; ".join(floats))
     raise WeightError("\n".join(lines))
 
 

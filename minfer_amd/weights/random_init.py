@@ -17,6 +17,7 @@ import os
 import zlib
 from typing import Dict
 
+import numpy as np
 import torch
 
 from .loader import TensorSpec
@@ -29,10 +30,20 @@ def tensor_seed(seed: int, name: str) -> int:
     return ((int(seed) & 0xFFFFFFFF) << 32) ^ zlib.crc32(name.encode("utf-8"))
 
 
+def random_table(seed: int, name: str, spec: TensorSpec) -> torch.Tensor:
+    """An integer table, int32: every row runs on from a random number below `spec.below`, wrapping round, so that
+    its entries differ."""
+    rows, cols = spec.shape
+    first = np.random.default_rng(tensor_seed(seed, name)).integers(0, spec.below, size=(rows, 1))
+    return torch.from_numpy(((first + np.arange(cols)) % spec.below).astype(np.int32))
+
+
 def random_tensor(seed: int, name: str, spec: TensorSpec, std: float,
                   dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
     """One tensor on the host.  A float32 tensor holds the unrounded float values; a bfloat16
     tensor the same values rounded to nearest even."""
+    if spec.below is not None:
+        return random_table(seed, name, spec)
     if spec.init == "ones":
         return torch.ones(spec.shape, dtype=dtype)
     if spec.init == "zeros":
@@ -60,7 +71,7 @@ def write_random_model(folder: str, config, seed: int, dtype: torch.dtype = torc
     order = list(expected)
     write_safetensors(
         os.path.join(folder, "model.safetensors"),
-        [(n, tuple(expected[n].shape), dtype) for n in order],
+        [(n, tuple(expected[n].shape), dtype if expected[n].below is None else torch.int32) for n in order],
         lambda n: random_tensor(seed, n, expected[n], config.random_init_std(n), dtype),
         metadata={"format": "pt", "seed": str(seed)})
     return folder
