@@ -14,8 +14,8 @@ import torch
 PAGE = 64
 
 
-def embed(table, ids, out):
-    out.copy_(table[ids.long()].to(torch.float32))
+def embed(table, ids, out, scale=1.0):
+    out.copy_(table[ids.long()].to(torch.float32) * scale)
 
 
 def rmsnorm(x, weight, eps, out, row_idx=None, cols=None):
@@ -478,7 +478,8 @@ def capped_attn(q, kcache, vcache, page_table, positions, seq_of_tok, temp, out,
             if cap:
                 s = cap * torch.tanh(s / cap)
             if far is not None:
-                s = s - float(far[0][h]) * torch.log1p(float(far[1][h]) * (p - pos).double())
+                d = (p - pos).double()
+                s = s - float(far[0][h]) * (d if far[1] is None else torch.log1p(float(far[1][h]) * d))
             if bias is not None:
                 s = s + bias[h].double()[torch.clamp(p - pos, max=bias.shape[1] - 1)]
             out[i, h * v_dim:(h + 1) * v_dim] = (torch.softmax(s, dim=0) @ vals).to(out.dtype)
@@ -587,6 +588,124 @@ def unrotate(rows, value_tables, positions, n_heads, scale=1.0):
     rows.copy_((x * scale).reshape(t_all, -1).to(rows.dtype))
 
 
+# ------------------------------------------------------------------ layer norms behind scaled sums, normed pairs
+def layernorm_reference(u, weight, eps):
+    c = u - u.mean(dim=-1, keepdim=True)
+    return c / torch.sqrt((c * c).mean(dim=-1, keepdim=True) + eps) * weight.double()
+
+
+def layernorm(x, weight, eps, out, row_idx=None):
+    src = x if row_idx is None else x[row_idx.long()]
+    out.copy_(layernorm_reference(src.double(), weight, eps).to(out.dtype))
+
+
+def layernorm_join(h, y, alpha, weight, eps, cast_out=None):
+    h.copy_(layernorm_reference(alpha * h.double() + y.double(), weight, eps).float())
+    if cast_out is not None:
+        cast_out.copy_(h.to(cast_out.dtype))
+
+
+def rmsnorm_pair(a, wa, b, wb, eps, scale, out, accumulate=False):
+    y = scale * (rmsnorm_reference(a, wa, eps) + rmsnorm_reference(b, wb, eps))
+    out.copy_((y + out.double() if accumulate else y).float())
+
+
+def relu2(x, out):
+    out.copy_((torch.clamp(x.double(), min=0.0) ** 2).to(out.dtype))
+
+
+# ------------------------------------------------------------------ decays per token: low-rank gates, retention, memory
+def _heads(p, at, H, width):
+    return p[:, at:at + H * width].view(p.shape[0], H, width)
+
+
+def _walk(state_rows, keep, k, v, q, out, cu_seqlens, slot_ids):
+    """S_t = keep_t S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; keep [tokens][H][D or 1], state_rows [slots][H][D][V]."""
+    for b in range(slot_ids.numel()):
+        slot = int(slot_ids[b])
+        S = state_rows[slot].double()
+        for t in range(int(cu_seqlens[b]), int(cu_seqlens[b + 1])):
+            S = keep[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t]).reshape(-1).float()
+        state_rows[slot] = S.float()
+
+
+def low_rank_scan(proj, a2, bias, off_r, tau, q_scale, cu_seqlens, slot_ids, state, out, n_heads, dim, v_dim, chunks=None):
+    H, D, V = n_heads, dim, v_dim
+    p = proj.double()
+    z = p[:, off_r:off_r + a2.shape[1]] @ a2.double().T + bias.double()
+    keep = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(-1, H, D)
+    _walk(state, keep, _heads(p, H * D, H, D), _heads(p, 2 * H * D, H, V), _heads(p, 0, H, D) * q_scale, out, cu_seqlens, slot_ids)
+
+
+def retention_scan(proj, cu_seqlens, slot_ids, decays, tables, positions, q_scale, k_scale, state, out, n_heads, dim, v_dim,
+                   chunks=None):
+    H, D, V = n_heads, dim, v_dim
+    p = proj.double()
+    q, k = _heads(p, 0, H, D), _heads(p, H * D, H, D)
+    if tables is not None:
+        c, s = (t[positions.long()].double()[:, None, :] for t in tables)
+        q, k = _rotate_half_part(q, c, s), _rotate_half_part(k, c, s)
+    keep = decays.double()[None, :, None].expand(p.shape[0], H, 1)
+    _walk(state, keep, k * k_scale, _heads(p, 2 * H * D, H, V), q * q_scale, out, cu_seqlens, slot_ids)
+
+
+def memory_scan(proj, off_i, off_f, cap, q_scale, cu_seqlens, slot_ids, state, out, den, floor, n_heads, dim, v_dim, chunks=None):
+    H, D, V = n_heads, dim, v_dim
+    p = proj.double()
+    q, k, v = _heads(p, 0, H, D) * q_scale, _heads(p, H * D, H, D), _heads(p, 2 * H * D, H, V)
+    gate_i = cap * torch.tanh(p[:, off_i:off_i + H] / cap)
+    gate_f = torch.nn.functional.logsigmoid(cap * torch.tanh(p[:, off_f:off_f + H] / cap))
+    for b in range(slot_ids.numel()):
+        row = state[int(slot_ids[b])]
+        S, n, m = (row[:H * D * V].double().view(H, D, V), row[H * D * V:H * D * (V + 1)].double().view(H, D), row[H * D * (V + 1):].double())
+        for t in range(int(cu_seqlens[b]), int(cu_seqlens[b + 1])):
+            top = torch.maximum(gate_f[t] + m, gate_i[t])
+            keep, take = torch.exp(gate_f[t] + m - top), torch.exp(gate_i[t] - top)
+            S = keep[:, None, None] * S + take[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+            n = keep[:, None] * n + take[:, None] * k[t]
+            m = top
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t]).reshape(-1).float()
+            den[t] = (n * q[t]).sum(dim=-1).float()
+            floor[t] = torch.exp(-m).float()
+        state[int(slot_ids[b])] = torch.cat([S.reshape(-1), n.reshape(-1), m]).float()
+
+
+def gated_head_norm(o, proj, gate_offset, weight, eps, out, n_heads, act, den=None, floor=None):
+    rows, n = o.shape
+    u = o.double().view(rows, n_heads, -1)
+    if den is not None:
+        u = u / (torch.maximum(den.double().abs(), floor.double()) + 1e-6)[:, :, None]
+    u = u / torch.sqrt((u * u).mean(dim=-1, keepdim=True) + eps)
+    if weight is not None:
+        u = u * weight.double().view(-1, u.shape[-1])
+    g = proj[:, gate_offset:gate_offset + n].double()
+    out.copy_((u.reshape(rows, n) * torch.sigmoid(g) * (g if act == "silu" else 1.0)).to(out.dtype))
+
+
+# ------------------------------------------------------------------ queries and keys normed over whole projections
+def qk_row_prep(qkv, q_gain, k_gain, eps, temperature, seq_of_tok, positions, page_table, q_out, kcache, vcache, n_heads,
+                n_kv_heads, dim, v_dim, write_cache=True):
+    y = qkv.double()
+    nq, nk = n_heads * dim, n_kv_heads * dim
+    q = rmsnorm_reference(y[:, :nq], q_gain, eps)
+    k = rmsnorm_reference(y[:, nq:nq + nk], k_gain, eps).view(-1, n_kv_heads, dim)
+    v = y[:, nq + nk:].reshape(-1, n_kv_heads, v_dim)
+    if temperature is not None:
+        coef, every = temperature
+        q = q * (1.0 + coef * torch.log(torch.div(positions.long() + 1, every, rounding_mode="floor").double() + 1.0))[:, None]
+    q_out.copy_(q.to(q_out.dtype))
+    if not write_cache:
+        return
+    for i in range(positions.numel()):
+        p = int(positions[i])
+        page = int(page_table[int(seq_of_tok[i]), p // PAGE])
+        assert page >= 0
+        kcache[page, :, p % PAGE] = k[i].to(kcache.dtype)
+        for g in range(n_kv_heads):
+            _store_v(vcache, page, p % PAGE, g, v[i, g])
+
+
 # ------------------------------------------------------------------ mixture of experts
 MOE_MAX_EXPERTS = 1024
 MOE_SPARSE_TOKENS, MOE_SPARSE_PAIRS = 16, 128
@@ -651,6 +770,18 @@ def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0):
             e = int(chosen[t, k])
             y = _expert_act(gu[e, 0] @ x[t].double(), gu[e, 1] @ x[t].double(), limit, act).to(x.dtype).double()
             out[t] += (float(weights[t, k]) * (dn[e] @ y)).float()
+
+
+def moe_table(table, ids, rows, chosen, weights, weight):
+    picked = ids.long() if rows is None else ids.long()[rows.long()]
+    chosen.copy_(table[picked])
+    weights.fill_(weight)
+
+
+def gated_expert_act(gu, out):
+    F = out.shape[1]
+    g, u, z = gu[:, :F].double(), gu[:, F:2 * F].double(), gu[:, 2 * F:2 * F + 1].double()
+    out.copy_((g * torch.sigmoid(g) * u * torch.sigmoid(z)).to(out.dtype))
 
 
 def moe_group(chosen, n_experts, rank, counts):
@@ -754,7 +885,9 @@ NAMES = ["embed", "rmsnorm", "gather_rows", "swiglu", "convert", "fill_normal", 
          "headwise_linear", "latent_attn", "headwise_mfma_takes", "headwise_linear_mfma",
          "embed_pos", "gelu_tanh", "weighted_sum", "lightning_scan", "gated_rmsnorm", "rope_half_inplace",
          "qkv_conv_prep", "capped_attn", "capped_mfma_takes", "capped_attn_prefill", "moe_route", "moe_act", "moe_sparse", "moe_group", "moe_gather", "moe_combine",
-         "add_rows", "gr_chunks", "gated_scan", "head_rmsnorm", "qk_norm_prep", "unrotate", "softcap"]
+         "add_rows", "gr_chunks", "gated_scan", "head_rmsnorm", "qk_norm_prep", "unrotate", "softcap",
+         "layernorm", "layernorm_join", "rmsnorm_pair", "relu2", "low_rank_scan", "retention_scan", "memory_scan",
+         "gated_head_norm", "qk_row_prep", "moe_table", "gated_expert_act"]
 
 
 def install(monkeypatch):
