@@ -1,0 +1,559 @@
+"""Rofizen on the GPU: each new or extended kernel alone against the plain stand-ins, slopes and temperatures by hand,
+far keys, carried states, the engine against the plain implementation under every way of cutting requests into
+steps, long decoding through the captured step, and the programs."""
+import copy
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+import plain_ops
+import plain_rofizen as pr
+from paged_cases import DEV, attention_case, pages, rnd, step_context
+from replays import batch_steps, chunk_steps, requests_for, run_steps, tail_steps, whole_steps
+from rofizen_tiny import RZ, RZ_B, dense, gla, left, moe, parallel, random_config, retention, right, write_rofizen
+from tiny import random_tokens
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+# bfloat16 logits against the 64-bit plain implementation, as fractions of the logits' standard deviation, at three
+# layers and growing with the root of their number beyond; 32-bit in absolute terms (times the logits' standard
+# deviation where that is above one)
+BF16_RMS, BF16_MAX, F32_ABS = 0.04, 0.2, 2e-4
+SHARP = 3.0
+# every head's result is brought to a root mean square of one without a floor worth the name, and so is its rounding
+# error where the head's sums all but cancel: the host stand-ins, which round where the kernels round and compute in 64
+# bits in between, differ from the plain implementation by 0.3 to 0.6 % rms at the median position and by up to 15 % at
+# one in some hundreds (the GPU by the same).  So in bfloat16 a few positions of a replay may lie beyond the bounds,
+# and the median has to lie well inside
+BF16_FEW, BF16_MEDIAN = 0.02, 0.5
+
+
+def check(engine, steps, plain, reqs, dtype, what, loosen=1.0, f32_abs=F32_ABS, ref=None):
+    loosen = loosen * max(1.0, len(plain.cfg["layers"]) / 3.0) ** 0.5
+    rows = run_steps(engine, steps)
+    assert rows, "nothing was produced"
+    ref = {} if ref is None else ref
+    ratios = {}
+    for (rid, p), got in sorted(rows.items()):
+        if rid not in ref:
+            ref[rid] = plain.forward(reqs[rid])
+        want = ref[rid][p]
+        assert np.isfinite(got).all(), f"{what} [{dtype}]: non-finite logits at request {rid} position {p}"
+        diff = got.astype(np.float64) - want
+        if dtype == "float32":
+            assert np.abs(diff).max() <= f32_abs * max(1.0, want.std()), \
+                f"{what} [float32]: request {rid} position {p} of {len(reqs[rid])}: {np.abs(diff).max():.3e}"
+        else:
+            rms = float(np.sqrt(np.mean(diff * diff)))
+            ratios[(rid, p)] = max(rms / BF16_RMS, np.abs(diff).max() / BF16_MAX) / (loosen * float(want.std()))
+    if ratios:
+        over = {k: round(float(v), 2) for k, v in ratios.items() if v > 1.0}
+        assert len(over) <= max(1, BF16_FEW * len(ratios)), f"{what} [bfloat16]: beyond the bounds by a factor of {over}"
+        assert np.median(list(ratios.values())) <= BF16_MEDIAN, f"{what} [bfloat16]: median {np.median(list(ratios.values())):.2f} of the bounds"
+
+
+# ------------------------------------------------------------------ kernels alone
+@pytest.mark.parametrize("rows, d", [(1, 1), (3, 30), (5, 62), (4, 96), (7, 1024), (3, 1028), (2, 2048), (2, 4096), (3, 8192), (2, 8196), (2, 3001)])
+def test_layer_norms_normed_pairs_and_the_square_of_relu(rows, d):
+    from minfer_amd.kernels import ops
+    x, y, w, v = rnd(rows, d, seed=1, scale=3.0) + 2.0, rnd(rows, d, seed=2), rnd(d, seed=3), rnd(d, seed=4)
+    idx = torch.tensor([rows - 1, 0], dtype=torch.int32)
+    for dt in (torch.float32, torch.bfloat16):
+        tol = 2e-5 if dt == torch.float32 else 2e-2
+        want, got = torch.empty(rows, d, dtype=dt), torch.empty(rows, d, dtype=dt, device=DEV)
+        plain_ops.layernorm(x, w, 1e-5, want)
+        ops.layernorm(x.to(DEV), w.to(DEV), 1e-5, got)
+        assert ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max() < tol
+        want, got = torch.empty(2, d, dtype=dt), torch.empty(2, d, dtype=dt, device=DEV)
+        plain_ops.layernorm(x, w, 1e-5, want, idx)
+        ops.layernorm(x.to(DEV), w.to(DEV), 1e-5, got, idx.to(DEV))
+        assert ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max() < tol
+        want, got = torch.empty(rows, d, dtype=dt), torch.empty(rows, d, dtype=dt, device=DEV)
+        plain_ops.relu2(x, want)
+        ops.relu2(x.to(DEV), got)
+        assert ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max() < tol
+    for cast in (False, True):
+        h, hg = x.clone(), x.to(DEV)
+        c = torch.empty(rows, d, dtype=torch.bfloat16) if cast else None
+        cg = torch.empty(rows, d, dtype=torch.bfloat16, device=DEV) if cast else None
+        plain_ops.layernorm_join(h, y, 1.7, w, 1e-5, c)
+        ops.layernorm_join(hg, y.to(DEV), 1.7, w.to(DEV), 1e-5, cg)
+        assert (hg.cpu() - h).abs().max() < 3e-5
+        if cast:
+            assert torch.equal(cg, hg.to(torch.bfloat16))
+    for acc in (False, True):
+        out = rnd(rows, d, seed=7)
+        og = out.to(DEV)
+        plain_ops.rmsnorm_pair(x, w, y, v, 1e-5, 0.5, out, acc)
+        ops.rmsnorm_pair(x.to(DEV), w.to(DEV), y.to(DEV), v.to(DEV), 1e-5, 0.5, og, acc)
+        assert (og.cpu() - out).abs().max() < 3e-5
+
+
+def test_a_scaled_embedding():
+    from minfer_amd.kernels import ops
+    table, ids = rnd(50, 33, seed=1).to(torch.bfloat16), torch.tensor([3, 49, 0, 3], dtype=torch.int32)
+    got = torch.empty(4, 33, device=DEV)
+    ops.embed(table.to(DEV), ids.to(DEV), got, 13.3)
+    assert torch.equal(got.cpu(), table[ids.long()].float() * torch.tensor(13.3))
+
+
+def _chunks(kind, new):
+    from minfer_amd.kernels import ops
+    table, count = (ops.gr_chunks if kind == "gla" else ops.la_chunks)(new)
+    return table.to(DEV), count
+
+
+def _scan_case(new, extra, H, D, V, seed, state_len):
+    """Rows q | k | v | `extra` columns for sequences in the slots 3, 0, 5, ... of nine; states that are not zero."""
+    slots = torch.tensor([3, 0, 5, 7, 1][:len(new)], dtype=torch.int32)
+    cu = torch.tensor([0] + list(np.cumsum(new)), dtype=torch.int32)
+    return rnd(sum(new), H * (2 * D + V) + extra, seed=seed), slots, cu, rnd(9, *state_len, seed=seed + 1)
+
+
+def _compare_scan(run, proj, state, outs, chunked_tol):
+    """`run(ops module, tensors..., outs, chunked)` on the host and on the GPU in both forms; slots that are not in
+    the step stay as they were."""
+    from minfer_amd.kernels import ops
+    want_state, want = state.clone(), [torch.zeros(s) for s in outs]
+    run(plain_ops, proj.clone(), want_state, want, False)
+    for chunked in (False, True):
+        got_state, got = state.to(DEV), [torch.full(s, float("nan"), device=DEV) for s in outs]
+        run(ops, proj.to(DEV), got_state, got, chunked)
+        for i, (a, b) in enumerate(zip(got, want)):
+            err = ((a.cpu() - b).abs() / b.abs().clamp(min=1.0)).max()
+            assert err < chunked_tol, f"output {i}, chunked {chunked}: {float(err):.3e}"
+        err = ((got_state.cpu() - want_state).abs() / want_state.abs().clamp(min=1.0)).max()
+        assert err < chunked_tol, f"state, chunked {chunked}: {float(err):.3e}"
+
+
+NEW = [(1,), (5, 64, 1), (70, 3, 128, 200), (1, 1, 1, 1, 1), (65, 63)]
+
+
+@pytest.mark.parametrize("H, D, V, rank, tau", [(3, 16, 48, 5, 8.0), (1, 9, 70, 3, 1.0), (2, 128, 64, 16, 16.0), (2, 132, 20, 1, 0.5), (5, 32, 64, 70, 4.0)])
+@pytest.mark.parametrize("new", NEW)
+def test_gated_linear_attention_scan(H, D, V, rank, tau, new):
+    """Decays from near 0 to near 1 (biases from -6 to 6), carried states, walks and chunks."""
+    proj, slots, cu, state = _scan_case(new, rank + 7, H, D, V, 3, (H, D, V))
+    a2, bias = rnd(H * D, rank, seed=5, scale=1.0 / rank ** 0.5), rnd(H * D, seed=6, scale=3.0)
+    off = H * (2 * D + V) + 4
+
+    def run(o, p, st, outs, chunked):
+        dev = p.device
+        o.low_rank_scan(p, a2.to(dev), bias.to(dev), off, tau, D ** -0.5, cu.to(dev), slots.to(dev), st, outs[0], H, D, V,
+                        _chunks("gla", new) if chunked else None)
+    _compare_scan(run, proj, state, [(sum(new), H * V)], 3e-5)
+
+
+@pytest.mark.parametrize("H, D, V, rot, decay", [(2, 40, 24, 16, (0.9, 0.995)), (3, 12, 7, 2, (1.0, 0.5, 0.97)), (1, 128, 64, 128, (0.99,)),
+                                                 (2, 130, 64, 30, (0.98, 0.2)), (4, 32, 100, 0, (0.9, 0.99, 0.999, 0.03125))])
+@pytest.mark.parametrize("new", NEW)
+def test_retention_scan(H, D, V, rot, decay, new):
+    """Sequences that stand at different positions when the step begins, rotations over part of a head, all of it, none."""
+    proj, slots, cu, state = _scan_case(new, 5, H, D, V, 13, (H, D, V))
+    pos = torch.cat([torch.arange(s, s + n) for s, n in zip((0, 100, 7, 250, 31), new)]).to(torch.int32)
+    tables = None
+    if rot:
+        ang = torch.arange(512, dtype=torch.float64)[:, None] * (100.0 ** (-2.0 * torch.arange(rot // 2) / rot))
+        tables = (torch.cos(ang).float(), torch.sin(ang).float())
+
+    def run(o, p, st, outs, chunked):
+        dev = p.device
+        o.retention_scan(p, cu.to(dev), slots.to(dev), torch.tensor(decay, device=dev), None if tables is None else tuple(t.to(dev) for t in tables),
+                         pos.to(dev), 1.0, D ** -0.5, st, outs[0], H, D, V, _chunks("la", new) if chunked else None)
+    _compare_scan(run, proj, state, [(sum(new), H * V)], 3e-5)
+
+
+@pytest.mark.parametrize("H, D, V, cap, shift", [(3, 24, 40, 5.0, 0.0), (1, 5, 11, 30.0, 3.0), (2, 128, 64, 12.0, -3.0), (2, 130, 66, 12.0, 0.0), (4, 32, 100, 1.5, 0.0),
+                                                 (2, 64, 64, 15.0, 8.0)])
+@pytest.mark.parametrize("new", NEW + [(1100, 40), (2, 1024, 1025)])
+def test_matrix_memory_scan(H, D, V, cap, shift, new):
+    """Gates that keep, that forget at once (`shift` moves both) and that swing from token to token; running maxima
+    that are carried over from other steps, on both sides of zero; more chunks than one round of the gates' kernel
+    takes."""
+    if sum(new) > 1000 and H * D * V > 10000:
+        pytest.skip("the stand-in walks every token on the host")
+    extra = 2 * H + 3
+    proj, slots, cu, state = _scan_case(new, extra, H, D, V, 23, (H * (D * V + D + 1),))
+    off = H * (2 * D + V) + 1
+    proj[:, off:] = proj[:, off:] * 4.0 + shift
+    state[:, -H:] *= 3.0
+    n = sum(new)
+
+    def run(o, p, st, outs, chunked):
+        dev = p.device
+        o.memory_scan(p, off, off + H + 1, cap, D ** -0.5, cu.to(dev), slots.to(dev), st, outs[0], outs[1], outs[2], H, D, V,
+                      _chunks("la", new) if chunked else None)
+    _compare_scan(run, proj, state, [(n, H * V), (n, H), (n, H)], 1e-4)
+
+
+def test_the_memory_remembers_a_token_among_a_thousand():
+    """Input gates far down but for one token, forget gates wide open: 900 tokens later the memory still answers with
+    that token's value, whether it came in the same step, in an earlier one, or is decoded upon."""
+    from minfer_amd.kernels import ops
+    H, D, V, n = 2, 32, 48, 900
+    proj = rnd(n, H * (2 * D + V) + 2 * H, seed=2)
+    off = H * (2 * D + V)
+    proj[:, off:off + H] = -9.0
+    proj[:, off + H:] = 9.5
+    proj[17, off:off + H] = 6.0
+    cu = lambda *m: torch.tensor([0] + list(np.cumsum(m)), dtype=torch.int32, device=DEV)
+    slots = torch.tensor([2], dtype=torch.int32, device=DEV)
+    want = proj[17, 2 * H * D:2 * H * D + H * V].view(H, V)
+    for cuts in ((n,), (18, n - 18), (500, 399, 1), (1, 16, 1, 882)):
+        state = torch.zeros(4, ops.memory_state_len(H, D, V), device=DEV)
+        at = 0
+        for m in cuts:
+            part = proj[at:at + m].contiguous().to(DEV)
+            out, den, floor = torch.empty(m, H * V, device=DEV), torch.empty(m, H, device=DEV), torch.empty(m, H, device=DEV)
+            ops.memory_scan(part, off, off + H, 20.0, 1.0, cu(m), slots, state, out, den, floor, H, D, V,
+                            _chunks("la", [m]) if m > 64 else None)
+            at += m
+        got = (out[-1].view(H, V) / den[-1][:, None]).cpu()
+        assert (got - want).abs().max() < 0.05, cuts
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H, V", [(1, 3), (3, 48), (6, 64), (5, 100), (2, 256)])
+def test_norm_per_head_with_gate(dtype, H, V):
+    from minfer_amd.kernels import ops
+    n = 9
+    o, proj = rnd(n, H * V, seed=1, scale=2.0), rnd(n, H * V + 11, seed=2, scale=3.0)
+    den, floor = rnd(n, H, seed=3), rnd(n, H, seed=4).abs()
+    den[0] = 0.0
+    floor[0] = 0.0
+    for weight in (None, rnd(V, seed=5), rnd(H * V, seed=6)):
+        for act in ("silu", "sigmoid"):
+            for d in (None, (den, floor)):
+                want, got = torch.empty(n, H * V, dtype=dtype), torch.empty(n, H * V, dtype=dtype, device=DEV)
+                kw = {} if d is None else dict(den=d[0], floor=d[1])
+                plain_ops.gated_head_norm(o, proj, 7, weight, 1e-5, want, H, act, **kw)
+                ops.gated_head_norm(o.to(DEV), proj.to(DEV), 7, None if weight is None else weight.to(DEV), 1e-5, got, H, act,
+                                    **{k: t.to(DEV) for k, t in kw.items()})
+                err = ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max()
+                assert err < (2e-5 if dtype == torch.float32 else 1e-2), (act, float(err))
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H, G, D, V, temp", [(6, 3, 32, 16, (0.7, 50)), (9, 1, 10, 6, None), (8, 8, 80, 144, (0.3, 1)), (2, 1, 130, 20, (2.0, 64))])
+def test_queries_and_keys_normed_over_their_whole_projections(dtype, H, G, D, V, temp):
+    from minfer_amd.cache.paged import v_page_shape
+    from minfer_amd.kernels import ops
+    held, new = (0, 3, 60, 127), (1, 2, 70, 5)
+    n = sum(new)
+    qkv = rnd(n, H * D + G * (D + V), seed=1, scale=2.0)
+    seq = torch.repeat_interleave(torch.arange(4, dtype=torch.int32), torch.tensor(new)).to(torch.int32)
+    pos = torch.cat([torch.arange(h, h + m) for h, m in zip(held, new)]).to(torch.int32)
+    table = pages([h + m for h, m in zip(held, new)], 7)
+    qg, kg = rnd(H * D, seed=2), rnd(G * D, seed=3)
+    for write in (True, False):
+        outs = []
+        for o, dev in ((plain_ops, "cpu"), (ops, DEV)):
+            kc = torch.full((40, G, 64, D), 7.0, dtype=dtype, device=dev)
+            vc = torch.full((40,) + v_page_shape(G, V, dtype), 7.0, dtype=dtype, device=dev)
+            q = torch.empty(n, H * D, dtype=dtype, device=dev)
+            o.qk_row_prep(qkv.to(dev), qg.to(dev), kg.to(dev), 1e-5, temp, seq.to(dev), pos.to(dev), table.to(dev), q, kc, vc, H, G, D, V, write)
+            outs.append([t.cpu().float() for t in (q, kc, vc)])
+        tol = 3e-5 if dtype == torch.float32 else 1e-2
+        for name, a, b in zip(("q", "k pages", "v pages"), *outs):
+            assert ((a - b).abs() / b.abs().clamp(min=1.0)).max() < tol, name
+        assert write or bool((outs[1][1] == 7.0).all() and (outs[1][2] == 7.0).all())
+
+
+def _attend(form, q, kc, vc, table, pos, seq, lens, new, H, G, D, V, scale, cap, far):
+    from minfer_amd.kernels import ops
+    if form == "stand-in":
+        out = torch.empty(sum(new), H * V, dtype=q.dtype)
+        plain_ops.capped_attn(q, kc, vc, table, pos, seq, torch.ones(H), out, H, G, D, V, scale, cap, 0, max(lens), far=far)
+        return out.float()
+    out = torch.empty(sum(new), H * V, dtype=q.dtype, device=DEV)
+    ones = torch.ones(H, device=DEV)
+    f = None if far is None else (far[0].to(DEV), None)
+    if form == "matrix cores":
+        ops.capped_attn_prefill(q.to(DEV), kc.to(DEV), vc.to(DEV), table.to(DEV), step_context(lens, new, table, pos, seq), ones,
+                                out, H, G, D, V, scale, cap, 0, far=f)
+    else:
+        ops.capped_attn(q.to(DEV), kc.to(DEV), vc.to(DEV), table.to(DEV), pos.to(DEV), seq.to(DEV), ones, out, H, G, D, V, scale,
+                        cap, 0, max(lens), far=f)
+    return out.float().cpu()
+
+
+_WANT = {}
+
+
+@pytest.mark.parametrize("form, dtype", [("plain", torch.float32), ("plain", torch.bfloat16), ("matrix cores", torch.bfloat16)])
+@pytest.mark.parametrize("H, G, D, V, cap", [(6, 3, 32, 48, 0.0), (8, 2, 96, 48, 3.0), (4, 4, 16, 16, 20.0), (9, 1, 10, 6, 2.0), (8, 8, 80, 144, 0.0)])
+@pytest.mark.parametrize("new", [(1, 130, 3, 1, 40), (1, 1, 1, 1, 1)])
+def test_slopes_by_distance_in_both_attention_kernels(form, dtype, H, G, D, V, cap, new):
+    if form == "matrix cores" and (D % 16 or V % 16):
+        pytest.skip("sizes the plain kernel takes")
+    lens = (1, 130, 64, 300, 65)
+    q, kc, vc, table, pos, seq, _ = attention_case(dtype, H, G, D, V, lens, new, 0, 0.0, 3)
+    far = (torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)]), None)
+    case = (dtype, H, G, D, V, cap, new)
+    if case not in _WANT:
+        _WANT[case] = _attend("stand-in", q, kc, vc, table, pos, seq, lens, new, H, G, D, V, 0.2, cap, far)
+    got = _attend(form, q, kc, vc, table, pos, seq, lens, new, H, G, D, V, 0.2, cap, far)
+    err = (got - _WANT[case]).abs().max()
+    assert torch.isfinite(got).all() and err < (2e-5 if dtype == torch.float32 else 4e-2), float(err)
+
+
+@pytest.mark.parametrize("form", ["plain float32", "plain bfloat16", "matrix cores"])
+@pytest.mark.parametrize("key", [299, 298, 256, 255, 192, 64, 63, 1, 0])
+def test_a_far_key_decides_against_the_slope(form, key):
+    """A key made to win the softmax, at a page's edges and up to 299 positions back: it decides for the head whose
+    slope it outweighs, at the end of a prompt, of a portion and for a single token."""
+    H, G, D, V = 4, 2, 16, 16
+    dtype = torch.float32 if form == "plain float32" else torch.bfloat16
+    far = (torch.tensor([0.002] * H), None)
+    for lens, new in (((300, 90), (300, 20)), ((300, 90), (45, 1)), ((300, 90), (1, 1))):
+        q, kc, vc, table, pos, seq, _ = attention_case(dtype, H, G, D, V, lens, new, 0, 0.0, 5, needle=(0, key, 1))
+        got = _attend("plain" if form.startswith("plain") else form, q, kc, vc, table, pos, seq, lens, new, H, G, D, V, 1.0, 0.0, far)
+        assert (got[new[0] - 1].view(H, V)[2:] - 50.0).abs().max() < 0.5, (lens, new)
+
+
+def test_the_slope_comes_behind_the_cap():
+    """Two equal keys with different values, one 1 and one 200 positions back, scores far above the cap: the farther
+    one weighs exp(-slope 199) of the nearer, whatever the cap."""
+    from minfer_amd.kernels import ops
+    H, G, D, V = 2, 1, 16, 16
+    table = pages((201,), 1)
+    kc, vc = torch.zeros(40, G, 64, D), torch.zeros(40, G, 64, V)
+    key = torch.zeros(D)
+    key[3] = 10.0
+    for p in range(201):
+        kc[int(table[0, p // 64]), 0, p % 64] = key if p in (0, 199) else -key
+        vc[int(table[0, p // 64]), 0, p % 64] = {0: 1.0, 199: 3.0}.get(p, 0.0)
+    q = torch.cat([key, key]).view(1, H * D)
+    slope = torch.tensor([0.004, 0.01])
+    pos, seq = torch.tensor([200], dtype=torch.int32), torch.tensor([0], dtype=torch.int32)
+    got = torch.empty(1, H * V, device=DEV)
+    ops.capped_attn(q.to(DEV), kc.to(DEV), vc.to(DEV), table.to(DEV), pos.to(DEV), seq.to(DEV), torch.ones(H, device=DEV), got,
+                    H, G, D, V, 1.0, 20.0, 0, 201, far=(slope.to(DEV), None))
+    for h in range(H):
+        ratio = float(torch.exp(-slope[h] * 199))
+        assert abs(float(got[0, h * V]) - (ratio * 1.0 + 3.0) / (ratio + 1.0)) < 1e-4, h
+
+
+def test_choices_from_a_table_and_the_shared_experts_activation():
+    from minfer_amd.kernels import ops
+    table = torch.stack([torch.randperm(7, generator=torch.Generator().manual_seed(i))[:3] for i in range(50)]).to(torch.int32)
+    ids = torch.tensor([3, 49, 0, 3, 7], dtype=torch.int32)
+    for rows in (None, torch.tensor([4, 1, 1], dtype=torch.int32)):
+        n = 5 if rows is None else 3
+        chosen, weights = torch.empty(n, 3, dtype=torch.int32, device=DEV), torch.empty(n, 3, device=DEV)
+        ops.moe_table(table.to(DEV), ids.to(DEV), None if rows is None else rows.to(DEV), chosen, weights, 1.0 / 3)
+        assert torch.equal(chosen.cpu(), table[(ids if rows is None else ids[rows.long()]).long()]) and bool((weights == 1.0 / 3).all())
+    for F, pad in ((8, 1), (33, 14), (700, 3)):
+        gu = rnd(6, 2 * F + pad, seed=F, scale=2.0)
+        for dt, tol in ((torch.float32, 1e-5), (torch.bfloat16, 1e-2)):
+            want, got = torch.empty(6, F, dtype=dt), torch.empty(6, F, dtype=dt, device=DEV)
+            plain_ops.gated_expert_act(gu, want)
+            ops.gated_expert_act(gu.to(DEV), got)
+            assert ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max() < tol
+
+
+# ------------------------------------------------------------------ the engine
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    tmp = tmp_path_factory.mktemp("rofizen")
+    return {name: write_rofizen(str(tmp / name), raw, seed=i) for i, (name, raw) in enumerate(RZ.items())}
+
+
+@pytest.fixture(scope="module")
+def plains(folders):
+    return {name: pr.PlainRofizen.from_folder(f) for name, f in folders.items()}
+
+
+def engine_for(folder, dtype, max_tokens=64 * 16, **kw):
+    from minfer_amd import Engine, load_model
+    return Engine(load_model(folder, dtype=dtype, device="cuda:0"), max_tokens=max_tokens, poison_cache=True, **kw)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", list(RZ))
+def test_replays_agree_with_plain(folders, plains, name, dtype):
+    """Whole; the last tokens one by one; unequal batches one after another (slots, states and pages used again over
+    a poisoned pool); prompts in portions down to two tokens and one, alone and in mixed batches."""
+    reqs = requests_for(RZ[name]["vocab"], (1, 7, 64, 150, 65, 33, 290), seed=3)
+    ids = list(reqs)
+    eng = engine_for(folders[name], dtype)
+    plain, ref = plains[name], {}
+    check(eng, whole_steps(reqs), plain, reqs, dtype, f"{name} whole", ref=ref)
+    check(eng, tail_steps(reqs, tail=80), plain, reqs, dtype, f"{name} last 80 one by one", ref=ref)
+    check(eng, batch_steps(reqs, [ids[:4], ids[4:]]), plain, reqs, dtype, f"{name} unequal batches", ref=ref)
+    check(eng, chunk_steps(reqs, [ids[:3], ids[3:]]), plain, reqs, dtype, f"{name} portions in batches", ref=ref)
+    check(eng, chunk_steps(reqs, [[r] for r in ids], sizes=(2,)), plain, reqs, dtype, f"{name} portions of 2", ref=ref)
+    check(eng, chunk_steps(reqs, [[r] for r in ids], sizes=(129, 3, 64)), plain, reqs, dtype, f"{name} portions of 129", ref=ref)
+    assert not eng.cache.live_slots()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_steps_in_which_nothing_or_little_is_wanted(folders, plains, dtype):
+    """Prompt steps that ask for no logits or for a few rows (the last layer's experts then see those rows' tokens
+    alone), then single tokens of which one sequence's are wanted."""
+    raw = dict(copy.deepcopy(RZ["A"]), layers=copy.deepcopy(RZ["A"]["layers"][1::-1]))      # the routed layer last
+    for name in ("A", "routed"):
+        if name == "A":
+            folder, plain = folders["A"], plains["A"]
+        else:
+            folder = write_rofizen(os.path.join(os.path.dirname(folders["A"]), f"routed_{dtype}"), raw, seed=4)
+            plain = pr.PlainRofizen.from_folder(folder)
+        eng = engine_for(folder, dtype)
+        toks = random_tokens(300, 100, 5)
+        a, b = eng.new_sequence(), eng.new_sequence()
+        full = plain.forward(toks)
+
+        def close(got, rows):
+            want = full[rows]
+            assert got.shape == want.shape
+            for g, w in zip(got, want):
+                tol = F32_ABS * max(1.0, w.std()) if dtype == "float32" else SHARP * BF16_MAX * w.std()
+                assert np.abs(g - w).max() <= tol
+        step = lambda *args: eng.step([a, b], *args).cpu().numpy()
+        assert step([toks[:60], toks[:20]], [[], []]).shape == (0, 300)
+        close(step([toks[60:90], toks[20:50]], [list(range(29, 1, -1)), [3]]), list(range(89, 61, -1)) + [23])
+        close(step([toks[90:91], toks[50:51]], [[0], []]), [90])
+        close(step([toks[91:92], toks[51:52]], [[], [0]]), [51])
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_batch_of_more_sequences_than_one_launch_of_the_experts_takes(folders, plains, dtype):
+    """Twenty sequences that start and decode together: the routed layers' few-token form runs in slices."""
+    reqs = requests_for(RZ["A"]["vocab"], tuple(3 + (7 * i) % 11 for i in range(20)), seed=12)
+    eng = engine_for(folders["A"], dtype, max_tokens=64 * 24)
+    check(eng, batch_steps(reqs, [list(reqs)], prompt_frac=0.4), plains["A"], reqs, dtype, "twenty together")
+    assert not eng.cache.live_slots()
+
+
+@pytest.mark.parametrize("seed", range(8))
+def test_configurations_drawn_at_random(tmp_path, seed):
+    """Whatever config.json may say: sizes, orders and options drawn at random, both run types, whole, one by one,
+    in batches and in portions."""
+    raw = random_config(np.random.default_rng(3600 + seed))
+    folder = write_rofizen(str(tmp_path / "m"), raw, seed=seed)
+    plain = pr.PlainRofizen.from_folder(folder)
+    reqs = requests_for(raw["vocab"], (1, 9, 70, 200, 131), seed=seed)
+    ids, ref = list(reqs), {}
+    for dtype in ("float32", "bfloat16"):
+        eng = engine_for(folder, dtype)
+        what = f"random configuration {seed} ({json.dumps(raw)[:600]})"
+        check(eng, whole_steps(reqs), plain, reqs, dtype, what + " whole", SHARP, ref=ref)
+        check(eng, tail_steps(reqs, tail=33), plain, reqs, dtype, what + " one by one", SHARP, ref=ref)
+        check(eng, batch_steps(reqs, [ids[:3], ids[3:]]), plain, reqs, dtype, what + " batches", SHARP, ref=ref)
+        check(eng, chunk_steps(reqs, [ids[:2], ids[2:]]), plain, reqs, dtype, what + " portions", SHARP, ref=ref)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_sharp_attention_and_long_decoding(tmp_path, dtype):
+    """Query gains raised so that the softmax picks single keys among hundreds, slopes that are small beside them,
+    temperatures that step while decoding, decays near one: a prompt of 700 tokens whole, then as 500 + 200 one by
+    one, then in three portions."""
+    raw = dict(architecture="Rofizen", vocab=300, width=96, norm=dict(eps=1e-5), embedding=dict(scale=4.0), postln_alpha=1.5, layers=[
+        dict(parallel(left(4, 2, 32, 16, 0.2, softcap=40.0, coef=0.5, every=64), right(2, 32, 24, 9.0)), mlp=moe(6, 2, 40, shared=24)),
+        dict(retention(2, 32, 32, (0.999, 0.9999), 32, base=100000.0), mlp=None),
+        dict(parallel(left(2, 1, 16, 48, 0.3, coef=0.2, every=100), right(3, 16, 48, 20.0)), mlp=dense(80)),
+        dict(gla(2, 32, 32, 16.0, 8), mlp=moe(4, 1, 56)),
+    ])
+    folder = write_rofizen(str(tmp_path / "sharp"), raw, seed=21, sharpen=6.0 if dtype == "float32" else 2.5)
+    plain = pr.PlainRofizen.from_folder(folder)
+    reqs, ref = {"long": random_tokens(300, 700, 77)}, {}
+    eng = engine_for(folder, dtype, max_tokens=64 * 16)
+    check(eng, whole_steps(reqs), plain, reqs, dtype, "sharp whole", SHARP, 1e-3, ref=ref)
+    check(eng, tail_steps(reqs, tail=200), plain, reqs, dtype, "sharp 500 + 200 one by one", SHARP, 1e-3, ref=ref)
+    check(eng, chunk_steps(reqs, [["long"]], sizes=(333, 2, 365)), plain, reqs, dtype, "sharp in portions", SHARP, 1e-3, ref=ref)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_row_does_not_depend_on_the_cut_or_the_company(folders, dtype):
+    """The last row of a request alone and whole, cut in two, and among others, closer than the comparison with 64 bits."""
+    eng = engine_for(folders["A"], dtype)
+    toks = random_tokens(300, 190, 15)
+    others = [random_tokens(300, n, 40 + n) for n in (3, 77, 130)]
+
+    def run(parts, company):
+        slots = [eng.new_sequence() for _ in range(1 + len(company))]
+        at = 0
+        for i, n in enumerate(parts):
+            with_them = company if i == 0 else []
+            used = slots[:1 + len(with_them)]
+            row = eng.step(used, [toks[at:at + n]] + with_them, [[n - 1]] + [[] for _ in with_them])
+            at += n
+        for s in slots:
+            eng.end_sequence(s)
+        return row[0].cpu().numpy()
+    whole = run([190], [])
+    for parts, company in (([190], others), ([100, 90], []), ([63, 65, 62], others), ([2, 188], others[:1]), ([189, 1], others)):
+        got = run(parts, company)
+        rms = float(np.sqrt(np.mean((got - whole) ** 2)))
+        assert rms <= (2e-5 if dtype == "float32" else 0.03) * whole.std(), (parts, len(company), rms / whole.std())
+
+
+def test_greedy_generation_through_the_entry_point(folders, plains):
+    """`LLM.generate`: the scheduler, slots used again (more prompts than slots), the captured decode step; 70 new
+    tokens so that every sequence crosses a page edge and a step of the temperature while decoding."""
+    from minfer_amd import LLM
+    llm = LLM(folders["A"], dtype="float32", n_ctx=256, n_slots=2)
+    prompts = [random_tokens(300, n, 30 + i) for i, n in enumerate((5, 60, 1, 17))]
+    res = llm.generate(prompts, max_new=70, temp=0.0, repeat_penalty=1.0, stop_tokens=[])
+    eager = llm.generate(prompts, max_new=70, temp=0.0, repeat_penalty=1.0, stop_tokens=[], use_graph=False)
+    assert res.tokens == eager.tokens
+    for p, toks in zip(prompts, res.tokens):
+        assert len(toks) == 70
+        logits = plains["A"].forward(list(p) + toks)
+        for i, t in enumerate(toks):
+            row = logits[len(p) + i - 1]
+            top = np.sort(row)[-2:]
+            assert t == pr.greedy(row) or top[1] - top[0] < 1e-4, f"token {i}"
+    bf = LLM(folders["A"], dtype="bfloat16", n_ctx=256, n_slots=4)
+    a = bf.generate(prompts, max_new=20, temp=0.0, repeat_penalty=1.0, stop_tokens=[]).tokens
+    b = bf.generate(prompts, max_new=20, temp=0.0, repeat_penalty=1.0, stop_tokens=[], use_graph=False).tokens
+    assert a == b
+
+
+def test_programs(folders, plains, tmp_path):
+    """bin/minfer generates greedily from a Rofizen folder; bin/trace_run replays a batch."""
+    env = dict(os.environ, PYTHONPATH=ROOT)
+    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "minfer"), folders["B"], "--prompt-tokens", "5,6,7;9",
+                        "--greedy", "--repeat-penalty", "1.0", "-n", "4", "--dtype", "float32", "--n-ctx", "64",
+                        "--stop-token", "100000"], capture_output=True, text=True, env=env, timeout=300)
+    assert r.returncode == 0, r.stderr
+    lines = [l for l in r.stdout.strip().splitlines() if l]
+    for line, prompt in zip(lines, ([5, 6, 7], [9])):
+        seq = list(prompt)
+        for t in (int(x) for x in line.split(",")):
+            assert t == pr.greedy(plains["B"].forward(seq)[-1])
+            seq.append(t)
+    vocab = RZ_B["vocab"]
+    reqs = requests_for(vocab, (3, 70, 20), seed=9)
+    ref = {rid: plains["B"].forward(toks) for rid, toks in reqs.items()}
+    steps = batch_steps(reqs, [list(reqs)])
+    out = str(tmp_path / "out")
+    p = subprocess.Popen([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", folders["B"], "--dtype",
+                          "float32", "--out", out, "--max-tokens", "93"], stdin=subprocess.PIPE, stdout=subprocess.PIPE,
+                         text=True, bufsize=1)
+    rows, pos = {}, {}
+    try:
+        for st in steps:
+            p.stdin.write(json.dumps(st) + "\n")
+            p.stdin.flush()
+            assert p.stdout.readline().strip() == f"done {st['step']}"
+            arr = np.fromfile(os.path.join(out, f"{st['step']}.f32"), dtype="<f4").reshape(-1, vocab)
+            i = 0
+            for e in st["entries"]:
+                for w in e["want"]:
+                    rows[(e["id"], pos.get(e["id"], 0) + w)] = arr[i]
+                    i += 1
+                pos[e["id"]] = pos.get(e["id"], 0) + len(e["tokens"])
+        p.stdin.close()
+        assert p.wait(timeout=60) == 0
+    finally:
+        if p.poll() is None:
+            p.kill()
+    for (rid, p), got in rows.items():
+        assert np.abs(got - ref[rid][p]).max() <= F32_ABS * max(1.0, ref[rid][p].std()), f"trace_run: request {rid} position {p}"
