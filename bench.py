@@ -68,12 +68,12 @@ def parse():
                     help="cache size in tokens (default: batch x context, or what fits in free memory if less)")
     ap.add_argument("--no-graph", action="store_true")
     ap.add_argument("--only", choices=["decode", "prefill"], help="run one part (for profiles); prints no JSON line")
-    ap.add_argument("--design", choices=["tabezen", "lagedra", "nodutar", "katarax"], default=None,
+    ap.add_argument("--design", choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen"], default=None,
                     help="instead of the default workload: prefill and decode of this design at a few layer sizes "
                          "beside its nearest relative of the same width, depth and feed-forward size (the Qwen2 "
                          "decoder; for nodutar, Lagedra), kernel by kernel")
     ap.add_argument("--design-sizes", default="small,medium", help="which of the design's sizes to run")
-    ap.add_argument("--design-model", default=None, choices=["tabezen", "lagedra", "nodutar", "katarax", "qwen2"],
+    ap.add_argument("--design-model", default=None, choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen", "qwen2"],
                     help="with --design and --only: which of the two models runs the one part (for profiles; "
                          "default: the design itself)")
     return ap.parse_args()
@@ -310,6 +310,25 @@ def katarax_config(width, layers, heads, ff, dim=128, vdim=128, window=1024, ran
     return dict(architecture="Katarax", vocab=vocab, width=width, norm=dict(eps=1e-6), logit_softcap=30.0, layers=made)
 
 
+def rofizen_config(width, layers, heads, ff, dim=128, vdim=128, experts=8, rank=16, vocab=32768):
+    """Gated linear attention and retention with the attention beside a matrix memory after each of them, in turn; the
+    first layer of four with a dense feed-forward of `ff`, the others with routed experts of ff / 2 values, one a
+    token, beside a shared one of ff / 2 (a token passes as many values as in `nodutar_config`); head sizes and kv
+    heads as there, every recurrence's state as its gated recurrence's."""
+    kv = max(1, heads // 4)
+    gla = dict(type="gla", mixer=dict(heads=heads, dim=dim, vdim=vdim, tau=16.0, rank=rank))
+    ret = dict(type="retention", mixer=dict(heads=heads, dim=dim, vdim=vdim, rot=dict(base=10000.0, dims=dim),
+                                            decay=[1.0 - 2.0 ** (-5.0 - 3.0 * h / max(1, heads - 1)) for h in range(heads)]))
+    both = dict(type="parallel", mixer=dict(
+        left=dict(heads=heads, kv_heads=kv, dim=dim, vdim=vdim, scale=dim ** -0.5, softcap=50.0, q_temp=dict(coef=0.5, every=1024)),
+        right=dict(heads=heads, dim=dim, vdim=vdim, gate_cap=15.0)))
+    dense = dict(kind="dense", ff=ff)
+    routed = dict(kind="moe", expert=dict(ff=ff // 2), router=dict(experts=experts, top=1), shared=dict(ff=ff // 2))
+    return dict(architecture="Rofizen", vocab=vocab, width=width, norm=dict(eps=1e-6), embedding=dict(scale=width ** 0.5),
+                postln_alpha=(2.0 * layers) ** 0.25,
+                layers=[dict((gla, both, ret, both)[i % 4], mlp=dense if i % 4 == 0 else routed) for i in range(layers)])
+
+
 def qwen2_like(width, layers, heads, ff, vocab=32768):
     """The Qwen2 decoder of the same width, depth, head count and feed-forward size (head size 128)."""
     return dict(QWEN25_7B, num_hidden_layers=layers, hidden_size=width, num_attention_heads=heads,
@@ -324,9 +343,9 @@ DESIGN_SIZES = {
 
 
 DESIGN_CONFIGS = {"tabezen": tabezen_config, "lagedra": lagedra_config, "nodutar": nodutar_config, "katarax": katarax_config,
-                  "qwen2": qwen2_like}
+                  "rofizen": rofizen_config, "qwen2": qwen2_like}
 # the model a design is measured beside
-NEAREST = {"tabezen": "qwen2", "lagedra": "qwen2", "nodutar": "lagedra", "katarax": "nodutar"}
+NEAREST = {"tabezen": "qwen2", "lagedra": "qwen2", "nodutar": "lagedra", "katarax": "nodutar", "rofizen": "nodutar"}
 
 
 def traced_step(eng, slots, toks, want):

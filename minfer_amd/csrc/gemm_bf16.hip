@@ -139,14 +139,20 @@ __device__ __forceinline__ void tile_position(int tile, int tiles_m, int tiles_n
   bn = in_band / rows;
 }
 
+// Rows of a product that belong to one of several matrices: `rows` of them (at most a tile's) from row `first` on.
+struct RowGroup { int first, rows, matrix, unused; };
+
 // ------------------------------------------------------------------ tiled kernel
 // LDS row stride is BK + 8 elements (144 bytes for BK 64, 80 for BK 32): conflict-free b128 reads
-template <int BM, int BN, int WM, int WN, int BK, bool VEC>
+// GROUPED: rows in groups, each with a matrix of its own (experts): entry bm of `groups` names the rows of tile row bm
+// and the matrix, one of a stack [matrices][N][ldw] (see RowGroup).
+template <int BM, int BN, int WM, int WN, int BK, bool VEC, bool GROUPED = false>
 __global__ __launch_bounds__(64 * (BM / WM) * (BN / WN)) void tile_kernel(const bf16* __restrict__ A, int lda,
                                                    const bf16* __restrict__ W, int ldw,
                                                    const float* __restrict__ bias, void* __restrict__ C,
                                                    int ldc, int M, int N, int K, int epi, int tiles_m,
-                                                   int xcd_remap, int k_per_split) {
+                                                   int xcd_remap, int k_per_split,
+                                                   const RowGroup* __restrict__ groups = nullptr) {
   constexpr int NTHR = 64 * (BM / WM) * (BN / WN);
   constexpr int LDS_LD = BK + 8;
   if (k_per_split > 0) {
@@ -177,6 +183,14 @@ __global__ __launch_bounds__(64 * (BM / WM) * (BN / WN)) void tile_kernel(const 
   }
   int bm, bn;
   tile_position(tile, tiles_m, gridDim.x / tiles_m, bm, bn);
+  if (GROUPED) {
+    const RowGroup rg = groups[bm];
+    A += (size_t)rg.first * lda;
+    W += (size_t)rg.matrix * N * ldw;
+    C = (float*)C + (size_t)rg.first * ldc;
+    M = rg.rows;
+    bm = 0;
+  }
   const int m0 = bm * BM, n0 = bn * BN;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int wm = (wid % (BM / WM)) * WM, wn = (wid / (BM / WM)) * WN;
@@ -314,12 +328,13 @@ __device__ __forceinline__ void dma_wait(int tiles) {
 
 // BN: the tile's width (256 or 128); WAVES_M x (8 / WAVES_M): the grid of the 8 waves over the
 // tile; STAGES: k tiles of a tile in LDS (2 or 3), (256 + BN) * 128 bytes each.
-template <int BN, int WAVES_M, int STAGES>
+template <int BN, int WAVES_M, int STAGES, bool GROUPED = false>
 __global__ __launch_bounds__(512) void tile_dma_kernel(const bf16* __restrict__ A, int lda,
                                                        const bf16* __restrict__ W, int ldw,
                                                        const float* __restrict__ bias, void* __restrict__ C,
                                                        int ldc, int M, int N, int K, int epi, int tiles_m,
-                                                       int xcd_remap, int k_per_split) {
+                                                       int xcd_remap, int k_per_split,
+                                                       const RowGroup* __restrict__ groups = nullptr) {
   constexpr int WAVES_N = 8 / WAVES_M;
   constexpr int WM = DMA_BM / WAVES_M, WN = BN / WAVES_N;
   constexpr int TM = WM / 32, TN = WN / 32;
@@ -346,6 +361,14 @@ __global__ __launch_bounds__(512) void tile_dma_kernel(const bf16* __restrict__ 
   }
   int bm, bn;
   tile_position(tile, tiles_m, gridDim.x / tiles_m, bm, bn);
+  if (GROUPED) {
+    const int first = __builtin_amdgcn_readfirstlane(groups[bm].first), matrix = __builtin_amdgcn_readfirstlane(groups[bm].matrix);
+    M = __builtin_amdgcn_readfirstlane(groups[bm].rows);
+    A += (size_t)first * lda;
+    W += (size_t)matrix * N * ldw;
+    C = (float*)C + (size_t)first * ldc;
+    bm = 0;
+  }
   const int m0 = bm * DMA_BM, n0 = bn * BN;
   const int lane = threadIdx.x & 63;
   const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -484,7 +507,7 @@ int launch_tile_dma(const bf16* A, int lda, const bf16* W, int ldw, const float*
   }
   const int tiles_m = (M + DMA_BM - 1) / DMA_BM, tiles_n = (N + BN - 1) / BN;
   kern<<<dim3(tiles_m * tiles_n, splits), 512, smem, stream>>>(A, lda, W, ldw, bias, C, ldc, M, N, K, epi, tiles_m,
-                                                               tiles_m * tiles_n >= 16, k_per_split);
+                                                               tiles_m * tiles_n >= 16, k_per_split, nullptr);
   return mf_launch_status();
 }
 
@@ -503,7 +526,7 @@ int launch_tile_v(const bf16* A, int lda, const bf16* W, int ldw, const float* b
   }
   const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
   kern<<<dim3(tiles_m * tiles_n, splits), NTHR, smem, stream>>>(A, lda, W, ldw, bias, C, ldc, M, N, K, epi,
-                                                                tiles_m, tiles_m * tiles_n >= 16, k_per_split);
+                                                                tiles_m, tiles_m * tiles_n >= 16, k_per_split, nullptr);
   return mf_launch_status();
 }
 
@@ -515,6 +538,41 @@ int launch_tile(const bf16* A, int lda, const bf16* W, int ldw, const float* bia
                                                           splits, k_per_split)
                 : launch_tile_v<BM, BN, WM, WN, BK, false>(A, lda, W, ldw, bias, C, ldc, M, N, K, epi, stream,
                                                            splits, k_per_split);
+}
+
+// The grouped forms: a tile row per entry of `groups` (int32 [n_groups][4] on the device), 32-bit sums stored.
+template <int BN, int WAVES_M, int STAGES>
+int launch_grouped_dma(const bf16* A, int lda, const bf16* W, int ldw, float* C, int ldc, const RowGroup* groups, int n_groups,
+                       int N, int K, hipStream_t stream) {
+  constexpr int smem = STAGES * (DMA_BM + BN) * DMA_BK * 2;
+  static bool configured = false;
+  auto kern = tile_dma_kernel<BN, WAVES_M, STAGES, true>;
+  if (!configured) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+    if (e != hipSuccess) return (int)e;
+    configured = true;
+  }
+  const int tiles_n = (N + BN - 1) / BN;
+  kern<<<dim3(n_groups * tiles_n), 512, smem, stream>>>(A, lda, W, ldw, nullptr, C, ldc, 0, N, K, EPI_F32, n_groups,
+                                                        n_groups * tiles_n >= 16, 0, groups);
+  return mf_launch_status();
+}
+
+template <int BM, int BN, int WM, int WN, int BK>
+int launch_grouped_tile(const bf16* A, int lda, const bf16* W, int ldw, float* C, int ldc, const RowGroup* groups, int n_groups,
+                        int N, int K, hipStream_t stream) {
+  constexpr int smem = 2 * (BM + BN) * (BK + 8) * (int)sizeof(bf16);
+  static bool configured = false;
+  auto kern = tile_kernel<BM, BN, WM, WN, BK, true, true>;
+  if (!configured) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+    if (e != hipSuccess) return (int)e;
+    configured = true;
+  }
+  const int tiles_n = (N + BN - 1) / BN;
+  kern<<<dim3(n_groups * tiles_n), 64 * (BM / WM) * (BN / WN), smem, stream>>>(A, lda, W, ldw, nullptr, C, ldc, 0, N, K, EPI_F32,
+                                                                               n_groups, n_groups * tiles_n >= 16, 0, groups);
+  return mf_launch_status();
 }
 
 // ------------------------------------------------------------------ skinny kernel
@@ -1975,6 +2033,26 @@ SkinnyChoice skinny_choice(int M, int N, int K, bool aligned, int epi, int split
 }
 
 }  // namespace
+
+// Products of rows that stand in groups with a matrix each: rows first .. first + rows - 1 of A (a row group's, at most
+// the variant's tile rows) with matrix `matrix` of the stack W [matrices][N][K], 32-bit sums into the same rows of C.
+// variant 2: tiles of 128 x 128, 12: 256 x 256 (K in 64s), 13: 256 x 128 (K in 64s).
+MF_API int mf_gemm_bf16_grouped(const void* A, const void* W, float* C, const int* groups, int n_groups, int N, int K,
+                                int variant, hipStream_t stream) {
+  if (n_groups <= 0 || N <= 0) return 0;
+  if (K <= 0 || K % 8 || !groups || (uintptr_t)A % 16 || (uintptr_t)W % 16 || (variant != 2 && K % DMA_BK) ||
+      (size_t)N * K * 2 >= (1ull << 32))
+    return (int)hipErrorInvalidValue;
+  const bf16* a = (const bf16*)A;
+  const bf16* w = (const bf16*)W;
+  const RowGroup* g = (const RowGroup*)groups;
+  switch (variant) {
+    case 2: return launch_grouped_tile<128, 128, 64, 64, 64>(a, K, w, K, C, N, g, n_groups, N, K, stream);
+    case 12: return launch_grouped_dma<256, 2, 2>(a, K, w, K, C, N, g, n_groups, N, K, stream);
+    case 13: return launch_grouped_dma<128, 4, 3>(a, K, w, K, C, N, g, n_groups, N, K, stream);
+  }
+  return (int)hipErrorInvalidValue;
+}
 
 // `variant`: 0 picks by shape among the whole-K kernels; 1: 256x256 tile with 4 waves, 2: 128x128,
 // 3: 64x64, 6: 256x128 with 8 waves, 9: 256x256 with 8 waves; through the direct-to-LDS pipeline, K in

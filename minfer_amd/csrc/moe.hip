@@ -21,8 +21,8 @@
 // matrices side by side gives the weighted sum of the chosen experts' outputs.
 // `gated_expert_act_kernel`: an expert that every token takes, weighed by a sigmoid of its own per token:
 // y = silu(gate) up sigmoid(z), from one row gate [F] | up [F] | z | padding.
-// `moe_sparse_*`: for steps of few tokens, only the chosen experts' matrices are read: a wave per
-// output row of a (token, choice) pair.
+// `moe_sparse_*`: for steps of few tokens, only the chosen experts' matrices are read, each once: on the matrix
+// cores (`moe_sparse_mfma_kernel`), or a wave per output row of an expert.
 #include "common.h"
 
 #define MF_MOE_MAX_EXPERTS 1024
@@ -257,9 +257,9 @@ template <typename WT>
 __global__ __launch_bounds__(256) void moe_sparse_up_kernel(const WT* __restrict__ x, const WT* __restrict__ gate_up,
                                                             const int* __restrict__ chosen, WT* __restrict__ y,
                                                             int n_pairs, int top, int F, int K, float limit, int act) {
-  const int e = blockIdx.x;
+  const int e = blockIdx.y;
   const int lane = threadIdx.x & 63;
-  const int f = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int f = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int c0 = lane < n_pairs ? chosen[lane] : -1, c1 = lane + 64 < n_pairs ? chosen[lane + 64] : -1;
   const unsigned long long mine0 = __ballot(c0 == e), mine1 = __ballot(c1 == e);
   if (!(mine0 | mine1) || f >= F) return;
@@ -303,9 +303,9 @@ template <typename WT>
 __global__ __launch_bounds__(256) void moe_sparse_down_kernel(const WT* __restrict__ y, const WT* __restrict__ down,
                                                               const int* __restrict__ chosen, float* __restrict__ rows,
                                                               int n_pairs, int F, int N) {
-  const int e = blockIdx.x;
+  const int e = blockIdx.y;
   const int lane = threadIdx.x & 63;
-  const int n = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int c0 = lane < n_pairs ? chosen[lane] : -1, c1 = lane + 64 < n_pairs ? chosen[lane + 64] : -1;
   const unsigned long long mine0 = __ballot(c0 == e), mine1 = __ballot(c1 == e);
   if (!(mine0 | mine1) || n >= N) return;
@@ -338,6 +338,91 @@ __global__ __launch_bounds__(256) void moe_sparse_down_kernel(const WT* __restri
       if (lane == 0) rows[(size_t)pr * N + n] = v;
     }
   }
+}
+
+// The same two products on the matrix cores, bfloat16, for rows of a multiple of 64 values and a multiple of 16 output
+// rows.  A workgroup of NW waves owns (expert, 16 output rows) and leaves at once where nobody chose the expert; its
+// waves share K, 64 values a step: A = 16 rows of a matrix (16x16x32 MFMA, a lane two neighbouring runs of 8 values, so
+// that a step reads 128 bytes of every row side by side), B = the rows of the expert's pairs, a column each, with the
+// same order of k.  The waves' sums meet in LDS and are added in the waves' order.
+//   UP:  two matrices (gate and up) share B; y[pair][f] gets the activation.
+//   else: rows[pair][n] gets the product.
+template <int NW, bool UP>
+__global__ __launch_bounds__(NW * 64) void moe_sparse_mfma_kernel(const bf16* __restrict__ x, const bf16* __restrict__ weights,
+                                                                  const int* __restrict__ chosen, bf16* __restrict__ y,
+                                                                  float* __restrict__ rows, int n_pairs, int top, int N,
+                                                                  int K, float limit, int act) {
+  constexpr int MATS = UP ? 2 : 1;
+  __shared__ float sums[NW][MATS][256];
+  __shared__ int pair_of[MF_MOE_SPARSE_TOKENS];
+  const int e = blockIdx.y, n0 = blockIdx.x * 16;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int c0 = lane < n_pairs ? chosen[lane] : -1, c1 = lane + 64 < n_pairs ? chosen[lane + 64] : -1;
+  const unsigned long long mine0 = __ballot(c0 == e), mine1 = __ballot(c1 == e);
+  const int n0_pairs = __popcll(mine0), n_mine = min(n0_pairs + __popcll(mine1), MF_MOE_SPARSE_TOKENS);
+  if (n_mine == 0) return;                     // (the same for all waves)
+  if (w == 0) {
+    const unsigned long long below = (1ull << lane) - 1;
+    const int r0 = __popcll(mine0 & below), r1 = n0_pairs + __popcll(mine1 & below);
+    if (c0 == e && r0 < MF_MOE_SPARSE_TOKENS) pair_of[r0] = lane;
+    if (c1 == e && r1 < MF_MOE_SPARSE_TOKENS) pair_of[r1] = lane + 64;
+  }
+  __syncthreads();
+  const int col = lane & 15, g = lane >> 4;
+  const int pr = pair_of[min(col, n_mine - 1)];
+  const bf16* xr = x + (size_t)(UP ? pr / top : pr) * K + 16 * g;
+  const bf16* wr[MATS];
+#pragma unroll
+  for (int m = 0; m < MATS; ++m) wr[m] = weights + ((size_t)e * MATS * N + (size_t)m * N + n0 + col) * K + 16 * g;
+  floatx4 acc[MATS];
+#pragma unroll
+  for (int m = 0; m < MATS; ++m) acc[m] = floatx4{0.f, 0.f, 0.f, 0.f};
+  const int steps = K / 64;
+  const int s1 = (w + 1) * steps / NW;
+#pragma unroll 4
+  for (int s = w * steps / NW; s < s1; ++s) {
+    bf16x8 b[2], a[MATS][2];
+#pragma unroll
+    for (int q = 0; q < 2; ++q) {
+#pragma unroll
+      for (int m = 0; m < MATS; ++m) a[m][q] = *(const bf16x8*)(wr[m] + s * 64 + 8 * q);
+      b[q] = *(const bf16x8*)(xr + s * 64 + 8 * q);
+    }
+#pragma unroll
+    for (int q = 0; q < 2; ++q)
+#pragma unroll
+      for (int m = 0; m < MATS; ++m) acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[m][q], b[q], acc[m], 0, 0, 0);
+  }
+  // D[i = 4 g + r][j = col]: output row n0 + i of the pair in column j
+#pragma unroll
+  for (int m = 0; m < MATS; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) sums[w][m][(4 * g + r) * 16 + col] = acc[m][r];
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_mine * 16; i += NW * 64) {
+    const int row = i & 15, j = i >> 4;
+    float v[MATS];
+#pragma unroll
+    for (int m = 0; m < MATS; ++m) {
+      v[m] = 0.f;
+#pragma unroll
+      for (int k = 0; k < NW; ++k) v[m] += sums[k][m][row * 16 + j];
+    }
+    const size_t at = (size_t)pair_of[j] * N + n0 + row;
+    if (UP) y[at] = (bf16)expert_act(v[0], v[MATS - 1], limit, act);
+    else rows[at] = v[0];
+  }
+}
+
+template <bool UP>
+static int launch_sparse_mfma(const bf16* x, const bf16* weights, const int* chosen, bf16* y, float* rows, int n_pairs, int top,
+                              int E, int N, int K, float limit, int act, hipStream_t stream) {
+  const dim3 grid(N / 16, E);      // (an expert's workgroups next to each other, so that they spread over the XCDs)
+  if (K >= 4096)
+    moe_sparse_mfma_kernel<8, UP><<<grid, 512, 0, stream>>>(x, weights, chosen, y, rows, n_pairs, top, N, K, limit, act);
+  else
+    moe_sparse_mfma_kernel<4, UP><<<grid, 256, 0, stream>>>(x, weights, chosen, y, rows, n_pairs, top, N, K, limit, act);
+  return mf_launch_status();
 }
 
 // ------------------------------------------------------------------ many tokens: the tokens of an expert together
@@ -428,15 +513,22 @@ MF_API int mf_moe_act(const float* gu, const float* dense, void* y, int y_is_bf1
 
 MF_API int mf_moe_sparse(const void* x, const void* gate_up, const void* down, const int* chosen, const float* weights,
                          void* y, float* rows, float* out, int is_bf16, int n_tok, int top, int E, int F, int K, int N,
-                         float limit, int act, hipStream_t stream) {
+                         float limit, int act, int add, hipStream_t stream) {
   if (n_tok <= 0) return 0;
   if (act != MF_MOE_ACT_CLAMPED && act != MF_MOE_ACT_SILU) return (int)hipErrorInvalidValue;
   if (top <= 0 || E <= 0 || F <= 0 || K <= 0 || N <= 0 || n_tok > MF_MOE_SPARSE_TOKENS || n_tok * top > MF_MOE_SPARSE_PAIRS ||
       !y || !rows)
     return (int)hipErrorInvalidValue;
-  dim3 g1(E, (F + 3) / 4), g2(E, (N + 3) / 4);
+  dim3 g1((F + 3) / 4, E), g2((N + 3) / 4, E);
   const int pairs = n_tok * top;
-  if (is_bf16) {
+  if (is_bf16 && K % 64 == 0 && F % 64 == 0 && N % 16 == 0) {
+    const int rc = launch_sparse_mfma<true>((const bf16*)x, (const bf16*)gate_up, chosen, (bf16*)y, nullptr, pairs, top, E, F, K,
+                                            limit, act, stream);
+    if (rc) return rc;
+    const int rd = launch_sparse_mfma<false>((const bf16*)y, (const bf16*)down, chosen, nullptr, rows, pairs, top, E, N, F, limit,
+                                             act, stream);
+    if (rd) return rd;
+  } else if (is_bf16) {
     moe_sparse_up_kernel<bf16><<<g1, 256, 0, stream>>>((const bf16*)x, (const bf16*)gate_up, chosen, (bf16*)y, pairs, top, F, K, limit, act);
     int rc = mf_launch_status();
     if (rc) return rc;
@@ -449,7 +541,7 @@ MF_API int mf_moe_sparse(const void* x, const void* gate_up, const void* down, c
   }
   int rc = mf_launch_status();
   if (rc) return rc;
-  moe_combine_kernel<<<dim3(n_tok, (N + 255) / 256), 256, 0, stream>>>(rows, chosen, nullptr, nullptr, weights, out, top, N, 1);
+  moe_combine_kernel<<<dim3(n_tok, (N + 255) / 256), 256, 0, stream>>>(rows, chosen, nullptr, nullptr, weights, out, top, N, add);
   return mf_launch_status();
 }
 

@@ -96,7 +96,7 @@ _PROTOTYPES = {
         "mf_moe_route": [_P, c_int, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_float, _P],
         "mf_moe_act": [_P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P],
         "mf_moe_sparse": [_P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
-                          _P],
+                          c_int, _P],
         "mf_moe_table": [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_gated_expert_act": [_P, c_int, _P, c_int, c_int, c_int, _P],
         "mf_moe_group": [_P, c_int, c_int, _P, _P, _P],
@@ -132,6 +132,7 @@ _PROTOTYPES = {
     },
     "gemm_bf16": {
         "mf_gemm_bf16": [_P, c_int, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P],
+        "mf_gemm_bf16_grouped": [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
         "mf_gemm_bf16_splitk": [_P, c_int, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_int,
                                 c_int, _P],
         "mf_gemm_bf16_skinny": [_P, c_int, _P, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int, c_int,
@@ -1335,9 +1336,9 @@ def moe_act(gu: torch.Tensor, dense: torch.Tensor, out: torch.Tensor, limit: flo
 
 
 def moe_sparse(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-               out: torch.Tensor, n_experts: int, limit: float, act: int = 0) -> None:
+               out: torch.Tensor, n_experts: int, limit: float, act: int = 0, accumulate: bool = True) -> None:
     """The chosen experts only, for steps of few tokens: `gate_up` `[experts][2 F][K]` (an expert's gate
-    rows, then its up rows), `down` `[experts][N][F]`; out `[tokens][N]` float32 += the weighted sum of the
+    rows, then its up rows), `down` `[experts][N][F]`; out `[tokens][N]` float32 (+)= the weighted sum of the
     chosen experts' outputs, choices added in their order."""
     n_tok, K = x.shape
     top = chosen.shape[1]
@@ -1354,7 +1355,8 @@ def moe_sparse(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chose
     y = torch.empty((n_tok, top, F), dtype=x.dtype, device=x.device)
     rows = torch.empty((n_tok * top, N), dtype=torch.float32, device=x.device)
     _check(_fn("moe", "mf_moe_sparse")(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(chosen), _ptr(weights), _ptr(y), _ptr(rows), _ptr(out),
-                                        _is_bf16(x), n_tok, top, n_experts, F, K, N, float(limit), int(act), _stream()), "moe_sparse")
+                                        _is_bf16(x), n_tok, top, n_experts, F, K, N, float(limit), int(act),
+                                        1 if accumulate else 0, _stream()), "moe_sparse")
 
 SCAN_CHUNK = 32          # tokens of a chunk of the chunked scan (MF_SCAN_CHUNK in csrc/recurrence.hip)
 
@@ -1754,6 +1756,55 @@ def linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], 
             return
     _check(_fn("gemm_bf16", "mf_gemm_bf16")(_ptr(x), k, _ptr(weight), k, _ptr(bias), _ptr(out), n, m,
                                              n, k, epi, variant, _stream()), f"gemm_bf16 {m}x{n}x{k}")
+
+
+# variants of the grouped product: (tile rows, tile columns, blocks a CU, microseconds a k tile of 64 with every CU
+# busy), as the plan of the single product has them
+GROUPED_TILES = {12: (256, 256, 1, 1.75), 13: (256, 128, 1, 1.0), 2: (128, 128, 2, 1.45)}
+
+
+def grouped_takes(dtype, n: int, k: int) -> bool:
+    """Whether `linear_grouped` takes matrices `[n][k]` of this type."""
+    return dtype == torch.bfloat16 and k % 64 == 0 and n * k * 2 < 1 << 32
+
+
+def grouped_plan(counts, n: int, k: int) -> int:
+    """The tile variant for groups of `counts` rows against `[n][k]` matrices: the fewest rounds of tiles times what
+    a round takes (a last round that is not full counts somewhat less)."""
+    best, best_us = 0, 0.0
+    for variant, (bm, bn, per_cu, step) in GROUPED_TILES.items():
+        blocks = sum((c + bm - 1) // bm for c in counts) * ((n + bn - 1) // bn)
+        full, rest = divmod(blocks, per_cu * cu_count())
+        us = (k // 64) * step * (full + (0.7 + 0.3 * rest / (per_cu * cu_count()) if rest else 0.0))
+        if not best or us < best_us * 0.98:
+            best, best_us = variant, us
+    return best
+
+
+def row_groups(counts, variant: int):
+    """The table of a grouped product for groups of `counts` rows that stand one after the other: int32
+    `[tile rows][4]` (first row, rows, group, 0), no tile row across two groups."""
+    bm = GROUPED_TILES[variant][0]
+    out, first = [], 0
+    for g, c in enumerate(counts):
+        out += [(first + r, min(bm, c - r), g, 0) for r in range(0, c, bm)]
+        first += c
+    return out
+
+
+def linear_grouped(x: torch.Tensor, weights: torch.Tensor, groups: torch.Tensor, variant: int, out: torch.Tensor) -> None:
+    """out[r] = weights[g] x[r] for the rows r of every group g, in bfloat16 with 32-bit sums.  `weights`
+    `[groups][n][k]`; `groups`: `row_groups` on the device, made for `variant`; out float32 `[rows][n]`."""
+    rows, k = x.shape
+    n = weights.shape[1]
+    _need(x, "linear_grouped.x", torch.bfloat16)
+    _need(weights, "linear_grouped.weights", torch.bfloat16, (weights.shape[0], n, k))
+    _need(groups, "linear_grouped.groups", torch.int32)
+    _need(out, "linear_grouped.out", torch.float32, (rows, n))
+    if not grouped_takes(x.dtype, n, k) or variant not in GROUPED_TILES or groups.dim() != 2 or groups.shape[1] != 4:
+        raise KernelError(f"linear_grouped: matrices [{n}][{k}], variant {variant}, groups {tuple(groups.shape)}")
+    _check(_fn("gemm_bf16", "mf_gemm_bf16_grouped")(_ptr(x), _ptr(weights), _ptr(out), _ptr(groups), groups.shape[0], n, k, variant,
+                                                     _stream()), f"gemm_bf16_grouped {rows}x{n}x{k}")
 
 
 def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:

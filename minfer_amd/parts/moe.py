@@ -22,7 +22,8 @@ Two forms, both of which read or multiply only what was chosen.  Steps of few to
 may be captured, so nothing may wait for the host): `ops.moe_sparse`, up to 16 tokens a launch, reads every
 chosen expert's matrices once.  Steps of many tokens: the (token, choice) pairs are grouped by expert
 (`ops.moe_group`; the host reads the experts' counts, the one wait of the step), the tokens' rows are put side by
-side expert by expert, every expert with tokens runs its two products over its rows, and the rows' results are
+side expert by expert, the experts' two products run over their rows (all experts in one launch where the sizes
+allow it, `ops.linear_grouped`, else an expert at a time), and the rows' results are
 added into the stream with the tokens' weights, a token's choices in their order.  (With a table nothing waits:
 the host counts the experts' pairs itself.)
 
@@ -146,11 +147,9 @@ class Experts(FeedForward):
             accumulate = True
         few = min(SPARSE_UP_TO, max(1, ops.MOE_SPARSE_PAIRS // self.top))
         if (n <= few or (ctx is not None and ctx.all_decode)) and x.dtype == self.gate_up.dtype:
-            if not accumulate:
-                h.zero_()
             for t0 in range(0, n, few):      # (slices of a contiguous tensor's rows are contiguous)
                 ops.moe_sparse(x[t0:t0 + few], self.gate_up, self.down, chosen[t0:t0 + few], weights[t0:t0 + few],
-                               h[t0:t0 + few], self.ne, self.limit, self.act)
+                               h[t0:t0 + few], self.ne, self.limit, self.act, accumulate=accumulate)
             return
         rank = torch.empty_like(chosen)
         counts = torch.empty(self.ne, dtype=torch.int32, device=dev)
@@ -161,21 +160,36 @@ class Experts(FeedForward):
         starts = [0]
         for c in per_expert:
             starts.append(starts[-1] + c)
-        # from pinned memory the copy does not wait for what the stream still has to do
-        offsets = torch.tensor(starts[:-1], dtype=torch.int32, pin_memory=dev.type == "cuda").to(dev, non_blocking=True)
         pairs = n * self.top
+        # one product over all experts' rows where its kernel takes the sizes, else a product an expert
+        grouped = x.dtype == self.gate_up.dtype and ops.grouped_takes(x.dtype, 2 * self.inter, self.hidden) \
+            and ops.grouped_takes(x.dtype, self.hidden, self.inter)
+        plans = [ops.grouped_plan(per_expert, 2 * self.inter, self.hidden), ops.grouped_plan(per_expert, self.hidden, self.inter)] \
+            if grouped else []
+        tables = [ops.row_groups(per_expert, v) for v in plans]
+        flat = starts[:-1] + [0] * (-self.ne % 4) + [v for t in tables for row in t for v in row]
+        # from pinned memory the copy does not wait for what the stream still has to do
+        meta = torch.tensor(flat, dtype=torch.int32, pin_memory=dev.type == "cuda").to(dev, non_blocking=True)
+        offsets, at = meta[:self.ne], (self.ne + 3) // 4 * 4
         xs = torch.empty((pairs, self.hidden), dtype=x.dtype, device=dev)
         ops.moe_gather(x, chosen, rank, offsets, xs)
         gu = torch.empty((pairs, 2 * self.inter), dtype=torch.float32, device=dev)
-        for e, (gate_up, _) in enumerate(self.experts):
-            if per_expert[e]:
-                gate_up(xs[starts[e]:starts[e + 1]], out=gu[starts[e]:starts[e + 1]])
         y = torch.empty((pairs, self.inter), dtype=self.rt.dtype, device=dev)
-        ops.moe_act(gu, self._ones(pairs, dev), y, self.limit, self.act)
         rows = torch.empty((pairs, self.hidden), dtype=torch.float32, device=dev)
-        for e, (_, down) in enumerate(self.experts):
-            if per_expert[e]:
-                down(y[starts[e]:starts[e + 1]], out=rows[starts[e]:starts[e + 1]])
+        if grouped:
+            sizes = [4 * len(t) for t in tables]
+            up_groups, down_groups = (meta[at + o:at + o + s].view(-1, 4) for o, s in zip((0, sizes[0]), sizes))
+            ops.linear_grouped(xs, self.gate_up, up_groups, plans[0], gu)
+            ops.moe_act(gu, self._ones(pairs, dev), y, self.limit, self.act)
+            ops.linear_grouped(y, self.down, down_groups, plans[1], rows)
+        else:
+            for e, (gate_up, _) in enumerate(self.experts):
+                if per_expert[e]:
+                    gate_up(xs[starts[e]:starts[e + 1]], out=gu[starts[e]:starts[e + 1]])
+            ops.moe_act(gu, self._ones(pairs, dev), y, self.limit, self.act)
+            for e, (_, down) in enumerate(self.experts):
+                if per_expert[e]:
+                    down(y[starts[e]:starts[e + 1]], out=rows[starts[e]:starts[e + 1]])
         ops.moe_combine(rows, chosen, rank, offsets, weights, h, accumulate=accumulate)
 
     def _ones(self, n: int, dev) -> torch.Tensor:

@@ -760,7 +760,9 @@ def moe_act(gu, dense, out, limit, act=0):
     out.copy_(y.reshape(n_tok, E * F).to(out.dtype))
 
 
-def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0):
+def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0, accumulate=True):
+    if not accumulate:
+        out.zero_()
     n_tok, K = x.shape
     _, N, F = down.shape
     gu = gate_up.double().view(n_experts, 2, F, K)
@@ -782,6 +784,16 @@ def gated_expert_act(gu, out):
     F = out.shape[1]
     g, u, z = gu[:, :F].double(), gu[:, F:2 * F].double(), gu[:, 2 * F:2 * F + 1].double()
     out.copy_((g * torch.sigmoid(g) * u * torch.sigmoid(z)).to(out.dtype))
+
+
+def grouped_plan(counts, n, k):
+    return 2
+
+
+def linear_grouped(x, weights, groups, variant, out):
+    out.fill_(float("nan"))
+    for first, rows, g, _ in groups.tolist():
+        out[first:first + rows] = (x[first:first + rows].double() @ weights[g].double().T).float()
 
 
 def moe_group(chosen, n_experts, rank, counts):
@@ -887,7 +899,8 @@ NAMES = ["embed", "rmsnorm", "gather_rows", "swiglu", "convert", "fill_normal", 
          "qkv_conv_prep", "capped_attn", "capped_mfma_takes", "capped_attn_prefill", "moe_route", "moe_act", "moe_sparse", "moe_group", "moe_gather", "moe_combine",
          "add_rows", "gr_chunks", "gated_scan", "head_rmsnorm", "qk_norm_prep", "unrotate", "softcap",
          "layernorm", "layernorm_join", "rmsnorm_pair", "relu2", "low_rank_scan", "retention_scan", "memory_scan",
-         "gated_head_norm", "qk_row_prep", "moe_table", "gated_expert_act"]
+         "gated_head_norm", "qk_row_prep", "moe_table", "gated_expert_act",
+         "grouped_plan", "linear_grouped"]
 
 
 def install(monkeypatch):

@@ -358,6 +358,44 @@ def test_choices_from_a_table_and_the_shared_experts_activation():
             assert ((got.cpu() - want).abs() / want.abs().clamp(min=1.0)).max() < tol
 
 
+@pytest.mark.parametrize("E, F, K, N, top", [(8, 64, 64, 16, 1), (8, 128, 192, 48, 2), (3, 4096, 2048, 2048, 1), (16, 320, 4096, 96, 8), (1, 64, 128, 64, 1),
+                                             (5, 64, 100, 30, 3)])
+@pytest.mark.parametrize("act", [0, 1])
+def test_few_tokens_experts_on_the_matrix_cores(E, F, K, N, top, act):
+    """Bfloat16 sizes the matrix-core form takes (and one set it does not), one token to sixteen, choices that pile up
+    on one expert, added to what is there or stored over it."""
+    from minfer_amd.kernels import ops
+    w1, w2 = (rnd(E, 2 * F, K, seed=1) / K ** 0.5).bfloat16(), (rnd(E, N, F, seed=2) / F ** 0.5).bfloat16()
+    for n in (1, 7, min(16, 128 // top)):
+        x = rnd(n, K, seed=n).bfloat16()
+        for piled in (False, True):
+            g = torch.Generator().manual_seed(n)
+            chosen = torch.stack([torch.arange(top) if piled else torch.randperm(E, generator=g)[:top] for _ in range(n)]).to(torch.int32)
+            weights = rnd(n, top, seed=4)
+            for acc in (True, False):
+                want, got = rnd(n, N, seed=5), rnd(n, N, seed=5).to(DEV)
+                plain_ops.moe_sparse(x, w1, w2, chosen, weights, want, E, 1.5, act, accumulate=acc)
+                ops.moe_sparse(x.to(DEV), w1.to(DEV), w2.to(DEV), chosen.to(DEV), weights.to(DEV), got, E, 1.5, act, accumulate=acc)
+                assert (got.cpu() - want).abs().max() < 3e-2, (n, piled, acc)
+
+
+@pytest.mark.parametrize("variant", [2, 12, 13])
+@pytest.mark.parametrize("n, k", [(128, 64), (300, 192), (2048, 128), (96, 1024)])
+def test_products_of_rows_in_groups(variant, n, k):
+    """Groups of none, one, a tile's rows and one more, against each group's own matrix; rows of no group stay."""
+    from minfer_amd.kernels import ops
+    counts = [3, 0, 128, 129, 1, 257, 0, 256]
+    w = (rnd(len(counts), n, k, seed=1) / k ** 0.5).bfloat16()
+    x = rnd(sum(counts) + 5, k, seed=2).bfloat16()
+    table = torch.tensor(ops.row_groups(counts, variant), dtype=torch.int32)
+    want, got = torch.empty(x.shape[0], n), torch.full((x.shape[0], n), 7.0, device=DEV)
+    plain_ops.linear_grouped(x, w, table, variant, want)
+    ops.linear_grouped(x.to(DEV), w.to(DEV), table.to(DEV), variant, got)
+    got = got.cpu()
+    assert (got[:-5] - want[:-5]).abs().max() < 2e-3 and bool((got[-5:] == 7.0).all())
+    assert ops.grouped_plan(counts, n, k) in ops.GROUPED_TILES
+
+
 # ------------------------------------------------------------------ the engine
 @pytest.fixture(scope="module")
 def folders(tmp_path_factory):
