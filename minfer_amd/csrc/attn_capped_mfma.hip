@@ -35,6 +35,7 @@ namespace {
 constexpr int D = MF_CAPM_D, V = MF_CAPM_V;
 constexpr int DKS = (D + 31) / 32;     // k steps of the first product
 constexpr int NVT = V / 16;            // output tiles
+constexpr float RAISE = 6.0f;          // how far scores may pass the softmax's reference before it is raised
 static_assert(D % 16 == 0 && V % 16 == 0 && D <= 256 && V <= 256, "sizes the kernel takes");
 
 typedef short short4v __attribute__((ext_vector_type(4)));
@@ -65,9 +66,9 @@ __device__ __forceinline__ void bias_run(const float* __restrict__ row, int n, i
 }
 
 __device__ __forceinline__ float fast_tanh(float y) {
-  // 1 - 2 / (e^(2y) + 1), exact at both ends
+  // 1 - 2 / (e^(2y) + 1), exact at both ends (the reciprocal to one unit in the last place: an absolute error of 1e-7)
   const float e = __expf(2.0f * y);
-  return 1.0f - 2.0f / (e + 1.0f);
+  return fmaf(-2.0f, __builtin_amdgcn_rcpf(e + 1.0f), 1.0f);
 }
 
 template <int RB>
@@ -177,13 +178,15 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
       vlo[c] = *(const short4v*)(vbase + (size_t)c * 16 * 32);
       vhi[c] = *(const short4v*)(vbase + (size_t)c * 16 * 32 + 16);
     }
-    // which of this lane's 8 keys its token sees: slot j < 4: key kb + 4 g + j, else kb + 16 + 4 g + j - 4
+    // which of this lane's 8 keys its token sees: slot j < 4: key kb + 4 g + j, else kb + 16 + 4 g + j - 4.  Most steps
+    // of a long walk lie wholly in sight of all the tile's tokens
+    const bool all_seen = rows == 16 && kb + 31 <= p0 && (window <= 0 || p_last - kb < window) && (chunk <= 0 || kb >= p_last / chunk * chunk);
     bool seen[8];
     float dist[8];
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int key = kb + (j < 4 ? 4 * g + j : 16 + 4 * g + j - 4);
-      seen[j] = row_ok && key <= p_mine && (window <= 0 || p_mine - key < window || key < keep_first) && key >= chunk_lo;
+      seen[j] = all_seen || (row_ok && key <= p_mine && (window <= 0 || p_mine - key < window || key < keep_first) && key >= chunk_lo);
       dist[j] = (float)max(0, p_mine - key);
     }
     bf16x8 pf[RB];
@@ -196,7 +199,6 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
         s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][ks], qf[r][ks], s1, 0, 0, 0);
       }
       float x[8];
-      float mx = -INFINITY;
       float add_lo[4] = {0.f, 0.f, 0.f, 0.f}, add_hi[4] = {0.f, 0.f, 0.f, 0.f};
       if (bias) {        // this lane's keys are two runs of four neighbours, 16 keys apart
         const float* brow = bias + (size_t)(h0 + r) * n_bias;
@@ -204,31 +206,51 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
         bias_run(brow, n_bias, p_mine - (kb + 16 + 4 * g), add_hi);
       }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        float y = (j < 4 ? s0[j] : s1[j - 4]) * sc[r];
-        if (cap > 0.f) y = cap * fast_tanh(y * inv_cap);
-        if (far_a) y -= fa[r] * (far_b ? __logf(1.0f + fb[r] * dist[j]) : dist[j]);
-        if (bias) y += j < 4 ? add_lo[j] : add_hi[j - 4];
-        x[j] = seen[j] ? y : -INFINITY;
-        mx = fmaxf(mx, x[j]);
+      for (int j = 0; j < 8; ++j) x[j] = (j < 4 ? s0[j] : s1[j - 4]) * sc[r];
+      if (cap > 0.f) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = cap * fast_tanh(x[j] * inv_cap);
       }
+      if (far_b) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] -= fa[r] * __logf(1.0f + fb[r] * dist[j]);
+      } else if (far_a) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = fmaf(-fa[r], dist[j], x[j]);
+      }
+      if (bias) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] += j < 4 ? add_lo[j] : add_hi[j - 4];
+      }
+      if (!all_seen) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = seen[j] ? x[j] : -INFINITY;
+      }
+      float mx = fmaxf(fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3])), fmaxf(fmaxf(x[4], x[5]), fmaxf(x[6], x[7])));
       mx = fmaxf(mx, __shfl_xor(mx, 16, MF_WAVE));
       mx = fmaxf(mx, __shfl_xor(mx, 32, MF_WAVE));
-      const float m_new = fmaxf(m[r], mx);
-      const float corr = m[r] == -INFINITY ? 1.f : __expf(m[r] - m_new);
+      // The sums are kept relative to a score m that some token's keys have passed by less than RAISE (or not at
+      // all): only when a token's keys pass it by more is m raised and what was summed scaled down.  The
+      // probabilities then stay below e^RAISE, and a result is sums over weight whatever m is.
+      if (__any(mx > m[r] + RAISE)) {
+        const float m_new = fmaxf(m[r], mx);
+        const float corr = m[r] == -INFINITY ? 1.f : __expf(m[r] - m_new);
+        l[r] *= corr;
+        m[r] = m_new;
+#pragma unroll
+        for (int c = 0; c < NVT; ++c) oacc[r][c] *= corr;
+      }
       float sum = 0.f;
       bf16x8 p;
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const float pe = seen[j] ? __expf(x[j] - m_new) : 0.f;
+        float pe = __expf(x[j] - m[r]);
+        if (!all_seen) pe = seen[j] ? pe : 0.f;        // (a token that has seen no key yet has no m)
         sum += pe;
         p[j] = (bf16)pe;
       }
       pf[r] = p;
-      l[r] = l[r] * corr + sum;
-      m[r] = m_new;
-#pragma unroll
-      for (int c = 0; c < NVT; ++c) oacc[r][c] *= corr;
+      l[r] += sum;
     }
     const bool tail = kb + 32 > seq_end;           // some of these keys were never written
 #pragma unroll

@@ -113,15 +113,38 @@ __global__ __launch_bounds__(256) void qk_row_prep_kernel(
     }
     return;
   }
+  // a row of at most 256 KEEP values stays in registers between the sum and the scaling
+  constexpr int KEEP = 16;
+  const float* gain = kind == 0 ? q_gain : k_gain;
+  const bool kept = n <= 256 * KEEP;
+  float xv[KEEP];
   float ss = 0.f;
-  for (int i = threadIdx.x; i < n; i += 256) ss = fmaf(row[i], row[i], ss);
+  if (kept) {
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = c * 256 + threadIdx.x;
+      xv[c] = i < n ? row[i] : 0.f;
+    }
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) ss = fmaf(xv[c], xv[c], ss);
+  } else {
+    for (int i = threadIdx.x; i < n; i += 256) ss = fmaf(row[i], row[i], ss);
+  }
   float r = 1.0f / sqrtf(block_sum<256>(ss, scratch) / (float)n + eps);
   if (kind == 0 && temp_every > 0) r *= 1.0f + temp_coef * logf((float)((p + 1) / temp_every) + 1.0f);
-  const float* gain = kind == 0 ? q_gain : k_gain;
-  for (int i = threadIdx.x; i < n; i += 256) {
-    const T v = from_f32<T>(row[i] * r * gain[i]);
+  auto put = [&](int i, float x) {
+    const T v = from_f32<T>(x * r * gain[i]);
     if (kind == 0) q_out[(size_t)t * n + i] = v;
     else kc[(((size_t)page * G + i / D) * MF_PAGE + in_page) * D + i % D] = v;
+  };
+  if (kept) {
+#pragma unroll
+    for (int c = 0; c < KEEP; ++c) {
+      const int i = c * 256 + threadIdx.x;
+      if (i < n) put(i, xv[c]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < n; i += 256) put(i, row[i]);
   }
 }
 

@@ -38,7 +38,7 @@ __device__ __forceinline__ float gr_sigmoid(float x) { return 1.0f / (1.0f + exp
 #define MF_GR_DECAYS 2
 
 struct LowRankGate {
-  const float* a2;        // [H D][rank]
+  const float* a2;        // [rank][H D]
   const float* bias;      // [H D]
   const float* decays;    // [tokens][H D] (MF_GR_DECAYS)
   int rank, off_r;
@@ -113,9 +113,10 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(const float* __restrict
             av = lr.decays[(size_t)(tb + tt) * H * D + h * D + d];
           } else {
             const float* r = proj + (size_t)(tb + tt) * row_len + lr.off_r;
-            const float* w = lr.a2 + (size_t)(h * D + d) * lr.rank;
+            const float* w = lr.a2 + h * D + d;
             float z = lr.bias[h * D + d];
-            for (int i2 = 0; i2 < lr.rank; ++i2) z = fmaf(w[i2], r[i2], z);
+#pragma unroll 8
+            for (int i2 = 0; i2 < lr.rank; ++i2) z = fmaf(w[(size_t)i2 * H * D], r[i2], z);
             av = root_sigmoid(z, lr.inv_tau);
           }
         }
@@ -201,7 +202,7 @@ __global__ __launch_bounds__(256) void head_rmsnorm_kernel(const float* __restri
   }
 }
 
-// decays[t][d] = sigmoid(bias[d] + a2[d][:] . r_t)^(1/tau) for MF_GR_LR_TOKENS tokens a workgroup, a thread a
+// decays[t][d] = sigmoid(bias[d] + a2[:][d] . r_t)^(1/tau) for MF_GR_LR_TOKENS tokens a workgroup, a thread a
 // channel; r_t is the columns off_r .. of the token's row
 #define MF_GR_LR_TOKENS 16
 #define MF_GR_LR_RANK 64      // values of r staged together
@@ -221,12 +222,14 @@ __global__ __launch_bounds__(256) void low_rank_decay_kernel(const float* __rest
       sr[t][r] = t < nt ? proj[(size_t)(t0 + t) * row_len + lr.off_r + r0 + r] : 0.f;
     }
     __syncthreads();
-    if (d < C)
+    if (d < C) {
+#pragma unroll 8
       for (int r = 0; r < nr; ++r) {
-        const float w = lr.a2[(size_t)d * lr.rank + r0 + r];
+        const float w = lr.a2[(size_t)(r0 + r) * C + d];
 #pragma unroll
         for (int t = 0; t < MF_GR_LR_TOKENS; ++t) z[t] = fmaf(w, sr[t][r], z[t]);
       }
+    }
   }
   if (d >= C) return;
 #pragma unroll
@@ -303,7 +306,7 @@ MF_API int mf_gated_scan_chunked(const float* proj, const float* lower, const in
 }
 
 // rows of row_len floats: q [H D] | k [H D] | v [H V] | ..., the gate's r in the columns off_r ..; a2 float32
-// [H D][rank]; n_chunks 0: every sequence in one walk; decays float32 [tokens][H D], scratch of the chunked form
+// [rank][H D]; n_chunks 0: every sequence in one walk; decays float32 [tokens][H D], scratch of the chunked form
 MF_API int mf_low_rank_scan(const float* proj, int row_len, const float* a2, const float* bias, int rank, int off_r,
                             float inv_tau, float q_scale, const int* cu_seqlens, const int* chunks, int n_chunks,
                             const int* seq_first_chunk, const int* slot_ids, float* state, float* ws, float* ws_a,

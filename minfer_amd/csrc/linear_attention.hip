@@ -416,12 +416,15 @@ __global__ __launch_bounds__(256) void lightning_chunk_fold_kernel(const int* __
   float* st = is_n ? slot + (size_t)H * DV + (size_t)h * D + (e - DV) : slot + (size_t)h * DV + e;
   float* first = is_n ? ex.n_ws + (size_t)h * D + (e - DV) : bsum + (size_t)h * DV + e;
   const size_t stride = (size_t)H * (is_n ? D : DV);
+  const float whole = powf(decay, (float)MF_LA_CHUNK);      // a whole chunk's decay
   float S = *st;
   for (int c = c0; c < c1; ++c) {
     float* b = first + c * stride;
     const float B = *b;
     *b = S;
-    S = fmaf(KIND == MF_LA_MEMORY ? ex.chunk_decay[(size_t)c * H + h] : powf(decay, (float)chunk_n[c]), S, B);
+    S = fmaf(KIND == MF_LA_MEMORY ? ex.chunk_decay[(size_t)c * H + h]
+                                     : (chunk_n[c] == MF_LA_CHUNK ? whole : powf(decay, (float)chunk_n[c])),
+             S, B);
   }
   *st = S;
 }

@@ -741,13 +741,13 @@ def low_rank_scan(proj: torch.Tensor, a2: torch.Tensor, bias: torch.Tensor, off_
                   cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n_heads: int,
                   dim: int, v_dim: int, chunks=None) -> None:
     """Gated linear attention, S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t q_scale, with
-    a_t = sigmoid(a2 r_t + bias)^(1/tau), over a ragged step.  `proj` float32 rows that begin with q `[H dim]` |
-    k `[H dim]` | v `[H v_dim]` and hold r in the columns `off_r ..`; `a2` float32 `[H dim][rank]`; the rest as
+    a_t = sigmoid(a2^T r_t + bias)^(1/tau), over a ragged step.  `proj` float32 rows that begin with q `[H dim]` |
+    k `[H dim]` | v `[H v_dim]` and hold r in the columns `off_r ..`; `a2` float32 `[rank][H dim]`; the rest as
     `gated_scan`."""
     n_tok, row_len = proj.shape
-    n_seqs, rank = slot_ids.numel(), a2.shape[1]
+    n_seqs, rank = slot_ids.numel(), a2.shape[0]
     _need(proj, "low_rank_scan.proj", torch.float32)
-    _need(a2, "low_rank_scan.a2", torch.float32, (n_heads * dim, rank))
+    _need(a2, "low_rank_scan.a2", torch.float32, (rank, n_heads * dim))
     _need(bias, "low_rank_scan.bias", torch.float32, (n_heads * dim,))
     _need(cu_seqlens, "low_rank_scan.cu_seqlens", torch.int32, (n_seqs + 1,))
     _need(slot_ids, "low_rank_scan.slot_ids", torch.int32, (n_seqs,))
@@ -1260,7 +1260,7 @@ def capped_attn_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Ten
         if chunk:
             reach = min(reach, int(chunk))
         waves = n_tok * n_kv_heads * max(1, (n_heads // n_kv_heads) // 2)
-        n_splits = max(1, min(4 * cu_count() // max(1, waves), (reach + 31 + 127) // 128, 64))
+        n_splits = max(1, min(8 * cu_count() // max(1, waves), (reach + 31 + 127) // 128, 64))
         split_len = (((reach + 31 + n_splits - 1) // n_splits) + 31) // 32 * 32
         n_splits = (reach + 31 + split_len - 1) // split_len
         if n_splits > 1:

@@ -121,7 +121,7 @@ class GatedLinearAttention(Mixer):
         self.proj = Linear.stacked([get(n[k]) for k in ("q", "k", "v", "g", "a1")])      # one product
         self.o = Linear(get(n["o"]))
         self.norm_weight = get(n["norm"]).to(torch.float32).contiguous()
-        self.a2 = get(n["a2"]).to(torch.float32).contiguous()
+        self.a2 = get(n["a2"]).to(torch.float32).t().contiguous()      # [rank][heads dim], as the kernels read it
         self.a2_bias = get(n["a2_bias"]).to(torch.float32).contiguous()
 
     def cache_request(self):

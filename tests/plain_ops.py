@@ -633,7 +633,7 @@ def _walk(state_rows, keep, k, v, q, out, cu_seqlens, slot_ids):
 def low_rank_scan(proj, a2, bias, off_r, tau, q_scale, cu_seqlens, slot_ids, state, out, n_heads, dim, v_dim, chunks=None):
     H, D, V = n_heads, dim, v_dim
     p = proj.double()
-    z = p[:, off_r:off_r + a2.shape[1]] @ a2.double().T + bias.double()
+    z = p[:, off_r:off_r + a2.shape[0]] @ a2.double() + bias.double()
     keep = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(-1, H, D)
     _walk(state, keep, _heads(p, H * D, H, D), _heads(p, 2 * H * D, H, V), _heads(p, 0, H, D) * q_scale, out, cu_seqlens, slot_ids)
 

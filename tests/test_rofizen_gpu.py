@@ -140,7 +140,7 @@ NEW = [(1,), (5, 64, 1), (70, 3, 128, 200), (1, 1, 1, 1, 1), (65, 63)]
 def test_gated_linear_attention_scan(H, D, V, rank, tau, new):
     """Decays from near 0 to near 1 (biases from -6 to 6), carried states, walks and chunks."""
     proj, slots, cu, state = _scan_case(new, rank + 7, H, D, V, 3, (H, D, V))
-    a2, bias = rnd(H * D, rank, seed=5, scale=1.0 / rank ** 0.5), rnd(H * D, seed=6, scale=3.0)
+    a2, bias = rnd(rank, H * D, seed=5, scale=1.0 / rank ** 0.5), rnd(H * D, seed=6, scale=3.0)
     off = H * (2 * D + V) + 4
 
     def run(o, p, st, outs, chunked):
