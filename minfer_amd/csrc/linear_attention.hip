@@ -28,7 +28,8 @@
 // f = logsigmoid(cap tanh(zf / cap)) of a token and a running maximum m that starts at 0,
 //   m_t = max(f + m_(t-1), i),  S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k_t v_t^T,  n_t likewise with k
 // alone; the kernels leave S_t^T q_t, n_t . q_t and exp(-m_t), and what follows divides.  A slot's state holds
-// S [H][D][V], then n [H][D], then m [H].  In the chunked form `memory_gates_kernel` first walks m along every
+// S [H][D][V], then n [H][D], then m [H][column blocks]: the workgroups of a head's column blocks all walk m, each
+// from and into a copy of its own, since one may end before another begins.  In the chunked form `memory_gates_kernel` first walks m along every
 // sequence (a scan over (f, i) pairs under m -> max(m + f, i)), and leaves for every token the sum since its
 // chunk's start of the logarithms of the factors on S (in double: differences of two of them weigh the pairs
 // of tokens inside the chunk), the logarithm of its own weight, and exp(-m_t).
@@ -69,10 +70,13 @@ __device__ __forceinline__ float la_silu(float x) { return x * la_sigmoid(x); }
 __device__ __forceinline__ float la_log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float la_cap(float x, float cap) { return cap * tanhf(x / cap); }
 
+// copies of m a head keeps: one per block of 64 value columns
+__host__ __device__ __forceinline__ int la_m_copies(int V) { return (V + 63) / 64; }
+
 // floats of a slot's state
 template <int KIND>
 __device__ __forceinline__ size_t la_state_len(int H, int D, int V) {
-  return KIND == MF_LA_MEMORY ? (size_t)H * ((size_t)D * V + D + 1) : (size_t)H * D * V;
+  return KIND == MF_LA_MEMORY ? (size_t)H * ((size_t)D * V + D + la_m_copies(V)) : (size_t)H * D * V;
 }
 
 // value d of head `hd` of a row's q or k part: rotated in halves by the token's angles where it is to be
@@ -105,7 +109,7 @@ __global__ __launch_bounds__(256) void lightning_scan_kernel(const float* __rest
   float* slot = state + (size_t)slot_ids[seq] * la_state_len<KIND>(H, D, V);
   float* st = slot + ((size_t)h * D) * V + col;
   float* st_n = slot + (size_t)H * D * V + (size_t)h * D;
-  float* st_m = slot + (size_t)H * D * V + (size_t)H * D + h;
+  float* st_m = slot + (size_t)H * D * V + (size_t)H * D + (size_t)h * la_m_copies(V) + blockIdx.z;
   // n: lane l of a wave keeps value slice DS + l (the workgroup of the first columns alone); m: thread 0 alone
   const int lane = threadIdx.x & 63;
   const int dn = slice * DS + lane;
@@ -202,7 +206,7 @@ __global__ __launch_bounds__(256) void lightning_scan_kernel(const float* __rest
       if (d < D) st[(size_t)d * V] = S[i];
     }
   }
-  if (KIND == MF_LA_MEMORY && blockIdx.z == 0) {
+  if (KIND == MF_LA_MEMORY) {
     if (has_n) st_n[dn] = nn;
     if (threadIdx.x == 0) *st_m = m;
   }
@@ -235,7 +239,9 @@ __global__ __launch_bounds__(64 * MF_LA_GATE_WAVES) void memory_gates_kernel(
   const int seq = blockIdx.x, h = blockIdx.y;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int t0 = cu_seqlens[seq], t1 = cu_seqlens[seq + 1];
-  float* st_m = state + (size_t)slot_ids[seq] * la_state_len<MF_LA_MEMORY>(H, D, V) + (size_t)H * D * V + (size_t)H * D + h;
+  const int copies = la_m_copies(V);
+  float* st_m = state + (size_t)slot_ids[seq] * la_state_len<MF_LA_MEMORY>(H, D, V) + (size_t)H * D * V + (size_t)H * D +
+                (size_t)h * copies;
   float m = *st_m;                 // the maximum before the round's first token
   for (int base = t0; base < t1; base += 64 * MF_LA_GATE_WAVES) {
     const int t = base + threadIdx.x;
@@ -283,7 +289,7 @@ __global__ __launch_bounds__(64 * MF_LA_GATE_WAVES) void memory_gates_kernel(
     if (lane == 63 && base + 64 * w < t1)
       chunk_decay[(size_t)(seq_first_chunk[seq] + (base - t0) / 64 + w) * H + h] = expf((float)L);
   }
-  if (threadIdx.x == 0) *st_m = m;
+  if (threadIdx.x < copies) st_m[threadIdx.x] = m;
 }
 static_assert(MF_LA_CHUNK == 64, "a wave of memory_gates_kernel takes a chunk");
 
@@ -703,7 +709,7 @@ MF_API int mf_retention_scan(float* proj, int row_len, const int* cu_seqlens, co
 }
 
 // rows as above, with the gates' projections in the columns off_i + h and off_f + h; state float32
-// [slots][H D V + H D + H]; den, floor float32 [tokens][H]; gates [tokens][H], chunk_decay [n_chunks][H] and n_ws
+// [slots][H (D V + D + column blocks)]; den, floor float32 [tokens][H]; gates [tokens][H], chunk_decay [n_chunks][H] and n_ws
 // [n_chunks][H][D] scratch of the chunked form
 MF_API int mf_memory_scan(const float* proj, int row_len, const int* cu_seqlens, const int* chunks, int n_chunks,
                           const int* seq_first_chunk, const int* slot_ids, float q_scale, float k_scale, int off_i, int off_f,

@@ -992,8 +992,9 @@ MEMORY_GATE_FLOATS = 4       # floats of a token's and head's entry in the gates
 
 
 def memory_state_len(n_heads: int, dim: int, v_dim: int) -> int:
-    """Floats of a slot's state of the matrix memory: S `[H][dim][v_dim]`, n `[H][dim]`, m `[H]`."""
-    return n_heads * (dim * v_dim + dim + 1)
+    """Floats of a slot's state of the matrix memory: S `[H][dim][v_dim]`, n `[H][dim]`, m `[H]` in a copy for every
+    block of 64 value columns (whose workgroups each walk m and may not wait for one another)."""
+    return n_heads * (dim * v_dim + dim + (v_dim + 63) // 64)
 
 
 def memory_scan(proj: torch.Tensor, off_i: int, off_f: int, cap: float, q_scale: float, cu_seqlens: torch.Tensor,

@@ -658,7 +658,7 @@ def memory_scan(proj, off_i, off_f, cap, q_scale, cu_seqlens, slot_ids, state, o
     gate_f = torch.nn.functional.logsigmoid(cap * torch.tanh(p[:, off_f:off_f + H] / cap))
     for b in range(slot_ids.numel()):
         row = state[int(slot_ids[b])]
-        S, n, m = (row[:H * D * V].double().view(H, D, V), row[H * D * V:H * D * (V + 1)].double().view(H, D), row[H * D * (V + 1):].double())
+        S, n, m = (row[:H * D * V].double().view(H, D, V), row[H * D * V:H * D * (V + 1)].double().view(H, D), row[H * D * (V + 1):].double().view(H, -1)[:, 0])
         for t in range(int(cu_seqlens[b]), int(cu_seqlens[b + 1])):
             top = torch.maximum(gate_f[t] + m, gate_i[t])
             keep, take = torch.exp(gate_f[t] + m - top), torch.exp(gate_i[t] - top)
@@ -668,7 +668,7 @@ def memory_scan(proj, off_i, off_f, cap, q_scale, cu_seqlens, slot_ids, state, o
             out[t] = torch.einsum("hdv,hd->hv", S, q[t]).reshape(-1).float()
             den[t] = (n * q[t]).sum(dim=-1).float()
             floor[t] = torch.exp(-m).float()
-        state[int(slot_ids[b])] = torch.cat([S.reshape(-1), n.reshape(-1), m]).float()
+        state[int(slot_ids[b])] = torch.cat([S.reshape(-1), n.reshape(-1), m.repeat_interleave((V + 63) // 64)]).float()
 
 
 def gated_head_norm(o, proj, gate_offset, weight, eps, out, n_heads, act, den=None, floor=None):

@@ -178,11 +178,13 @@ def test_matrix_memory_scan(H, D, V, cap, shift, new):
     takes."""
     if sum(new) > 1000 and H * D * V > 10000:
         pytest.skip("the stand-in walks every token on the host")
+    from minfer_amd.kernels.ops import memory_state_len
     extra = 2 * H + 3
-    proj, slots, cu, state = _scan_case(new, extra, H, D, V, 23, (H * (D * V + D + 1),))
+    proj, slots, cu, state = _scan_case(new, extra, H, D, V, 23, (memory_state_len(H, D, V),))
     off = H * (2 * D + V) + 1
     proj[:, off:] = proj[:, off:] * 4.0 + shift
-    state[:, -H:] *= 3.0
+    copies = (V + 63) // 64          # of every head's running maximum, all alike
+    state[:, -H * copies:] = (3.0 * rnd(9, H, seed=29)).repeat_interleave(copies, dim=1)
     n = sum(new)
 
     def run(o, p, st, outs, chunked):
@@ -216,6 +218,30 @@ def test_the_memory_remembers_a_token_among_a_thousand():
             at += m
         got = (out[-1].view(H, V) / den[-1][:, None]).cpu()
         assert (got - want).abs().max() < 0.05, cuts
+
+
+def test_blocks_of_value_columns_do_not_see_each_others_state():
+    """Many more workgroups than fit the chip at once, several for the value columns of one head: a workgroup that
+    begins when another of its head has ended must start from what the state was before the step, for every sequence
+    and head alike; the same sequence in every slot gives the same rows."""
+    from minfer_amd.kernels import ops
+    n, H, D, V = 96, 16, 64, 256
+    off = H * (2 * D + V)
+    row = rnd(1, off + 2 * H, seed=3)
+    row[:, off:off + H] = 1.0 + rnd(1, H, seed=4).abs()            # input gates that raise the maximum every step
+    row[:, off + H:] = 3.0
+    proj = row.repeat(n, 1).to(DEV)
+    slots, cu = torch.arange(n, dtype=torch.int32, device=DEV), torch.arange(n + 1, dtype=torch.int32, device=DEV)
+    state = torch.zeros(n, ops.memory_state_len(H, D, V), device=DEV)
+    want_state, want = state[:1].cpu(), [torch.empty(1, H * V), torch.empty(1, H), torch.empty(1, H)]
+    for step in range(4):
+        proj[:, off:off + H] += 0.7
+        outs = [torch.empty(n, H * V, device=DEV), torch.empty(n, H, device=DEV), torch.empty(n, H, device=DEV)]
+        ops.memory_scan(proj, off, off + H, 12.0, D ** -0.5, cu, slots, state, *outs, H, D, V)
+        plain_ops.memory_scan(proj[:1].cpu(), off, off + H, 12.0, D ** -0.5, torch.tensor([0, 1]), torch.tensor([0]), want_state, *want, H, D, V)
+        for a, b in zip(outs, want):
+            assert ((a.cpu() - b).abs() / b.abs().clamp(min=1.0)).max() < 1e-4, step
+    assert torch.equal(state, state[:1].expand(n, -1)) and (state[:1].cpu() - want_state).abs().max() < 1e-3
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
