@@ -15,11 +15,11 @@ of its own: one K tensor `[entries][pages][kv_heads][64][head_dim]`, one V tenso
 in 32-bit, `[entries][pages][kv_heads][2][head_dim][32]` in bfloat16, see `v_page_shape`; with the
 request's own value width where it names one) and one page pool.
 A group with a window gives pages back as soon as every position in them has left the
-window of all later queries.
+window of all later queries (of every layer that reads the entry, see `widest_request`).
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
@@ -73,6 +73,23 @@ class StateRequest:
     """Fixed-size state per sequence for one entry (zeroed when a slot is taken)."""
     shape: Tuple[int, ...]
     dtype: torch.dtype = torch.float32
+
+
+def widest_request(owner: KVRequest, reader: KVRequest) -> KVRequest:
+    """What an entry needs that is written for `owner` and also read for `reader`: every position either of them still
+    sees.  Rows of other sizes cannot be shared; a window beside a chunk (or either beside neither) keeps everything."""
+    sizes = [(r.n_kv_heads, r.head_dim, r.value_dim) for r in (owner, reader)]
+    if sizes[0] != sizes[1]:
+        raise CacheError(f"an entry of {sizes[0]} (kv heads, key width, value width) cannot be read as {sizes[1]}")
+
+    def most(a, b):
+        return None if a is None or b is None else max(a, b)
+    if owner.chunk == reader.chunk:          # chunks of two lengths, one within the other or not, have no common form
+        window, chunk = most(owner.window, reader.window), owner.chunk
+    else:
+        window = chunk = None
+    keep = max(owner.keep_first or 0, reader.keep_first or 0) or None
+    return replace(owner, window=window, chunk=chunk, keep_first=keep if window is not None else None)
 
 
 def split_request(req):

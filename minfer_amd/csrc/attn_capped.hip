@@ -14,7 +14,9 @@
 // s_j -= a[h] (p - j) (behind the cap, like everything that joins the score), a number per
 // head and distance that joins the score, s_j += bias[h][min(p - j, n_bias - 1)] (a table the host lays out by
 // distance, whatever rule groups the distances), and, with a window, the sequence's first `keep_first`
-// positions, which every later token goes on seeing (split 0 walks them before its own keys).
+// positions, which every later token goes on seeing (split 0 walks them before its own keys).  With `sink`, a number per
+// head, the softmax's denominator also holds e^sink[h], as a key without a value would add it: split 0 starts its
+// maximum from the sink and its weight from one.
 //
 // `qkv_conv_prep_kernel`: one workgroup per (token, head of q, k or v); convolution of the head's channels
 // into LDS, then rotation, blending, the cache write and q rounded to the run type.
@@ -129,8 +131,8 @@ __global__ __launch_bounds__(256) void capped_attn_kernel(
     int pt_stride, const int* __restrict__ positions, const int* __restrict__ seq_of_tok,
     const float* __restrict__ temp, T* __restrict__ out, float* __restrict__ part, int nh, int nk, int D, int V,
     int VP, float scale, float cap, int window, int chunk, const float* __restrict__ far_a,
-    const float* __restrict__ far_b, int keep_first, const float* __restrict__ bias, int n_bias, int n_splits,
-    int split_len) {
+    const float* __restrict__ far_b, int keep_first, const float* __restrict__ bias, int n_bias,
+    const float* __restrict__ sink, int n_splits, int split_len) {
   extern __shared__ float lds[];
   float* sq = lds;                              // [GC][D]
   float* sc = sq + MF_CAP_GC * D;               // [GC][KEYS]
@@ -157,7 +159,12 @@ __global__ __launch_bounds__(256) void capped_attn_kernel(
 
   for (int i = threadIdx.x; i < gcount * D; i += 256)
     sq[i] = to_f32(q[((size_t)t * nh + h0) * D + i]);
-  if (threadIdx.x < MF_CAP_GC) { sm_m[threadIdx.x] = -INFINITY; sm_l[threadIdx.x] = 0.f; sm_corr[threadIdx.x] = 1.f; }
+  if (threadIdx.x < MF_CAP_GC) {
+    const bool with_sink = sink && split == 0 && threadIdx.x < gcount;
+    sm_m[threadIdx.x] = with_sink ? sink[h0 + threadIdx.x] : -INFINITY;
+    sm_l[threadIdx.x] = with_sink ? 1.f : 0.f;
+    sm_corr[threadIdx.x] = 1.f;
+  }
   const int v = threadIdx.x % VP, ks = threadIdx.x / VP, KS = 256 / VP;
   float acc[MF_CAP_GC];
 #pragma unroll
@@ -358,7 +365,7 @@ MF_API int mf_capped_attn(const void* q, const void* kc, const void* vc, const i
                           const int* positions, const int* seq_of_tok, const float* temp, void* out, float* part,
                           int is_bf16, int n_tok, int nh, int nk, int D, int V, float scale, float cap, int window,
                           int chunk, const float* far_a, const float* far_b, int keep_first, const float* bias,
-                          int n_bias, int n_splits, int split_len, hipStream_t stream) {
+                          int n_bias, const float* sink, int n_splits, int split_len, hipStream_t stream) {
   if (n_tok <= 0) return 0;
   if (nk <= 0 || nh % nk || D <= 0 || D > 512 || V <= 0 || V > 256 || n_splits < 1 || n_splits > 64 ||
       split_len < 1 || (n_splits > 1 && !part) || !temp || chunk < 0 || (far_b && !far_a) ||
@@ -373,7 +380,7 @@ MF_API int mf_capped_attn(const void* q, const void* kc, const void* vc, const i
   if (is_bf16) {
     capped_attn_kernel<bf16><<<grid, 256, lds, stream>>>((const bf16*)q, (const bf16*)kc, (const bf16*)vc, page_table,
                                                          pt_stride, positions, seq_of_tok, temp, (bf16*)out, part, nh, nk,
-                                                         D, V, VP, scale, cap, window, chunk, far_a, far_b, keep_first, bias, n_bias, n_splits,
+                                                         D, V, VP, scale, cap, window, chunk, far_a, far_b, keep_first, bias, n_bias, sink, n_splits,
                                                          split_len);
     rc = mf_launch_status();
     if (rc == 0 && n_splits > 1) {
@@ -383,7 +390,7 @@ MF_API int mf_capped_attn(const void* q, const void* kc, const void* vc, const i
   } else {
     capped_attn_kernel<float><<<grid, 256, lds, stream>>>((const float*)q, (const float*)kc, (const float*)vc, page_table,
                                                           pt_stride, positions, seq_of_tok, temp, (float*)out, part, nh,
-                                                          nk, D, V, VP, scale, cap, window, chunk, far_a, far_b, keep_first, bias, n_bias, n_splits,
+                                                          nk, D, V, VP, scale, cap, window, chunk, far_a, far_b, keep_first, bias, n_bias, sink, n_splits,
                                                          split_len);
     rc = mf_launch_status();
     if (rc == 0 && n_splits > 1) {

@@ -5,7 +5,8 @@
 // `chunk`, a token sees the keys of its own chunk of that many positions only; with `far_a`, `far_b`,
 // s -= far_a[h] ln(1 + far_b[h] (p - j)), and with `far_a` alone s -= far_a[h] (p - j); with `bias`, s += bias[h][min(p - j, n_bias - 1)]; with a window and
 // `keep_first`, every token also sees the sequence's first `keep_first` keys: the wave of split 0 walks their
-// half pages first and then jumps to the half page of its window's first key.
+// half pages first and then jumps to the half page of its window's first key; with `sink`, a number per head, the
+// denominator also holds e^sink[h] (split 0 starts from it as from a key without a value).
 //
 // A wave (a workgroup of its own) owns 16 consecutive new tokens of one sequence times RB query heads of one kv
 // head and walks the tokens' keys 32 at a time (half a page), with no LDS and no barrier; the key rows of a
@@ -78,7 +79,8 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
     const int* __restrict__ start_pos, const int* __restrict__ tile_seq, const int* __restrict__ tile_q0, int n_tiles,
     const float* __restrict__ temp, bf16* __restrict__ out, float* __restrict__ part, int n_splits, int split_len,
     int nh, int nk, float scale, float cap, int window, int chunk, const float* __restrict__ far_a,
-    const float* __restrict__ far_b, int keep_first, const float* __restrict__ bias, int n_bias) {
+    const float* __restrict__ far_b, int keep_first, const float* __restrict__ bias, int n_bias,
+    const float* __restrict__ sink) {
   const int lane = threadIdx.x & 63;
   const int tile = blockIdx.x;                    // a workgroup is one wave: the waves drift apart freely
   if (tile >= n_tiles) return;
@@ -137,8 +139,9 @@ __global__ __launch_bounds__(64) void capped_mfma_kernel(
   float m[RB], l[RB];
 #pragma unroll
   for (int r = 0; r < RB; ++r) {
-    m[r] = -INFINITY;
-    l[r] = 0.f;
+    // the sink weighs one against itself; a token's weight is spread over four lanes, of which one counts it
+    m[r] = sink && split == 0 ? sink[h0 + r] : -INFINITY;
+    l[r] = sink && split == 0 && g == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int c = 0; c < NVT; ++c) oacc[r][c] = floatx4{0.f, 0.f, 0.f, 0.f};
   }
@@ -316,7 +319,8 @@ MF_API int mf_capped_mfma(const void* q, const void* kc, const void* vc, const i
                           const int* cu_seqlens, const int* start_pos, const int* tile_seq, const int* tile_q0,
                           int n_tiles, const float* temp, void* out, float* part, int n_splits, int split_len, int n_tok,
                           int nh, int nk, int d, int v, float scale, float cap, int window, int chunk, const float* far_a,
-                          const float* far_b, int keep_first, const float* bias, int n_bias, hipStream_t stream) {
+                          const float* far_b, int keep_first, const float* bias, int n_bias, const float* sink,
+                          hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   if (d != D || v != V || nk <= 0 || nh % nk || !temp || n_splits < 1 || n_splits > 64 ||
       (n_splits > 1 && (!part || split_len < 32 || split_len % 32)) || chunk < 0 ||
@@ -332,7 +336,7 @@ MF_API int mf_capped_mfma(const void* q, const void* kc, const void* vc, const i
   capped_mfma_kernel<RB><<<grid, 64, 0, stream>>>((const bf16*)q, (const bf16*)kc, (const bf16*)vc, page_table, pt_stride, \
                                                    cu_seqlens, start_pos, tile_seq, tile_q0, n_tiles, temp, (bf16*)out, part, \
                                                    n_splits, split_len, nh, nk, scale, cap, window, chunk, far_a, far_b, \
-                                                   keep_first, bias, n_bias)
+                                                   keep_first, bias, n_bias, sink)
   if (rb == 4) MF_GO(4);
   else if (rb == 2) MF_GO(2);
   else MF_GO(1);

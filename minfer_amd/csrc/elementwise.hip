@@ -33,6 +33,62 @@ MF_API int mf_embed(const void* table, int table_is_bf16, const int* ids, float*
   return mf_launch_status();
 }
 
+// ---------------------------------------------------------------- table row + row of the pair with the token before
+// out[t][:] = table[ids[t]][:] scale + pairs[row][:], row = (previous mul_prev + id mul_cur) mod buckets, and row
+// `buckets` for a sequence's first token.  The previous token is the one ahead in the step, or, for the first token a
+// sequence brings, its state `last[slot]`; the workgroup of that token also leaves the sequence's last token there, so
+// that one workgroup reads and writes a slot's state.  An id outside the table gives a row of NaN, as `embed_kernel` does.
+template <typename TT>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(const TT* __restrict__ table, const TT* __restrict__ pairs,
+                                                          const int* __restrict__ ids, const int* __restrict__ positions,
+                                                          const int* __restrict__ seq_of_tok,
+                                                          const int* __restrict__ cu_seqlens,
+                                                          const int* __restrict__ slot_ids, int* __restrict__ last,
+                                                          float* __restrict__ out, int d, int vocab, int buckets,
+                                                          long long mul_prev, long long mul_cur, float scale) {
+  __shared__ int row_of;
+  const int t = blockIdx.x;
+  if (threadIdx.x == 0) {
+    const int b = seq_of_tok[t], first = cu_seqlens[b];
+    int before = t > first ? ids[t - 1] : -1;
+    if (t == first) {
+      int* mine = last + slot_ids[b];
+      if (positions[t] > 0) before = *mine;
+      *mine = ids[cu_seqlens[b + 1] - 1];
+    }
+    const long long sum = (long long)before * mul_prev + (long long)ids[t] * mul_cur;
+    row_of = positions[t] > 0 ? (int)((sum % buckets + buckets) % buckets) : buckets;
+  }
+  __syncthreads();
+  const int id = ids[t];
+  float* o = out + (size_t)t * d;
+  if (id < 0 || id >= vocab) {
+    for (int i = threadIdx.x; i < d; i += 256) o[i] = __builtin_nanf("");
+    return;
+  }
+  const TT* src = table + (size_t)id * d;
+  const TT* pr = pairs + (size_t)row_of * d;
+  for (int i = threadIdx.x; i < d; i += 256) o[i] = fmaf(to_f32(src[i]), scale, to_f32(pr[i]));
+}
+
+// table [vocab][d], pairs [buckets + 1][d] of one type; last int32 [slots]
+MF_API int mf_embed_pairs(const void* table, const void* pairs, int tables_are_bf16, const int* ids, const int* positions,
+                          const int* seq_of_tok, const int* cu_seqlens, const int* slot_ids, int* last, float* out, int rows,
+                          int d, int vocab, int buckets, long long mul_prev, long long mul_cur, float scale,
+                          hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (d <= 0 || vocab <= 0 || buckets <= 0) return (int)hipErrorInvalidValue;
+  if (tables_are_bf16)
+    embed_pairs_kernel<bf16><<<rows, 256, 0, stream>>>((const bf16*)table, (const bf16*)pairs, ids, positions, seq_of_tok,
+                                                        cu_seqlens, slot_ids, last, out, d, vocab, buckets, mul_prev, mul_cur,
+                                                        scale);
+  else
+    embed_pairs_kernel<float><<<rows, 256, 0, stream>>>((const float*)table, (const float*)pairs, ids, positions, seq_of_tok,
+                                                         cu_seqlens, slot_ids, last, out, d, vocab, buckets, mul_prev, mul_cur,
+                                                         scale);
+  return mf_launch_status();
+}
+
 // ---------------------------------------------------------------- RMSNorm
 // y = x * (1/sqrt(mean(x^2) + eps)) * w  (src/vec_ops.rs:500-522; eps inside the root).
 // Row r of the output reads row row_idx[r] of x when row_idx is given.
@@ -277,27 +333,28 @@ MF_API int mf_gather_rows(const float* x, const int* idx, float* out, int rows, 
 // of one [rows][2*nf] buffer.
 template <typename IT, typename OT>
 __global__ __launch_bounds__(256) void swiglu_kernel(const IT* __restrict__ gu, OT* __restrict__ out,
-                                                     int nf) {
+                                                     int nf, float limit) {
   const IT* g = gu + (size_t)blockIdx.y * 2 * nf;
   const IT* u = g + nf;
   OT* o = out + (size_t)blockIdx.y * nf;
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i < nf) {
     const float z = to_f32(g[i]);
-    o[i] = from_f32<OT>(z / (1.0f + expf(-z)) * to_f32(u[i]));
+    o[i] = from_f32<OT>(limit > 0.f ? clamped_gate(z, to_f32(u[i]), limit) : z / (1.0f + expf(-z)) * to_f32(u[i]));
   }
 }
 
-MF_API int mf_swiglu(const void* gu, int in_is_bf16, void* out, int out_is_bf16, int rows, int nf,
+// limit > 0: the clamped form, g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1)
+MF_API int mf_swiglu(const void* gu, int in_is_bf16, void* out, int out_is_bf16, int rows, int nf, float limit,
                      hipStream_t stream) {
   if (rows <= 0) return 0;
   dim3 grid((nf + 255) / 256, rows);
   if (in_is_bf16 && out_is_bf16)
-    swiglu_kernel<bf16, bf16><<<grid, 256, 0, stream>>>((const bf16*)gu, (bf16*)out, nf);
+    swiglu_kernel<bf16, bf16><<<grid, 256, 0, stream>>>((const bf16*)gu, (bf16*)out, nf, limit);
   else if (!in_is_bf16 && out_is_bf16)
-    swiglu_kernel<float, bf16><<<grid, 256, 0, stream>>>((const float*)gu, (bf16*)out, nf);
+    swiglu_kernel<float, bf16><<<grid, 256, 0, stream>>>((const float*)gu, (bf16*)out, nf, limit);
   else if (!in_is_bf16 && !out_is_bf16)
-    swiglu_kernel<float, float><<<grid, 256, 0, stream>>>((const float*)gu, (float*)out, nf);
+    swiglu_kernel<float, float><<<grid, 256, 0, stream>>>((const float*)gu, (float*)out, nf, limit);
   else
     return (int)hipErrorInvalidValue;
   return mf_launch_status();

@@ -30,7 +30,9 @@
 // same outputs (the last group padded with zero rows), so a gate column and its up column
 // are 32 apart inside one wave's tile; the epilogue writes bfloat16 y[M][ldc], ldc = number
 // of outputs, straight from the 32-bit accumulators and the [M][2 nf] intermediate is never
-// stored.
+// stored.  Its products have no bias; where `bias` is given all the same, it points to one number,
+// the limit of the clamped form y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
+// u = clamp(up, -limit, limit), which takes silu's place.
 #include <stdio.h>
 #include <stdlib.h>
 
@@ -58,7 +60,10 @@ __device__ __forceinline__ void store_out(void* C, int ldc, int m, int n, float 
   }
 }
 
-__device__ __forceinline__ float swiglu_f(float g, float u) { return g / (1.0f + expf(-g)) * u; }
+__device__ __forceinline__ float swiglu_f(float g, float u, const float* __restrict__ limit) {
+  if (limit) return clamped_gate(g, u, *limit);
+  return g / (1.0f + expf(-g)) * u;
+}
 
 // 8 consecutive k of one row, zero at and beyond k_end.  Rows are clamped by the caller to a
 // row that exists (results of such rows are never stored), so the fast form has no branch:
@@ -105,7 +110,7 @@ __device__ __forceinline__ void tile_epilogue(floatx16 (&acc)[TM][TN], const flo
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int m = m0 + wm + i * 32 + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
-            if (m < M) ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(acc[i][j][r], acc[i][j + 1][r]);
+            if (m < M) ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(acc[i][j][r], acc[i][j + 1][r], bias);
           }
         }
     }
@@ -864,7 +869,7 @@ __global__ __launch_bounds__(NW * 64) void skinny16_kernel(const bf16* __restric
           float g = 0.f, u = 0.f;
 #pragma unroll
           for (int w = 0; w < NW; ++w) { g += red[w][0][lane][r]; u += red[w][1][lane][r]; }
-          ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u);
+          ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u, bias);
         }
       }
     }
@@ -1132,7 +1137,7 @@ __global__ __launch_bounds__(NW * 64) void rolling16_kernel(const bf16* __restri
         float g = 0.f, u = 0.f;
 #pragma unroll
         for (int ww = 0; ww < NW; ++ww) { g += red[ww][m][r16]; u += red[ww][m][16 + r16]; }
-        ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u);
+        ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u, bias);
       }
     }
     return;
@@ -1452,7 +1457,7 @@ __global__ __launch_bounds__(NW * 64) void stationary16_kernel(const void* __res
         const float sc = NORM ? row_scale(m) : rfac[m];
         g *= sc;
         u *= sc;
-        ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u);
+        ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(g, u, bias);
       }
     } else {
       if (e_mine) {
@@ -1670,7 +1675,8 @@ __global__ __launch_bounds__(512) void panel_kernel(const bf16* __restrict__ A, 
         if (c < cnt * 8 && col < ldc) {
           const int o = (c >> 4) * 32 + (c & 15);
           for (int m = tid >> 8; m < M; m += 2)
-            ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(ot[m * OT_LD + o] * rfac[m], ot[m * OT_LD + o + 16] * rfac[m]);
+            ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(ot[m * OT_LD + o] * rfac[m], ot[m * OT_LD + o + 16] * rfac[m],
+                                                                    bias);
         }
       } else {
         const int col = u0 * 32 + c;
@@ -1734,7 +1740,7 @@ __global__ __launch_bounds__(256) void skinny_reduce_kernel(const float* __restr
     const int ng = (n >> 5) * 64 + (n & 31);
     const float g = sum_of_parts(part, stride, (size_t)m * N + ng, splits);
     const float u = sum_of_parts(part, stride, (size_t)m * N + ng + 32, splits);
-    ((bf16*)C)[(size_t)m * ldc + n] = (bf16)swiglu_f(g * rf, u * rf);
+    ((bf16*)C)[(size_t)m * ldc + n] = (bf16)swiglu_f(g * rf, u * rf, bias);
     return;
   }
   float v = 0.f;                 // the output's new value (0 beyond the row's end)
@@ -2061,7 +2067,7 @@ MF_API int mf_gemm_bf16(const void* A, int lda, const void* W, int ldw, const fl
                         int ldc, int M, int N, int K, int epi, int variant, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || lda < K || ldw < K || epi < 0 || epi > EPI_XIELU || (epi == EPI_XIELU && !bias)) return (int)hipErrorInvalidValue;
-  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32 || bias) : ldc < N)
+  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32) : ldc < N)
     return (int)hipErrorInvalidValue;
   const int vec_ok = (lda % 8 == 0) && (ldw % 8 == 0) && ((uintptr_t)A % 16 == 0) &&
                      ((uintptr_t)W % 16 == 0) && (K % 8 == 0);
@@ -2105,7 +2111,7 @@ MF_API int mf_gemm_bf16_splitk(const void* A, int lda, const void* W, int ldw, c
   if (K <= 0 || lda < K || ldw < K || epi < 0 || epi > EPI_XIELU || (epi == EPI_XIELU && !bias) || splits < 2 || !part || k_per_split % 64 != 0 ||
       (long)splits * k_per_split < K || (long)(splits - 1) * k_per_split >= K)
     return (int)hipErrorInvalidValue;
-  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32 || bias) : ldc < N)
+  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32) : ldc < N)
     return (int)hipErrorInvalidValue;
   const int vec_ok = (lda % 8 == 0) && (ldw % 8 == 0) && ((uintptr_t)A % 16 == 0) &&
                      ((uintptr_t)W % 16 == 0) && (K % 8 == 0);
@@ -2161,7 +2167,7 @@ static int skinny_product(const void* A, int lda, const void* W, const void* Wt,
   if (M > 64 || K <= 0 || lda < K || ldw < K || epi < 0 || epi > EPI_XIELU || (epi == EPI_XIELU && !bias) || splits < 1 ||
       k_per_split % KC != 0 || (long)splits * k_per_split < K || (splits > 1 && !part))
     return (int)hipErrorInvalidValue;
-  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32 || bias || (M > 16 && !part))
+  if (epi == EPI_SWIGLU ? (N % 64 != 0 || ldc > N / 2 || ldc <= N / 2 - 32 || (M > 16 && !part))
                         : ldc < N)
     return (int)hipErrorInvalidValue;
   const int vec_ok = (lda % 8 == 0) && (ldw % 8 == 0) && ((uintptr_t)A % 16 == 0) &&

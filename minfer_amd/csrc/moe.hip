@@ -9,7 +9,12 @@
 // softmax over the chosen logits alone (the scores' common divisor cancels).
 // Further options: the scores are sigmoid(logits) instead of the softmax; a correction per expert joins the
 // scores for the choice of groups and experts only (the weights take the scores themselves); a group's score is
-// the sum of its `group_top` best (corrected) scores instead of its best; the weights are multiplied by a scale.
+// the sum of its `group_top` best (corrected) scores instead of its best; the weights are multiplied by a scale;
+// the weights are the chosen scores as they are, not over their sum (`normalize` 0).
+//
+// An expert number from `n_real` on stands for no matrices at all: such an expert hands its input on as it is.  It
+// takes part in the choice like any other; grouping and products pass it by, and the sum of a token's choices takes
+// the token's input in its output's place (`moe_combine_kernel`).
 //
 // A table in a router's place (`moe_table_kernel`): row id of the table names the experts of token id, all of one
 // weight.
@@ -66,7 +71,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
                                                        float* __restrict__ dense, int* __restrict__ chosen,
                                                        float* __restrict__ weights, int E, int n_groups, int keep,
                                                        int top, int score_kind, const float* __restrict__ correction,
-                                                       int group_top, float weight_scale) {
+                                                       int group_top, float weight_scale, int normalize) {
   __shared__ float s[MF_MOE_MAX_EXPERTS], ms[MF_MOE_MAX_EXPERTS], gs[MF_MOE_MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const XT* xr = x + (size_t)t * K;
@@ -158,7 +163,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
     MF_WAVE_SYNC();
   }
   if (lane < top) {
-    const float wgt = s[mine] / (wsum + 1e-20f) * weight_scale;
+    const float wgt = (normalize ? s[mine] / (wsum + 1e-20f) : s[mine]) * weight_scale;
     if (dense) dense[(size_t)t * E + mine] = wgt;
     chosen[(size_t)t * top + lane] = mine;
     weights[(size_t)t * top + lane] = wgt;
@@ -184,9 +189,7 @@ __global__ __launch_bounds__(256) void moe_table_kernel(const int* __restrict__ 
 
 __device__ __forceinline__ float expert_act(float g, float u, float limit, int act) {
   if (act == MF_MOE_ACT_SILU) return g * (1.0f / (1.0f + expf(-g))) * u;
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g * (1.0f / (1.0f + expf(-1.702f * g))) * (u + 1.0f);
+  return clamped_gate(g, u, limit);
 }
 
 // gu [tokens][E][2 F] (an expert's gate sums, then its up sums); dense [tokens][E]; y [tokens][E F]
@@ -451,38 +454,57 @@ __global__ __launch_bounds__(256) void moe_group_kernel(const int* __restrict__ 
   if (threadIdx.x == 0) counts[e] = before;
 }
 
-// xs[row(p)][:] = x[p / top][:]
+// xs[row(p)][:] = x[p / top][:], for the pairs whose expert has matrices
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ x, const int* __restrict__ chosen,
                                                          const int* __restrict__ rank, const int* __restrict__ offsets,
-                                                         T* __restrict__ xs, int top, int K) {
+                                                         T* __restrict__ xs, int top, int K, int n_real) {
   const int p = blockIdx.x;
+  if (chosen[p] >= n_real) return;
   const T* src = x + (size_t)(p / top) * K;
   T* dst = xs + (size_t)(offsets[chosen[p]] + rank[p]) * K;
   for (int i = threadIdx.x; i < K; i += 256) dst[i] = src[i];
 }
 
-// out[t][:] (+)= sum_k w[t][k] rows[row(t top + k)][:], the choices in their order
+// out[t][:] (+)= sum_k w[t][k] rows[row(t top + k)][:], the choices in their order; x[t][:] in the row's place where the
+// expert hands its input on
+template <typename XT>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, const int* __restrict__ chosen,
                                                           const int* __restrict__ rank, const int* __restrict__ offsets,
-                                                          const float* __restrict__ weights, float* __restrict__ out,
-                                                          int top, int N, int add) {
+                                                          const float* __restrict__ weights, const XT* __restrict__ x,
+                                                          int n_real, float* __restrict__ out, int top, int N, int add) {
   const int t = blockIdx.x;
   const int i = blockIdx.y * 256 + threadIdx.x;
   if (i >= N) return;
   float a = add ? out[(size_t)t * N + i] : 0.f;
   for (int k = 0; k < top; ++k) {
     const int p = t * top + k;
+    if (chosen[p] >= n_real) {
+      a = fmaf(weights[p], to_f32(x[(size_t)t * N + i]), a);
+      continue;
+    }
     const int row = offsets ? offsets[chosen[p]] + rank[p] : p;      // without offsets: pair p's row is row p
     a = fmaf(weights[p], rows[(size_t)row * N + i], a);
   }
   out[(size_t)t * N + i] = a;
 }
 
+static int launch_combine(const float* rows, const int* chosen, const int* rank, const int* offsets, const float* weights,
+                          const void* x, int x_is_bf16, int n_real, float* out, int n_tok, int top, int N, int add,
+                          hipStream_t stream) {
+  if (!x) n_real = 0x7fffffff;       // every expert has matrices
+  const dim3 grid(n_tok, (N + 255) / 256);
+  if (x_is_bf16)
+    moe_combine_kernel<bf16><<<grid, 256, 0, stream>>>(rows, chosen, rank, offsets, weights, (const bf16*)x, n_real, out, top, N, add);
+  else
+    moe_combine_kernel<float><<<grid, 256, 0, stream>>>(rows, chosen, rank, offsets, weights, (const float*)x, n_real, out, top, N, add);
+  return mf_launch_status();
+}
+
 // ------------------------------------------------------------------ entry points
 MF_API int mf_moe_route(const void* x, int x_is_bf16, const float* router, const float* bias, int K, float* dense, int* chosen,
                         float* weights, int n_tok, int E, int n_groups, int keep, int top, int score_kind,
-                        const float* correction, int group_top, float weight_scale, hipStream_t stream) {
+                        const float* correction, int group_top, float weight_scale, int normalize, hipStream_t stream) {
   if (n_tok <= 0) return 0;
   if (K <= 0 || E <= 0 || E > MF_MOE_MAX_EXPERTS || n_groups <= 0 || E % n_groups || keep <= 0 || keep > n_groups || top <= 0 ||
       top > 64 || top > keep * (E / n_groups) || group_top < 1 ||
@@ -490,10 +512,10 @@ MF_API int mf_moe_route(const void* x, int x_is_bf16, const float* router, const
     return (int)hipErrorInvalidValue;
   if (x_is_bf16)
     moe_route_kernel<bf16><<<n_tok, 256, 0, stream>>>((const bf16*)x, router, bias, K, dense, chosen, weights, E, n_groups, keep, top,
-                                                      score_kind, correction, group_top, weight_scale);
+                                                      score_kind, correction, group_top, weight_scale, normalize);
   else
     moe_route_kernel<float><<<n_tok, 256, 0, stream>>>((const float*)x, router, bias, K, dense, chosen, weights, E, n_groups, keep, top,
-                                                      score_kind, correction, group_top, weight_scale);
+                                                      score_kind, correction, group_top, weight_scale, normalize);
   return mf_launch_status();
 }
 
@@ -513,8 +535,9 @@ MF_API int mf_moe_act(const float* gu, const float* dense, void* y, int y_is_bf1
 
 MF_API int mf_moe_sparse(const void* x, const void* gate_up, const void* down, const int* chosen, const float* weights,
                          void* y, float* rows, float* out, int is_bf16, int n_tok, int top, int E, int F, int K, int N,
-                         float limit, int act, int add, hipStream_t stream) {
+                         float limit, int act, int add, int hands_on, hipStream_t stream) {
   if (n_tok <= 0) return 0;
+  if (hands_on && K != N) return (int)hipErrorInvalidValue;
   if (act != MF_MOE_ACT_CLAMPED && act != MF_MOE_ACT_SILU) return (int)hipErrorInvalidValue;
   if (top <= 0 || E <= 0 || F <= 0 || K <= 0 || N <= 0 || n_tok > MF_MOE_SPARSE_TOKENS || n_tok * top > MF_MOE_SPARSE_PAIRS ||
       !y || !rows)
@@ -541,8 +564,8 @@ MF_API int mf_moe_sparse(const void* x, const void* gate_up, const void* down, c
   }
   int rc = mf_launch_status();
   if (rc) return rc;
-  moe_combine_kernel<<<dim3(n_tok, (N + 255) / 256), 256, 0, stream>>>(rows, chosen, nullptr, nullptr, weights, out, top, N, add);
-  return mf_launch_status();
+  // (experts from E on hand their input on, whose rows are the outputs' then)
+  return launch_combine(rows, chosen, nullptr, nullptr, weights, hands_on ? x : nullptr, is_bf16, E, out, n_tok, top, N, add, stream);
 }
 
 MF_API int mf_moe_group(const int* chosen, int n_pairs, int E, int* rank, int* counts, hipStream_t stream) {
@@ -552,20 +575,21 @@ MF_API int mf_moe_group(const int* chosen, int n_pairs, int E, int* rank, int* c
 }
 
 MF_API int mf_moe_gather(const void* x, int is_bf16, const int* chosen, const int* rank, const int* offsets, void* xs,
-                         int n_pairs, int top, int K, hipStream_t stream) {
+                         int n_pairs, int top, int K, int n_real, hipStream_t stream) {
   if (n_pairs <= 0) return 0;
   if (is_bf16)
-    moe_gather_kernel<bf16><<<n_pairs, 256, 0, stream>>>((const bf16*)x, chosen, rank, offsets, (bf16*)xs, top, K);
+    moe_gather_kernel<bf16><<<n_pairs, 256, 0, stream>>>((const bf16*)x, chosen, rank, offsets, (bf16*)xs, top, K, n_real);
   else
-    moe_gather_kernel<float><<<n_pairs, 256, 0, stream>>>((const float*)x, chosen, rank, offsets, (float*)xs, top, K);
+    moe_gather_kernel<float><<<n_pairs, 256, 0, stream>>>((const float*)x, chosen, rank, offsets, (float*)xs, top, K, n_real);
   return mf_launch_status();
 }
 
+// x [n_tok][N]: the tokens' inputs, read for the pairs of experts from n_real on (null where there are none)
 MF_API int mf_moe_combine(const float* rows, const int* chosen, const int* rank, const int* offsets, const float* weights,
-                          float* out, int n_tok, int top, int N, int add, hipStream_t stream) {
+                          const void* x, int x_is_bf16, int n_real, float* out, int n_tok, int top, int N, int add,
+                          hipStream_t stream) {
   if (n_tok <= 0) return 0;
-  moe_combine_kernel<<<dim3(n_tok, (N + 255) / 256), 256, 0, stream>>>(rows, chosen, rank, offsets, weights, out, top, N, add);
-  return mf_launch_status();
+  return launch_combine(rows, chosen, rank, offsets, weights, x, x_is_bf16, n_real, out, n_tok, top, N, add, stream);
 }
 
 // table int32 [vocab][top]; ids int32; rows int32 [n_tok] or null; chosen, weights [n_tok][top]

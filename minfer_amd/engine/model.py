@@ -12,8 +12,9 @@ from typing import Callable, Dict
 
 import torch
 
+from ..cache.paged import split_request, widest_request
 from ..kernels import ops, tuning
-from ..parts.base import (BLOCKS, COMBINERS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, Runtime, make_part,
+from ..parts.base import (BLOCKS, COMBINERS, EMBEDDING_ENTRY, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, Runtime, make_part,
                           normed_input)
 from ..parts.spec import BlockSpec, ModelSpec
 from ..weights.loader import TensorSpec
@@ -55,6 +56,8 @@ class DecoderModel:
         self.final_norm = make_part(NORMS, spec.final_norm, self.rt, "norm")
         self.embedding = make_part(EMBEDDINGS, spec.embedding, self.rt, "embedding")
         self.head = make_part(HEADS, spec.head, self.rt, "head")
+        if self.embedding.cache_request() is not None and any(e.adds_embedding for e in spec.schedule):
+            raise ValueError("an embedding that keeps state runs once a step; this run order takes its output in again")
         self.stop_tokens = tuple(spec.stop_tokens)      # a loader may add to them (generation_config.json)
         self.loaded = False
         self.decode_copy_bytes = 0      # of the parts' tiled second copies, once loaded
@@ -113,9 +116,24 @@ class DecoderModel:
 
     # ------------------------------------------------------------ cache needs
     def cache_requests(self) -> Dict[int, object]:
-        """cache entry -> what the mixer that writes it asks for."""
-        return {e.cache: None if self.blocks[e.block].mixer is None else self.blocks[e.block].mixer.cache_request()
-                for e in self.spec.schedule if e.writes_cache}
+        """cache entry -> what the mixer that writes it asks for, joined by the needs of those that only read it; and
+        the embedding's own, where it keeps state."""
+        def asked(e):
+            mixer = self.blocks[e.block].mixer
+            return None if mixer is None else mixer.cache_request()
+        out = {e.cache: asked(e) for e in self.spec.schedule if e.writes_cache}
+        for e in self.spec.schedule:
+            if e.writes_cache:
+                continue
+            # a reader may see further back than the layer that writes: the entry keeps what either sees
+            (kv, state), (read, _) = split_request(out[e.cache]), split_request(asked(e))
+            if kv is not None and read is not None:
+                kv = widest_request(kv, read)
+                out[e.cache] = kv if state is None else (kv, state)
+        own = self.embedding.cache_request()
+        if own is not None:
+            out[EMBEDDING_ENTRY] = own
+        return out
 
     def prepare(self, max_len: int) -> None:
         for part in (self.embedding, self.head, self.final_norm):

@@ -7,7 +7,7 @@ from __future__ import annotations
 
 import ctypes
 import sys
-from ctypes import c_char_p, c_double, c_float, c_int, c_size_t, c_uint64, c_void_p
+from ctypes import c_char_p, c_double, c_float, c_int, c_int64, c_size_t, c_uint64, c_void_p
 from typing import Dict, Optional, Tuple
 
 import torch
@@ -30,10 +30,11 @@ _P = c_void_p
 _PROTOTYPES = {
     "elementwise": {
         "mf_embed": [_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P],
+        "mf_embed_pairs": [_P, _P, c_int, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int64, c_int64, c_float, _P],
         "mf_rmsnorm": [_P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_rmsnorm_cols": [_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_gather_rows": [_P, _P, _P, c_int, c_int, _P],
-        "mf_swiglu": [_P, c_int, _P, c_int, c_int, c_int, _P],
+        "mf_swiglu": [_P, c_int, _P, c_int, c_int, c_int, c_float, _P],
         "mf_convert": [_P, c_int, _P, c_int, c_size_t, _P],
         "mf_rope_table": [_P, _P, c_int, c_int, c_double, c_double, _P],
         "mf_rope_kvwrite": [_P, _P, _P, _P, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int,
@@ -70,12 +71,12 @@ _PROTOTYPES = {
         "mf_qkv_conv_prep": [_P, _P, c_int, _P, _P, _P, _P, _P, _P, _P, c_int, c_float, _P, _P, _P, c_int, _P, _P, _P,
                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P],
         "mf_capped_attn": [_P, _P, _P, _P, c_int, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int,
-                           c_float, c_float, c_int, c_int, _P, _P, c_int, _P, c_int, c_int, c_int, _P],
+                           c_float, c_float, c_int, c_int, _P, _P, c_int, _P, c_int, _P, c_int, c_int, _P],
         "mf_rope_half_inplace": [_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     },
     "attn_capped_mfma": {
         "mf_capped_mfma": [_P, _P, _P, _P, c_int, _P, _P, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int,
-                           c_int, c_float, c_float, c_int, c_int, _P, _P, c_int, _P, c_int, _P],
+                           c_int, c_float, c_float, c_int, c_int, _P, _P, c_int, _P, c_int, _P, _P],
     },
     "attn_normed": {
         "mf_qk_norm_prep": [_P, _P, _P, c_float, c_int, _P, _P, _P, _P, c_int, c_int, c_int, _P, _P, c_int, _P, c_int, _P, _P, _P,
@@ -93,15 +94,15 @@ _PROTOTYPES = {
                              c_int, c_int, c_int, c_int, c_int, _P],
     },
     "moe": {
-        "mf_moe_route": [_P, c_int, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_float, _P],
+        "mf_moe_route": [_P, c_int, _P, _P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_float, c_int, _P],
         "mf_moe_act": [_P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P],
         "mf_moe_sparse": [_P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
-                          c_int, _P],
+                          c_int, c_int, _P],
         "mf_moe_table": [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
         "mf_gated_expert_act": [_P, c_int, _P, c_int, c_int, c_int, _P],
         "mf_moe_group": [_P, c_int, c_int, _P, _P, _P],
-        "mf_moe_gather": [_P, c_int, _P, _P, _P, _P, c_int, c_int, c_int, _P],
-        "mf_moe_combine": [_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
+        "mf_moe_gather": [_P, c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
+        "mf_moe_combine": [_P, _P, _P, _P, _P, _P, c_int, c_int, _P, c_int, c_int, c_int, c_int, _P],
     },
     "recurrence": {
         "mf_mingru_scan": [_P, _P, _P, _P, _P, c_int, c_int, c_int, _P],
@@ -370,6 +371,29 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: floa
                                            table.shape[0], float(scale), _stream()), "embed")
 
 
+def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, seq_of_tok: torch.Tensor,
+                cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, last: torch.Tensor, mul_prev: int, mul_cur: int,
+                out: torch.Tensor, scale: float = 1.0) -> None:
+    """out[t] = table[ids[t]] * scale + pairs[row], in 32-bit, with row = (previous * mul_prev + ids[t] * mul_cur) mod n for
+    `pairs` of n + 1 rows, and row n for a sequence's first token.  The previous token of the first one a sequence
+    brings is `last[slot]` (int32 `[slots]` or `[slots][1]`), which is left holding the last one it brings."""
+    _need(table, "embed_pairs.table", _FLOATS)
+    n, d = ids.numel(), table.shape[1]
+    buckets = pairs.shape[0] - 1
+    _need(pairs, "embed_pairs.pairs", table.dtype, (buckets + 1, d))
+    for name, t in (("ids", ids), ("positions", positions), ("seq_of_tok", seq_of_tok)):
+        _need(t, "embed_pairs." + name, torch.int32, (n,))
+    _need(slot_ids, "embed_pairs.slot_ids", torch.int32)
+    _need(cu_seqlens, "embed_pairs.cu_seqlens", torch.int32, (slot_ids.numel() + 1,))
+    _need(last, "embed_pairs.last", torch.int32)
+    _need(out, "embed_pairs.out", torch.float32, (n, d))
+    if buckets < 1 or max(abs(int(mul_prev)), abs(int(mul_cur))) >= 1 << 31:
+        raise KernelError(f"embed_pairs: {buckets} buckets, factors {mul_prev} and {mul_cur}")
+    _check(_fn("elementwise", "mf_embed_pairs")(
+        _ptr(table), _ptr(pairs), _is_bf16(table), _ptr(ids), _ptr(positions), _ptr(seq_of_tok), _ptr(cu_seqlens), _ptr(slot_ids),
+        _ptr(last), _ptr(out), n, d, table.shape[0], buckets, int(mul_prev), int(mul_cur), float(scale), _stream()), "embed_pairs")
+
+
 def rmsnorm(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out: torch.Tensor,
             row_idx: Optional[torch.Tensor] = None, cols: Optional[int] = None) -> None:
     """out = x / sqrt(mean(x^2) + eps) * weight, row by row (row r reads x[row_idx[r]] where given).  `cols`: the norm
@@ -406,7 +430,9 @@ def gather_rows(x: torch.Tensor, idx: torch.Tensor, out: torch.Tensor) -> None:
                                                  x.shape[1], _stream()), "gather_rows")
 
 
-def swiglu(gate_up: torch.Tensor, out: torch.Tensor) -> None:
+def swiglu(gate_up: torch.Tensor, out: torch.Tensor, limit: float = 0.0) -> None:
+    """out = silu(gate) * up of rows gate | up; with a `limit` above 0 the clamped form g sigmoid(1.702 g) (u + 1),
+    g = min(gate, limit), u = clamp(up, -limit, limit)."""
     _need(gate_up, "swiglu.gate_up", _FLOATS)
     rows, two_nf = gate_up.shape
     if two_nf % 2:
@@ -415,7 +441,7 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor) -> None:
     if _is_bf16(gate_up) and not _is_bf16(out):
         raise KernelError("swiglu: bfloat16 input with float32 output is not provided")
     _check(_fn("elementwise", "mf_swiglu")(_ptr(gate_up), _is_bf16(gate_up), _ptr(out), _is_bf16(out),
-                                            rows, two_nf // 2, _stream()), "swiglu")
+                                            rows, two_nf // 2, float(limit), _stream()), "swiglu")
 
 
 def convert(src: torch.Tensor, dst: torch.Tensor) -> None:
@@ -1153,14 +1179,16 @@ def _need_kv_pages(what: str, kcache: torch.Tensor, vcache: torch.Tensor, dtype,
 def capped_attn(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, page_table: torch.Tensor,
                 positions: torch.Tensor, seq_of_tok: torch.Tensor, temp: torch.Tensor, out: torch.Tensor,
                 n_heads: int, n_kv_heads: int, dim: int, v_dim: int, scale: float, cap: float, window: int,
-                max_len: int, chunk: int = 0, far=None, keep_first: int = 0, bias: Optional[torch.Tensor] = None) -> None:
+                max_len: int, chunk: int = 0, far=None, keep_first: int = 0, bias: Optional[torch.Tensor] = None,
+                sink: Optional[torch.Tensor] = None) -> None:
     """Each query token attends to its sequence's cache rows lo..position with
     s = cap tanh(q . k scale temp[head] / cap) (no cap where `cap` is 0), ordinary softmax; keys of
     `dim` and values of `v_dim` values.  `chunk`: a token sees only the keys of its own chunk of that many
     positions, counted from 0.  `far` = (a, b), float32 per head: s -= a[h] ln(1 + b[h] (position - key)); with b
     None, s -= a[h] (position - key).
     `keep_first`: with a window, the sequence's first so many positions stay in sight of every later token.
-    `bias` float32 `[heads][n]`: s += bias[h][min(position - key, n - 1)]."""
+    `bias` float32 `[heads][n]`: s += bias[h][min(position - key, n - 1)].  `sink` float32 `[heads]`: the softmax's
+    denominator also holds e^sink[h] (not scaled, once a head and token)."""
     n_tok = positions.numel()
     _need(q, "capped_attn.q", _FLOATS, (n_tok, n_heads * dim))
     _need(out, "capped_attn.out", q.dtype, (n_tok, n_heads * v_dim))
@@ -1175,6 +1203,8 @@ def capped_attn(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, pag
     if max_len > page_table.shape[1] * PAGE:
         raise KernelError(f"capped_attn: max_len {max_len} exceeds the page table ({page_table.shape[1]} pages)")
     far_a, far_b = _far_pair("capped_attn", far, n_heads)
+    if sink is not None:
+        _need(sink, "capped_attn.sink", torch.float32, (n_heads,))
     keep_first, n_bias = _kept_and_bias("capped_attn", keep_first, window, chunk, bias, n_heads)
     # keys split over workgroups where tokens x kv heads alone do not fill the chip: at least 256 keys a split;
     # a windowed token's splits start at its window's first key
@@ -1190,7 +1220,7 @@ def capped_attn(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, pag
         _ptr(q), _ptr(kcache), _ptr(vcache), _ptr(page_table), page_table.shape[1], _ptr(positions), _ptr(seq_of_tok),
         _ptr(temp), _ptr(out), _ptr(part), _is_bf16(q), n_tok, n_heads, n_kv_heads, dim, v_dim, float(scale),
         float(cap or 0.0), int(window or 0), int(chunk or 0), _ptr(far_a), _ptr(far_b), keep_first, _ptr(bias), n_bias,
-        n_splits, split_len, _stream()), "capped_attn")
+        _ptr(sink), n_splits, split_len, _stream()), "capped_attn")
 
 
 def _kept_and_bias(what: str, keep_first, window, chunk, bias: Optional[torch.Tensor], n_heads: int):
@@ -1231,7 +1261,7 @@ def capped_mfma_takes(dtype, dim: int, v_dim: int) -> bool:
 def capped_attn_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, page_table: torch.Tensor, ctx,
                         temp: torch.Tensor, out: torch.Tensor, n_heads: int, n_kv_heads: int, dim: int, v_dim: int,
                         scale: float, cap: float, window: int, chunk: int = 0, far=None, keep_first: int = 0,
-                        bias: Optional[torch.Tensor] = None) -> None:
+                        bias: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None) -> None:
     """`capped_attn` in bfloat16 on the matrix cores: blocks of 16 consecutive new tokens of a sequence
     (`ctx.query_tiles`) times the query heads of a kv head.  A decode step (one token a sequence) splits every
     token's keys over several waves (at least 128 keys a split) and merges the parts in their order."""
@@ -1251,6 +1281,8 @@ def capped_attn_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Ten
     if ctx.max_len > page_table.shape[1] * PAGE:
         raise KernelError(f"capped_attn_prefill: max_len {ctx.max_len} exceeds the page table")
     far_a, far_b = _far_pair("capped_attn_prefill", far, n_heads)
+    if sink is not None:
+        _need(sink, "capped_attn_prefill.sink", torch.float32, (n_heads,))
     keep_first, n_bias = _kept_and_bias("capped_attn_prefill", keep_first, window, chunk, bias, n_heads)
     n_splits, split_len, part = 1, 0, None
     if ctx.all_decode:
@@ -1273,7 +1305,7 @@ def capped_attn_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Ten
         _ptr(q), _ptr(kcache), _ptr(vcache), _ptr(page_table), page_table.shape[1], _ptr(ctx.cu_seqlens),
         _ptr(ctx.start_pos), _ptr(tile_seq), _ptr(tile_q0), tile_seq.numel(), _ptr(temp), _ptr(out), _ptr(part), n_splits,
         split_len, n_tok, n_heads, n_kv_heads, dim, v_dim, float(scale), float(cap or 0.0), int(window or 0),
-        int(chunk or 0), _ptr(far_a), _ptr(far_b), keep_first, _ptr(bias), n_bias, _stream()),
+        int(chunk or 0), _ptr(far_a), _ptr(far_b), keep_first, _ptr(bias), n_bias, _ptr(sink), _stream()),
         "capped_attn_decode" if ctx.all_decode else "capped_attn_prefill")
 
 
@@ -1285,7 +1317,7 @@ MOE_SPARSE_TOKENS, MOE_SPARSE_PAIRS = 16, 128     # what `moe_sparse` takes in o
 def moe_route(x: torch.Tensor, router: torch.Tensor, dense: Optional[torch.Tensor], chosen: torch.Tensor,
               weights: torch.Tensor, n_groups: int, keep: int, bias: Optional[torch.Tensor] = None,
               score: str = "softmax", correction: Optional[torch.Tensor] = None, group_top: int = 1,
-              weight_scale: float = 1.0) -> None:
+              weight_scale: float = 1.0, normalize: bool = True) -> None:
     """The router: logits = router x in 32-bit (`router` float32 `[experts][K]`, `x` `[tokens][K]` in the run
     type), softmax scores, the `keep` best of `n_groups` groups of neighbouring experts (a group's score is
     its best expert's), the `chosen.shape[1]` best experts of those groups, weighted by their scores over
@@ -1294,7 +1326,7 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, dense: Optional[torch.Tenso
     group the weights are the softmax over the chosen logits alone.  `score` "sigmoid": the scores are
     sigmoid(logits).  `correction` float32 `[experts]` joins the scores where groups and experts are chosen, not in
     the weights.  `group_top`: a group's score is the sum of its so many best (corrected) scores.  `weight_scale`
-    multiplies the weights."""
+    multiplies the weights.  Without `normalize` the weights are the chosen scores as they are, not over their sum."""
     n_tok, K = x.shape
     E = router.shape[0]
     top = chosen.shape[1]
@@ -1314,7 +1346,7 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, dense: Optional[torch.Tenso
         raise KernelError(f"moe_route: scores {score!r} (one of {sorted(MOE_SCORES)}), group_top {group_top}")
     _check(_fn("moe", "mf_moe_route")(_ptr(x), _is_bf16(x), _ptr(router), _ptr(bias), K, _ptr(dense), _ptr(chosen), _ptr(weights),
                                        n_tok, E, n_groups, keep, top, MOE_SCORES[score], _ptr(correction), int(group_top),
-                                       float(weight_scale), _stream()), "moe_route")
+                                       float(weight_scale), 1 if normalize else 0, _stream()), "moe_route")
 
 
 MOE_ACTS = {"clamped_swish": 0, "silu": 1}      # the experts' activations (MF_MOE_ACT_* in csrc/moe.hip)
@@ -1337,13 +1369,17 @@ def moe_act(gu: torch.Tensor, dense: torch.Tensor, out: torch.Tensor, limit: flo
 
 
 def moe_sparse(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-               out: torch.Tensor, n_experts: int, limit: float, act: int = 0, accumulate: bool = True) -> None:
+               out: torch.Tensor, n_experts: int, limit: float, act: int = 0, accumulate: bool = True,
+               hands_on: bool = False) -> None:
     """The chosen experts only, for steps of few tokens: `gate_up` `[experts][2 F][K]` (an expert's gate
     rows, then its up rows), `down` `[experts][N][F]`; out `[tokens][N]` float32 (+)= the weighted sum of the
-    chosen experts' outputs, choices added in their order."""
+    chosen experts' outputs, choices added in their order.  `hands_on`: `chosen` may also name experts from `n_experts`
+    on, whose output is their input."""
     n_tok, K = x.shape
     top = chosen.shape[1]
     _, N, F = down.shape
+    if hands_on and K != N:
+        raise KernelError(f"moe_sparse: inputs of {K} values cannot stand for outputs of {N}")
     _need(x, "moe_sparse.x", _FLOATS)
     _need(gate_up, "moe_sparse.gate_up", x.dtype, (n_experts, 2 * F, K))
     _need(down, "moe_sparse.down", x.dtype, (n_experts, N, F))
@@ -1357,7 +1393,7 @@ def moe_sparse(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chose
     rows = torch.empty((n_tok * top, N), dtype=torch.float32, device=x.device)
     _check(_fn("moe", "mf_moe_sparse")(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(chosen), _ptr(weights), _ptr(y), _ptr(rows), _ptr(out),
                                         _is_bf16(x), n_tok, top, n_experts, F, K, N, float(limit), int(act),
-                                        1 if accumulate else 0, _stream()), "moe_sparse")
+                                        1 if accumulate else 0, 1 if hands_on else 0, _stream()), "moe_sparse")
 
 SCAN_CHUNK = 32          # tokens of a chunk of the chunked scan (MF_SCAN_CHUNK in csrc/recurrence.hip)
 
@@ -1821,9 +1857,12 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 
 
 def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, variant: int = 0,
-                  tiled: Optional[torch.Tensor] = None) -> None:
+                  tiled: Optional[torch.Tensor] = None, limit: Optional[torch.Tensor] = None) -> None:
     """out = silu(x @ Wg^T) * (x @ Wu^T) in one kernel; `weight` is `interleave_gate_up(Wg, Wu)`,
-    everything bfloat16, `out` is [rows][nf].  `tiled`: `tile_weight(weight)`."""
+    everything bfloat16, `out` is [rows][nf].  `tiled`: `tile_weight(weight)`.  `limit` (float32, one number on the
+    device): the clamped form of `swiglu` with that limit."""
+    if limit is not None:
+        _need(limit, "linear_swiglu.limit", torch.float32, (1,))
     _need(x, "linear_swiglu.x", torch.bfloat16)
     _need(weight, "linear_swiglu.weight", torch.bfloat16)
     m, k = x.shape
@@ -1839,7 +1878,7 @@ def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, vari
         splits, per = _k_split(m, n, k, True, aligned, tiled=tiled is not None)
         part = workspace("skinny", splits * m * n, x.device) if m > 16 or splits > 1 else None
         _need_tiled(tiled, "linear_swiglu.tiled", n, k)
-        _check(_fn("gemm_bf16", "mf_gemm_bf16_skinny")(_ptr(x), k, _ptr(weight), _ptr(tiled), k, _ptr(None), _ptr(out), nf,
+        _check(_fn("gemm_bf16", "mf_gemm_bf16_skinny")(_ptr(x), k, _ptr(weight), _ptr(tiled), k, _ptr(limit), _ptr(out), nf,
                                                         _ptr(part), m, n, k, splits, per, EPI_SWIGLU, _stream()),
                f"gemm_bf16_skinny(swiglu) {m}x{n}x{k}")
         return
@@ -1847,11 +1886,11 @@ def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, vari
         variant, splits, per = tile_plan(m, n, k, EPI_SWIGLU, aligned)
         if splits > 1:
             part = workspace("skinny", splits * m * n, x.device)
-            _check(_fn("gemm_bf16", "mf_gemm_bf16_splitk")(_ptr(x), k, _ptr(weight), k, _ptr(None), _ptr(out), nf,
+            _check(_fn("gemm_bf16", "mf_gemm_bf16_splitk")(_ptr(x), k, _ptr(weight), k, _ptr(limit), _ptr(out), nf,
                                                             _ptr(part), m, n, k, splits, per, EPI_SWIGLU, variant,
                                                             _stream()), f"gemm_bf16_splitk(swiglu) {m}x{n}x{k}")
             return
-    _check(_fn("gemm_bf16", "mf_gemm_bf16")(_ptr(x), k, _ptr(weight), k, _ptr(None), _ptr(out), nf, m, n, k,
+    _check(_fn("gemm_bf16", "mf_gemm_bf16")(_ptr(x), k, _ptr(weight), k, _ptr(limit), _ptr(out), nf, m, n, k,
                                              EPI_SWIGLU, variant, _stream()), f"gemm_bf16(swiglu) {m}x{n}x{k}")
 
 
@@ -2337,30 +2376,47 @@ def moe_group(chosen: torch.Tensor, n_experts: int, rank: torch.Tensor, counts: 
     _check(_fn("moe", "mf_moe_group")(_ptr(chosen), chosen.numel(), n_experts, _ptr(rank), _ptr(counts), _stream()), "moe_group")
 
 
-def moe_gather(x: torch.Tensor, chosen: torch.Tensor, rank: torch.Tensor, offsets: torch.Tensor, xs: torch.Tensor) -> None:
+ALL_REAL = 0x7fffffff      # every expert number a router can name has matrices
+
+
+def _need_pair_rows(t: torch.Tensor, name: str, dtype, pairs: int, width: int, all_pairs: bool) -> None:
+    """Rows of (token, choice) pairs: of all of them, or of those whose expert has matrices."""
+    _need(t, name, dtype)
+    if t.dim() != 2 or t.shape[1] != width or not (t.shape[0] == pairs if all_pairs else t.shape[0] <= pairs):
+        raise KernelError(f"{name}: shape {tuple(t.shape)} for {pairs} pairs of {width}")
+
+
+def moe_gather(x: torch.Tensor, chosen: torch.Tensor, rank: torch.Tensor, offsets: torch.Tensor, xs: torch.Tensor,
+               n_real: Optional[int] = None) -> None:
     """xs[offsets[chosen[t][k]] + rank[t][k]] = x[t]: the tokens of every expert side by side, one expert after
-    the other."""
+    the other.  `n_real`: pairs whose expert number is not below it are left out (`xs` holds the others' rows)."""
     n_tok, K = x.shape
     top = chosen.shape[1]
     _need(x, "moe_gather.x", _FLOATS)
     _need(chosen, "moe_gather.chosen", torch.int32, (n_tok, top))
     _need(rank, "moe_gather.rank", torch.int32, (n_tok, top))
     _need(offsets, "moe_gather.offsets", torch.int32)
-    _need(xs, "moe_gather.xs", x.dtype, (n_tok * top, K))
+    _need_pair_rows(xs, "moe_gather.xs", x.dtype, n_tok * top, K, n_real is None)
     _check(_fn("moe", "mf_moe_gather")(_ptr(x), _is_bf16(x), _ptr(chosen), _ptr(rank), _ptr(offsets), _ptr(xs), n_tok * top,
-                                        top, K, _stream()), "moe_gather")
+                                        top, K, ALL_REAL if n_real is None else int(n_real), _stream()), "moe_gather")
 
 
 def moe_combine(rows: torch.Tensor, chosen: torch.Tensor, rank: torch.Tensor, offsets: torch.Tensor, weights: torch.Tensor,
-                out: torch.Tensor, accumulate: bool = True) -> None:
-    """out[t] (+)= sum_k weights[t][k] rows[offsets[chosen[t][k]] + rank[t][k]], a token's choices in their order."""
+                out: torch.Tensor, accumulate: bool = True, x: Optional[torch.Tensor] = None, n_real: Optional[int] = None) -> None:
+    """out[t] (+)= sum_k weights[t][k] rows[offsets[chosen[t][k]] + rank[t][k]], a token's choices in their order.  With `x`
+    (`[tokens][N]`, the tokens' inputs) and `n_real`, x[t] stands for the row of an expert from `n_real` on."""
     n_tok, top = chosen.shape
     N = out.shape[1]
-    _need(rows, "moe_combine.rows", torch.float32, (n_tok * top, N))
+    if (x is None) != (n_real is None):
+        raise KernelError("moe_combine: the inputs and the number of experts with matrices come together or not at all")
+    if x is not None:
+        _need(x, "moe_combine.x", _FLOATS, (n_tok, N))
+    _need_pair_rows(rows, "moe_combine.rows", torch.float32, n_tok * top, N, x is None)
     _need(chosen, "moe_combine.chosen", torch.int32)
     _need(rank, "moe_combine.rank", torch.int32, (n_tok, top))
     _need(offsets, "moe_combine.offsets", torch.int32)
     _need(weights, "moe_combine.weights", torch.float32, (n_tok, top))
     _need(out, "moe_combine.out", torch.float32, (n_tok, N))
-    _check(_fn("moe", "mf_moe_combine")(_ptr(rows), _ptr(chosen), _ptr(rank), _ptr(offsets), _ptr(weights), _ptr(out), n_tok,
-                                         top, N, 1 if accumulate else 0, _stream()), "moe_combine")
+    _check(_fn("moe", "mf_moe_combine")(_ptr(rows), _ptr(chosen), _ptr(rank), _ptr(offsets), _ptr(weights), _ptr(x),
+                                         0 if x is None else _is_bf16(x), ALL_REAL if n_real is None else int(n_real), _ptr(out),
+                                         n_tok, top, N, 1 if accumulate else 0, _stream()), "moe_combine")

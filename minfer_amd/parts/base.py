@@ -182,6 +182,10 @@ class FeedForward(Part):
         raise NotImplementedError
 
 
+# the cache entry of an embedding that keeps state (the run order's entries count from 0)
+EMBEDDING_ENTRY = -1
+
+
 class Embedding(Part):
     """Token ids in, rows of the 32-bit residual stream out."""
 
@@ -190,6 +194,11 @@ class Embedding(Part):
         `ctx` is the step (positions, sequences), for an embedding that depends on where a token
         stands."""
         raise NotImplementedError
+
+    def cache_request(self):
+        """A `StateRequest` for what the embedding keeps of a sequence between steps (cache entry
+        `EMBEDDING_ENTRY`), or None."""
+        return None
 
     def table(self) -> Optional[torch.Tensor]:
         """The `[vocab][hidden]` matrix a tied head multiplies by, if this embedding has one."""

@@ -7,9 +7,10 @@ from __future__ import annotations
 
 import torch
 
+from ..cache.paged import StateRequest
 from ..kernels import ops
 from ..weights.loader import TensorSpec
-from .base import NORMS, Runtime, Embedding, Head, make_part, register_embedding, register_head
+from .base import EMBEDDING_ENTRY, NORMS, Runtime, Embedding, Head, make_part, register_embedding, register_head
 from .linear import Linear
 
 
@@ -56,6 +57,39 @@ class NormedTokenEmbedding(TokenEmbedding):
     def forward(self, token_ids, out, ctx=None) -> None:
         ops.embed(self.weight, token_ids, out, self.scale)
         self.norm.forward(out, out=out)       # in place, 32-bit rows
+
+
+@register_embedding("token_pair_embedding")
+class TokenPairEmbedding(TokenEmbedding):
+    """The table's row (scaled), plus the row of a second table for the token and the one before it (not scaled):
+    row (previous mul_prev + token mul_cur) mod buckets, and the last row, number `buckets`, for a sequence's first
+    token.  A sequence's state is the last token it has brought.  params: name, pairs (tensors), vocab_size,
+    hidden_size, scale, buckets, mul_prev, mul_cur."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        p = spec.params
+        self.pairs_name = p["pairs"]
+        self.buckets, self.mul_prev, self.mul_cur = int(p["buckets"]), int(p["mul_prev"]), int(p["mul_cur"])
+        if self.buckets < 1:
+            raise ValueError(f"token_pair_embedding: {self.buckets} buckets")
+        self.pairs = None
+
+    def tensor_specs(self):
+        return dict(super().tensor_specs(), **{self.pairs_name: TensorSpec((self.buckets + 1, self.hidden))})
+
+    def load(self, get):
+        super().load(get)
+        self.pairs = get(self.pairs_name).contiguous()
+        if self.pairs.dtype != self.weight.dtype:          # one in 32-bit: both, which is exact
+            self.pairs, self.weight = self.pairs.to(torch.float32), self.weight.to(torch.float32)
+
+    def cache_request(self):
+        return StateRequest((1,), torch.int32)
+
+    def forward(self, token_ids, out, ctx=None) -> None:
+        ops.embed_pairs(self.weight, self.pairs, token_ids, ctx.positions, ctx.seq_of_tok, ctx.cu_seqlens, ctx.slot_ids,
+                        ctx.cache.state(EMBEDDING_ENTRY), self.mul_prev, self.mul_cur, out, self.scale)
 
 
 @register_head("linear_head")

@@ -15,29 +15,38 @@ from .linear import Linear
 
 @register_feed_forward("swiglu")
 class SwiGLU(FeedForward):
-    """params: hidden_size, intermediate_size, gate/up/down (tensor name stems)."""
+    """With `limit`, the clamped form in silu's place: g = min(gate x, limit), u = clamp(up x, -limit, limit),
+    down( g sigmoid(1.702 g) (u + 1) ), in the same kernels.
+    params: hidden_size, intermediate_size, gate/up/down (tensor name stems), suffix (of the tensor names, default
+    ".weight"), limit (None, or a positive number)."""
+
+    can_overwrite = True
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
         p = spec.params
         self.hidden, self.inter = int(p["hidden_size"]), int(p["intermediate_size"])
-        self.names = {k: p[k] for k in ("gate", "up", "down")}
-        self.gate_up = self.down = self.fused = self.fused_tiled = None
+        self.names = {k: p[k] + p.get("suffix", ".weight") for k in ("gate", "up", "down")}
+        self.limit = None if p.get("limit") is None else float(p["limit"])
+        if self.limit is not None and not self.limit > 0:
+            raise ValueError(f"swiglu: limit {self.limit} must be positive")
+        self.gate_up = self.down = self.fused = self.fused_tiled = self.limit_on_device = None
 
     def tensor_specs(self):
         n = self.names
-        return {n["gate"] + ".weight": TensorSpec((self.inter, self.hidden)),
-                n["up"] + ".weight": TensorSpec((self.inter, self.hidden)),
-                n["down"] + ".weight": TensorSpec((self.hidden, self.inter))}
+        return {n["gate"]: TensorSpec((self.inter, self.hidden)), n["up"]: TensorSpec((self.inter, self.hidden)),
+                n["down"]: TensorSpec((self.hidden, self.inter))}
 
     def load(self, get):
         n = self.names
-        gate, up = get(n["gate"] + ".weight"), get(n["up"] + ".weight")
+        gate, up = get(n["gate"]), get(n["up"])
         if self.rt.is_bf16 and gate.dtype == up.dtype == torch.bfloat16:
             self.fused = ops.interleave_gate_up(gate, up)
         else:
             self.gate_up = Linear.stacked([gate, up])
-        self.down = Linear(get(n["down"] + ".weight"))
+        self.down = Linear(get(n["down"]))
+        if self.limit is not None:
+            self.limit_on_device = torch.tensor([self.limit], dtype=torch.float32, device=self.down.weight.device)
 
     def decode_copies(self, make: bool, min_row_length: int = 0) -> int:
         n = self.down.decode_copy(make, min_row_length)
@@ -52,10 +61,11 @@ class SwiGLU(FeedForward):
 
     takes_normed = True
 
-    def forward(self, x, h, ctx) -> None:
+    def forward(self, x, h, ctx, accumulate: bool = True) -> None:
         y = torch.empty((x.shape[0], self.inter), dtype=self.rt.dtype, device=x.device)
         if self.fused is not None:
-            fold = x.norm.rms_scale() if isinstance(x, Normed) else None
+            # (the clamped form has no fold of the norm before it)
+            fold = x.norm.rms_scale() if isinstance(x, Normed) and self.limit is None else None
             done = False
             if fold is not None and x.ahead is not None:      # the product before prepared this norm's input
                 done = ops.linear_fused(x.ahead.xg, self.fused, None, y, tiled=self.fused_tiled, swiglu=True,
@@ -64,10 +74,11 @@ class SwiGLU(FeedForward):
                 done = ops.linear_normed(x.h, fold[0], fold[1], x.row_idx, self.fused, None, y, swiglu=True,
                                          tiled=self.fused_tiled)
             if not done:
-                ops.linear_swiglu(x.tensor() if isinstance(x, Normed) else x, self.fused, y, tiled=self.fused_tiled)
+                ops.linear_swiglu(x.tensor() if isinstance(x, Normed) else x, self.fused, y, tiled=self.fused_tiled,
+                                  limit=self.limit_on_device)
         else:
-            ops.swiglu(self.gate_up(x, out_dtype=torch.float32), y)
-        self.down(y, out=h, accumulate=True, ctx=ctx)
+            ops.swiglu(self.gate_up(x, out_dtype=torch.float32), y, limit=self.limit or 0.0)
+        self.down(y, out=h, accumulate=accumulate, ctx=ctx)
 
 
 def _softplus(v: float) -> float:

@@ -7,7 +7,10 @@ can be among the `top` chosen; the chosen experts' scores over their sum are the
 With one group (and so all of it kept) the weights are the softmax over the chosen logits alone.  A router may
 add a bias per expert to its logits.  A router may also score with sigmoid(z) instead of the softmax, choose
 groups and experts by score plus a correction per expert while weighing by the scores themselves, count a group
-by the sum of its `group_top` best (corrected) scores, and multiply the weights by a scale.
+by the sum of its `group_top` best (corrected) scores, multiply the weights by a scale, and weigh by the chosen
+scores as they are, not over their sum.
+Experts that hand their input on (`identity` of them, behind the others in the router's order) have no matrices: the
+router scores and chooses them like any other, and their output is the token's input.
 Expert (no biases): g = min(Wg x, limit), u = clamp(Wu x, -limit, limit), y = g sigmoid(1.702 g) (u + 1),
 output Wd y; or, with `act` "silu", the plain gated form y = silu(Wg x) (Wu x).  The result is the weighted sum
 of the chosen experts' outputs.
@@ -81,7 +84,8 @@ class Experts(FeedForward):
     """The experts and their two forms; who takes which is a subclass's `choose`.  params: hidden_size,
     intermediate_size (of one expert), n_experts, top, act ("clamped_swish", the default, with `limit`; or "silu"),
     expert (format of an expert's tensor stem, e.g. "mlp.e{}"; its matrices are stem + ".gate", ".up", ".down"),
-    shared (None, or dict(stem, weight, intermediate_size): the expert every token takes)."""
+    shared (None, or dict(stem, weight, intermediate_size): the expert every token takes), identity (how many expert
+    numbers from n_experts on stand for experts that hand their input on; default 0)."""
 
     can_overwrite = True
 
@@ -97,8 +101,11 @@ class Experts(FeedForward):
         self.limit = float(p["limit"]) if act == "clamped_swish" else 0.0
         self.expert_name = p["expert"]
         self.shared = None if p.get("shared") is None else SharedExpert(p["shared"], self.hidden, rt)
-        if not 1 <= self.top <= min(64, self.ne) or self.ne > ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"{spec.kind}: {self.top} of {self.ne} experts chosen (at most 64 of at most {ops.MOE_MAX_EXPERTS})")
+        self.identity = int(p.get("identity") or 0)
+        self.choices = self.ne + self.identity             # expert numbers that can be chosen
+        if self.ne < 1 or self.identity < 0 or not 1 <= self.top <= min(64, self.choices) or self.choices > ops.MOE_MAX_EXPERTS:
+            raise ValueError(f"{spec.kind}: {self.top} of {self.ne} + {self.identity} experts chosen (at most 64 of at most "
+                             f"{ops.MOE_MAX_EXPERTS})")
         self.gate_up = self.down = None
 
     def tensor_specs(self):
@@ -149,20 +156,21 @@ class Experts(FeedForward):
         if (n <= few or (ctx is not None and ctx.all_decode)) and x.dtype == self.gate_up.dtype:
             for t0 in range(0, n, few):      # (slices of a contiguous tensor's rows are contiguous)
                 ops.moe_sparse(x[t0:t0 + few], self.gate_up, self.down, chosen[t0:t0 + few], weights[t0:t0 + few],
-                               h[t0:t0 + few], self.ne, self.limit, self.act, accumulate=accumulate)
+                               h[t0:t0 + few], self.ne, self.limit, self.act, accumulate=accumulate, hands_on=self.identity > 0)
             return
         rank = torch.empty_like(chosen)
-        counts = torch.empty(self.ne, dtype=torch.int32, device=dev)
-        ops.moe_group(chosen, self.ne, rank, counts)
+        counts = torch.empty(self.choices, dtype=torch.int32, device=dev)
+        ops.moe_group(chosen, self.choices, rank, counts)
         per_expert = self.host_counts(ctx)
         if per_expert is None:
-            per_expert = [int(c) for c in counts.cpu()]      # the step waits for the host here
+            per_expert = [int(c) for c in counts.cpu()[:self.ne]]      # the step waits for the host here
         starts = [0]
         for c in per_expert:
             starts.append(starts[-1] + c)
-        pairs = n * self.top
+        pairs = starts[-1]                   # of experts with matrices; the others' stand nowhere
+        handed = dict(x=x, n_real=self.ne) if self.identity else {}
         # one product over all experts' rows where its kernel takes the sizes, else a product an expert
-        grouped = x.dtype == self.gate_up.dtype and ops.grouped_takes(x.dtype, 2 * self.inter, self.hidden) \
+        grouped = pairs > 0 and x.dtype == self.gate_up.dtype and ops.grouped_takes(x.dtype, 2 * self.inter, self.hidden) \
             and ops.grouped_takes(x.dtype, self.hidden, self.inter)
         plans = [ops.grouped_plan(per_expert, 2 * self.inter, self.hidden), ops.grouped_plan(per_expert, self.hidden, self.inter)] \
             if grouped else []
@@ -172,11 +180,13 @@ class Experts(FeedForward):
         meta = torch.tensor(flat, dtype=torch.int32, pin_memory=dev.type == "cuda").to(dev, non_blocking=True)
         offsets, at = meta[:self.ne], (self.ne + 3) // 4 * 4
         xs = torch.empty((pairs, self.hidden), dtype=x.dtype, device=dev)
-        ops.moe_gather(x, chosen, rank, offsets, xs)
+        ops.moe_gather(x, chosen, rank, offsets, xs, n_real=self.ne if self.identity else None)
         gu = torch.empty((pairs, 2 * self.inter), dtype=torch.float32, device=dev)
         y = torch.empty((pairs, self.inter), dtype=self.rt.dtype, device=dev)
         rows = torch.empty((pairs, self.hidden), dtype=torch.float32, device=dev)
-        if grouped:
+        if pairs == 0:
+            pass                             # every token's choices hand their input on
+        elif grouped:
             sizes = [4 * len(t) for t in tables]
             up_groups, down_groups = (meta[at + o:at + o + s].view(-1, 4) for o, s in zip((0, sizes[0]), sizes))
             ops.linear_grouped(xs, self.gate_up, up_groups, plans[0], gu)
@@ -190,7 +200,7 @@ class Experts(FeedForward):
             for e, (_, down) in enumerate(self.experts):
                 if per_expert[e]:
                     down(y[starts[e]:starts[e + 1]], out=rows[starts[e]:starts[e + 1]])
-        ops.moe_combine(rows, chosen, rank, offsets, weights, h, accumulate=accumulate)
+        ops.moe_combine(rows, chosen, rank, offsets, weights, h, accumulate=accumulate, **handed)
 
     def _ones(self, n: int, dev) -> torch.Tensor:
         """[n][1] ones: the activation kernel's weights where the weighting happens later."""
@@ -204,7 +214,8 @@ class Experts(FeedForward):
 class GroupedMoE(Experts):
     """params: those of `Experts`, and groups and keep (default 1: no groups), router (tensor name), router_bias
     (tensor name, or None), score ("softmax", the default, or "sigmoid"), correction (tensor name, or None),
-    group_top (default 1), weight_scale (default 1.0)."""
+    group_top (default 1), weight_scale (default 1.0), normalize (default True: the weights are the chosen scores over
+    their sum; False: the scores as they are).  The router has a row for each of the n_experts + identity experts."""
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
@@ -217,17 +228,18 @@ class GroupedMoE(Experts):
         self.weight_scale = float(p.get("weight_scale", 1.0))
         if self.score not in ops.MOE_SCORES or self.group_top < 1:
             raise ValueError(f"grouped_moe: scores {self.score!r} (one of {sorted(ops.MOE_SCORES)}), group_top {self.group_top}")
-        per = self.ne // max(1, self.groups)
-        if self.ne % self.groups or not 1 <= self.keep <= self.groups or not self.top <= self.keep * per:
-            raise ValueError(f"grouped_moe: {self.ne} experts in {self.groups} groups, {self.keep} kept, {self.top} chosen")
+        self.normalize = bool(p.get("normalize", True))
+        per = self.choices // max(1, self.groups)
+        if self.choices % self.groups or not 1 <= self.keep <= self.groups or not self.top <= self.keep * per:
+            raise ValueError(f"grouped_moe: {self.choices} experts in {self.groups} groups, {self.keep} kept, {self.top} chosen")
         self.router = self.router_bias = self.correction = None
 
     def tensor_specs(self):
-        s = {self.router_name: TensorSpec((self.ne, self.hidden))}
+        s = {self.router_name: TensorSpec((self.choices, self.hidden))}
         if self.bias_name is not None:
-            s[self.bias_name] = TensorSpec((self.ne,))
+            s[self.bias_name] = TensorSpec((self.choices,))
         if self.correction_name is not None:
-            s[self.correction_name] = TensorSpec((self.ne,))
+            s[self.correction_name] = TensorSpec((self.choices,))
         s.update(super().tensor_specs())
         return s
 
@@ -242,7 +254,7 @@ class GroupedMoE(Experts):
     def choose(self, x, ctx, chosen, weights) -> None:
         ops.moe_route(x, self.router, None, chosen, weights, self.groups, self.keep, bias=self.router_bias,
                       score=self.score, correction=self.correction, group_top=self.group_top,
-                      weight_scale=self.weight_scale)
+                      weight_scale=self.weight_scale, normalize=self.normalize)
 
 
 @register_feed_forward("table_moe")
@@ -252,6 +264,8 @@ class TableMoE(Experts):
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
+        if self.identity:
+            raise ValueError("table_moe: a table picks among experts with matrices")
         self.table_name, self.vocab = spec.params["table"], int(spec.params["vocab_size"])
         self.table = self.host_table = None
 

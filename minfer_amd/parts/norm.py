@@ -43,13 +43,15 @@ class RMSNorm(Norm):
 class GroupRMSNorm(Norm):
     """RMS norm taken over `groups` equal consecutive parts of the vector: each part is divided by
     its own sqrt(mean(part^2) + eps), then the whole is multiplied by the weight.  One group is the
-    plain RMS norm.  params: size, eps, groups, weight (tensor name)."""
+    plain RMS norm.  `gain_scale` is a number the whole gain is multiplied by, once, in 32-bit, when the weights
+    arrive (a factor behind the matrix that reads the norm, such as a scale of the logits, may stand here instead).
+    params: size, eps, groups, weight (tensor name), gain_scale (default 1)."""
 
     def __init__(self, spec, rt):
         super().__init__(spec, rt)
         p = spec.params
         self.size, self.eps, self.groups = int(p["size"]), float(p["eps"]), int(p.get("groups", 1))
-        self.name = p["weight"]
+        self.name, self.gain_scale = p["weight"], float(p.get("gain_scale", 1.0))
         if self.groups < 1 or self.size % self.groups:
             raise ValueError(f"group_rmsnorm: {self.size} values do not split into {self.groups} equal parts")
         self.weight = None
@@ -59,6 +61,8 @@ class GroupRMSNorm(Norm):
 
     def load(self, get):
         self.weight = get(self.name).to(torch.float32).contiguous()
+        if self.gain_scale != 1.0:
+            self.weight = self.weight * self.gain_scale
 
     def rms_scale(self):
         return (self.weight, self.eps) if self.groups == 1 else None

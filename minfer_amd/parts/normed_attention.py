@@ -20,7 +20,8 @@ values another layer's run left in its cache entry (the run order gives it that 
 biases on all four projections; `row_norm`: q and k over the root mean square of the whole projection, all heads at
 once, with gains as long as the projections (no rotation then); a query temperature that grows with the position,
 q <- q (1 + coef ln(floor((p + 1) / every) + 1)); a cap on the scaled score, cap tanh(s / cap); a penalty in proportion
-to the distance, slopes[h] (i - j), behind the cap.
+to the distance, slopes[h] (i - j), behind the cap; biases on queries, keys and values alone (`out_bias` False); a sink,
+a learned number per head whose exponential joins the softmax's denominator and nothing else.
 
 The attention itself runs in the kernels of the capped attention (temperatures of one).
 """
@@ -62,7 +63,7 @@ class NormedAttention(Mixer):
     chunk (None or int each), distance (None, or the names of the penalty's two per-head tensors), out_scale,
     qk_norm (default True), keep_first (None or int; needs a window), distance_bias (None, or dict(table: tensor
     name of `[rows][heads]`, rows, far)), shared_kv (default False), biases (default False; a bias is its
-    projection's name + ".b"), row_norm (default False; q_norm and k_norm name the gains), q_temperature (None, or
+    projection's name + ".b"), out_bias (default: as `biases`), sink (None, or the tensor's name), row_norm (default False; q_norm and k_norm name the gains), q_temperature (None, or
     dict(coef, every); needs row_norm), cap (None or a number), slopes (None, or one number per head), q, k, v, o,
     q_norm, k_norm (tensor names)."""
 
@@ -85,6 +86,8 @@ class NormedAttention(Mixer):
         self.bias_spec = p.get("distance_bias")
         self.shared_kv = bool(p.get("shared_kv", False))
         self.biases, self.row_norm = bool(p.get("biases", False)), bool(p.get("row_norm", False))
+        self.out_bias = bool(p.get("out_bias", self.biases))
+        self.sink_name = p.get("sink")
         self.q_temperature = None
         if p.get("q_temperature") is not None:
             self.q_temperature = (float(p["q_temperature"]["coef"]), int(p["q_temperature"]["every"]))
@@ -129,11 +132,14 @@ class NormedAttention(Mixer):
                 raise ValueError("normed_attention: the position encoding must be a rotation in pairs (pair_tables) or, for "
                                  "queries and keys, in halves (half_tables)")
         self.halves = self.position is not None and not hasattr(self.position, "pair_tables")
-        self.qkv = self.o = self.q_gain = self.k_gain = self.far = self.ones = self.bias = None
-        self.bias_names = [n + ".b" for n in (self.names["q"], self.names["k"], self.names["v"], self.names["o"])] \
-            if self.biases else []
-        if self.biases and (self.shared_kv or self.v_from_k):
-            raise ValueError("normed_attention: biases go with keys and values of the layer's own")
+        self.qkv = self.o = self.q_gain = self.k_gain = self.far = self.ones = self.bias = self.sink = None
+        if self.biases and self.v_from_k:
+            raise ValueError("normed_attention: biases go with a value matrix of the layer's own")
+
+    def _projections(self):
+        """(key of `names`, rows) of the stacked projections, in their order."""
+        own = (("k", self.nk * self.dim),) + (() if self.v_from_k else (("v", self.nk * self.vdim),))
+        return (("q", self.nh * self.dim),) + (() if self.shared_kv else own)
 
     def tensor_specs(self):
         n = self.names
@@ -147,12 +153,18 @@ class NormedAttention(Mixer):
             s[self.bias_spec["table"]] = TensorSpec((int(self.bias_spec["rows"]), self.nh))
         if self.gains:
             s[n["q_norm"]] = TensorSpec((self.dim,), init="ones")
-            s[n["k_norm"]] = TensorSpec((self.dim,), init="ones")
+            if not self.shared_kv:
+                s[n["k_norm"]] = TensorSpec((self.dim,), init="ones")
         if self.row_norm:
             s[n["q_norm"]] = TensorSpec((self.nh * self.dim,), init="ones")
             s[n["k_norm"]] = TensorSpec((self.nk * self.dim,), init="ones")
-        for name, rows in zip(self.bias_names, (self.nh * self.dim, self.nk * self.dim, self.nk * self.vdim, self.hidden)):
-            s[name] = TensorSpec((rows,))
+        if self.biases:
+            for k, rows in self._projections():
+                s[n[k] + ".b"] = TensorSpec((rows,))
+        if self.out_bias:
+            s[n["o"] + ".b"] = TensorSpec((self.hidden,))
+        if self.sink_name is not None:
+            s[self.sink_name] = TensorSpec((self.nh,))
         if self.distance is not None:
             # random weights: positive numbers, or the logarithm has no value
             s[self.distance[0]] = TensorSpec((self.nh,), init="halves")
@@ -161,18 +173,20 @@ class NormedAttention(Mixer):
 
     def load(self, get):
         n = self.names
-        self.qkv = Linear.stacked([get(n[k]) for k in (("q",) if self.shared_kv else ("q", "k") if self.v_from_k
-                                                       else ("q", "k", "v"))],
-                                  [get(name) for name in self.bias_names[:3]] if self.biases else None)
+        self.qkv = Linear.stacked([get(n[k]) for k, _ in self._projections()],
+                                  [get(n[k] + ".b") for k, _ in self._projections()] if self.biases else None)
         if self.bias_spec is not None:
             # the table by distance, a row a head: what the kernels look up
             table = get(self.bias_spec["table"]).to(torch.float32)
             rows = torch.tensor(self.bias_rows, dtype=torch.long, device=table.device)
             self.bias = table[rows].t().contiguous()
-        self.o = Linear(get(n["o"]), get(self.bias_names[3]) if self.biases else None)
+        self.o = Linear(get(n["o"]), get(n["o"] + ".b") if self.out_bias else None)
         if self.gains or self.row_norm:
             self.q_gain = get(n["q_norm"]).to(torch.float32).contiguous()
-            self.k_gain = get(n["k_norm"]).to(torch.float32).contiguous()
+            if not self.shared_kv:
+                self.k_gain = get(n["k_norm"]).to(torch.float32).contiguous()
+        if self.sink_name is not None:
+            self.sink = get(self.sink_name).to(torch.float32).contiguous()
         if self.distance is not None:
             self.far = tuple(get(name).to(torch.float32).contiguous() for name in self.distance)
         if self.slopes is not None:
@@ -216,11 +230,12 @@ class NormedAttention(Mixer):
         chunk = 0 if self.chunk is None else int(self.chunk)
         if ops.capped_mfma_takes(self.rt.dtype, self.dim, self.vdim):
             ops.capped_attn_prefill(q, kc, vc, table, ctx, self.ones, o, self.nh, self.nk, self.dim, self.vdim, self.scale,
-                                    self.cap, window, chunk=chunk, far=self.far, keep_first=self.keep_first, bias=self.bias)
+                                    self.cap, window, chunk=chunk, far=self.far, keep_first=self.keep_first, bias=self.bias,
+                                    sink=self.sink)
         else:
             ops.capped_attn(q, kc, vc, table, ctx.positions, ctx.seq_of_tok, self.ones, o, self.nh, self.nk, self.dim,
                             self.vdim, self.scale, self.cap, window, ctx.max_len, chunk=chunk, far=self.far,
-                            keep_first=self.keep_first, bias=self.bias)
+                            keep_first=self.keep_first, bias=self.bias, sink=self.sink)
         if vrot is not None or self.out_scale != 1.0:
             ops.unrotate(o, vrot, ctx.positions, self.nh, self.out_scale)
         self.o(o, out=h, accumulate=accumulate)

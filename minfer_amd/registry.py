@@ -52,6 +52,8 @@ def _register_builtin() -> None:
     register_architecture(katarax.ARCHITECTURE, katarax.KataraxConfig)
     from .config import rofizen
     register_architecture(rofizen.ARCHITECTURE, rofizen.RofizenConfig)
+    from .config import dolutar
+    register_architecture(dolutar.ARCHITECTURE, dolutar.DolutarConfig)
 
 
 _register_builtin()

@@ -39,9 +39,25 @@ def gather_rows(x, idx, out):
     out.copy_(x[idx.long()])
 
 
-def swiglu(gate_up, out):
+def embed_pairs(table, pairs, ids, positions, seq_of_tok, cu_seqlens, slot_ids, last, mul_prev, mul_cur, out, scale=1.0):
+    buckets = pairs.shape[0] - 1
+    for b in range(slot_ids.numel()):
+        r0, r1 = int(cu_seqlens[b]), int(cu_seqlens[b + 1])
+        before = int(last.view(-1)[int(slot_ids[b])])
+        for t in range(r0, r1):
+            assert int(seq_of_tok[t]) == b
+            row = buckets if int(positions[t]) == 0 else (before * mul_prev + int(ids[t]) * mul_cur) % buckets
+            out[t] = (table[int(ids[t])].double() * scale + pairs[row].double()).float()
+            before = int(ids[t])
+        last.view(-1)[int(slot_ids[b])] = before
+
+
+def swiglu(gate_up, out, limit=0.0):
     nf = gate_up.shape[1] // 2
     g, u = gate_up[:, :nf].double(), gate_up[:, nf:].double()
+    if limit > 0:
+        out.copy_(_expert_act(g, u, limit).to(out.dtype))
+        return
     out.copy_((g / (1.0 + torch.exp(-g)) * u).to(out.dtype))
 
 
@@ -129,11 +145,14 @@ def interleave_gate_up(gate, up):
     return out
 
 
-def linear_swiglu(x, weight, out, variant=0, tiled=None):
+def linear_swiglu(x, weight, out, variant=0, tiled=None, limit=None):
     nf = out.shape[1]
     idx = torch.arange(nf)
     g = x.double() @ weight.double()[(idx // 32) * 64 + idx % 32].t()
     u = x.double() @ weight.double()[(idx // 32) * 64 + 32 + idx % 32].t()
+    if limit is not None:
+        out.copy_(_expert_act(g, u, float(limit)).to(out.dtype))
+        return
     out.copy_((g / (1.0 + torch.exp(-g)) * u).to(out.dtype))
 
 
@@ -456,7 +475,7 @@ def qkv_conv_prep(qkv, conv_w, conv_state, cu_seqlens, seq_of_tok, slot_ids, pos
 
 
 def capped_attn(q, kcache, vcache, page_table, positions, seq_of_tok, temp, out, n_heads, n_kv_heads, dim, v_dim,
-                scale, cap, window, max_len, chunk=0, far=None, keep_first=0, bias=None):
+                scale, cap, window, max_len, chunk=0, far=None, keep_first=0, bias=None, sink=None):
     t_all = positions.numel()
     group = n_heads // n_kv_heads
     qq = q.double().view(t_all, n_heads, dim)
@@ -482,6 +501,8 @@ def capped_attn(q, kcache, vcache, page_table, positions, seq_of_tok, temp, out,
                 s = s - float(far[0][h]) * (d if far[1] is None else torch.log1p(float(far[1][h]) * d))
             if bias is not None:
                 s = s + bias[h].double()[torch.clamp(p - pos, max=bias.shape[1] - 1)]
+            if sink is not None:         # one more score, whose value is nothing
+                s, vals = torch.cat([s, sink[h:h + 1].double()]), torch.cat([vals, torch.zeros(1, v_dim, dtype=torch.float64)])
             out[i, h * v_dim:(h + 1) * v_dim] = (torch.softmax(s, dim=0) @ vals).to(out.dtype)
 
 
@@ -490,9 +511,9 @@ def capped_mfma_takes(dtype, dim, v_dim):
 
 
 def capped_attn_prefill(q, kcache, vcache, page_table, ctx, temp, out, n_heads, n_kv_heads, dim, v_dim, scale, cap, window,
-                        chunk=0, far=None, keep_first=0, bias=None):
+                        chunk=0, far=None, keep_first=0, bias=None, sink=None):
     capped_attn(q, kcache, vcache, page_table, ctx.positions, ctx.seq_of_tok, temp, out, n_heads, n_kv_heads, dim, v_dim,
-                scale, cap, window, ctx.max_len, chunk=chunk, far=far, keep_first=keep_first, bias=bias)
+                scale, cap, window, ctx.max_len, chunk=chunk, far=far, keep_first=keep_first, bias=bias, sink=sink)
 
 
 # ------------------------------------------------------------------ rows added into rows, the gated recurrence,
@@ -718,7 +739,7 @@ MOE_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
 def moe_route(x, router, dense, chosen, weights, n_groups, keep, bias=None, score="softmax", correction=None,
-              group_top=1, weight_scale=1.0):
+              group_top=1, weight_scale=1.0, normalize=True):
     logits = x.double() @ router.double().t()
     if bias is not None:
         logits = logits + bias.double()
@@ -737,7 +758,7 @@ def moe_route(x, router, dense, chosen, weights, n_groups, keep, bias=None, scor
         for g in kept.tolist():
             masked[g * per:(g + 1) * per] = choice[t, g * per:(g + 1) * per]
         pick = torch.argsort(-masked, stable=True)[:top]
-        w = s[t, pick] / (s[t, pick].sum() + 1e-20) * weight_scale
+        w = s[t, pick] / (s[t, pick].sum() + 1e-20 if normalize else 1.0) * weight_scale
         chosen[t] = pick.to(torch.int32)
         weights[t] = w
         if dense is not None:
@@ -760,7 +781,7 @@ def moe_act(gu, dense, out, limit, act=0):
     out.copy_(y.reshape(n_tok, E * F).to(out.dtype))
 
 
-def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0, accumulate=True):
+def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0, accumulate=True, hands_on=False):
     if not accumulate:
         out.zero_()
     n_tok, K = x.shape
@@ -770,6 +791,10 @@ def moe_sparse(x, gate_up, down, chosen, weights, out, n_experts, limit, act=0, 
     for t in range(n_tok):
         for k in range(chosen.shape[1]):
             e = int(chosen[t, k])
+            if e >= n_experts:
+                assert hands_on
+                out[t] += (float(weights[t, k]) * x[t].double()).float()
+                continue
             y = _expert_act(gu[e, 0] @ x[t].double(), gu[e, 1] @ x[t].double(), limit, act).to(x.dtype).double()
             out[t] += (float(weights[t, k]) * (dn[e] @ y)).float()
 
@@ -809,14 +834,18 @@ def _rows_of(chosen, rank, offsets):
     return (offsets.long()[chosen.long()] + rank.long()).reshape(-1)
 
 
-def moe_gather(x, chosen, rank, offsets, xs):
+def moe_gather(x, chosen, rank, offsets, xs, n_real=None):
     top = chosen.shape[1]
-    xs[_rows_of(chosen, rank, offsets)] = x.repeat_interleave(top, dim=0)
+    real = torch.ones(chosen.numel(), dtype=torch.bool) if n_real is None else chosen.reshape(-1) < n_real
+    xs[_rows_of(chosen.reshape(-1)[real], rank.reshape(-1)[real], offsets)] = x.repeat_interleave(top, dim=0)[real]
 
 
-def moe_combine(rows, chosen, rank, offsets, weights, out, accumulate=True):
+def moe_combine(rows, chosen, rank, offsets, weights, out, accumulate=True, x=None, n_real=None):
     n_tok, top = chosen.shape
-    picked = rows[_rows_of(chosen, rank, offsets)].double().view(n_tok, top, -1)
+    real = torch.ones(chosen.numel(), dtype=torch.bool) if n_real is None else chosen.reshape(-1) < n_real
+    picked = out.new_zeros(n_tok * top, out.shape[1]).double() if x is None else x.double().repeat_interleave(top, dim=0)
+    picked[real] = rows[_rows_of(chosen.reshape(-1)[real], rank.reshape(-1)[real], offsets)].double()
+    picked = picked.view(n_tok, top, -1)
     acc = out.double() if accumulate else torch.zeros(out.shape, dtype=torch.float64)
     for k in range(top):
         acc = acc + weights.double()[:, k, None] * picked[:, k]
@@ -890,7 +919,7 @@ def advance(next_ids, sampled, positions, steps, prev=None, n_prev=None, cursor=
             n_prev[i] = min(int(n_prev[i]) + 1, prev.shape[1])
 
 
-NAMES = ["embed", "rmsnorm", "gather_rows", "swiglu", "convert", "fill_normal", "rope_table",
+NAMES = ["embed", "embed_pairs", "rmsnorm", "gather_rows", "swiglu", "convert", "fill_normal", "rope_table",
          "rope_kvwrite", "rope_inplace", "linear", "attn_tokens", "attn_prefill", "argmax", "sample", "penalties",
          "top_k", "top_p", "sample_filtered", "sample_filtered_takes", "advance", "interleave_gate_up", "linear_swiglu", "linear_normed", "linear_fused", "attn_decode_rope",
          "group_rmsnorm", "xielu", "rope_table_freqs", "rope_pairs_inplace", "mingru_scan", "latent_prep",
