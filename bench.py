@@ -68,12 +68,12 @@ def parse():
                     help="cache size in tokens (default: batch x context, or what fits in free memory if less)")
     ap.add_argument("--no-graph", action="store_true")
     ap.add_argument("--only", choices=["decode", "prefill"], help="run one part (for profiles); prints no JSON line")
-    ap.add_argument("--design", choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen"], default=None,
+    ap.add_argument("--design", choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen", "dolutar"], default=None,
                     help="instead of the default workload: prefill and decode of this design at a few layer sizes "
                          "beside its nearest relative of the same width, depth and feed-forward size (the Qwen2 "
-                         "decoder; for nodutar, Lagedra), kernel by kernel")
+                         "decoder; a later design, the closest of the earlier ones), kernel by kernel")
     ap.add_argument("--design-sizes", default="small,medium", help="which of the design's sizes to run")
-    ap.add_argument("--design-model", default=None, choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen", "qwen2"],
+    ap.add_argument("--design-model", default=None, choices=["tabezen", "lagedra", "nodutar", "katarax", "rofizen", "dolutar", "qwen2"],
                     help="with --design and --only: which of the two models runs the one part (for profiles; "
                          "default: the design itself)")
     return ap.parse_args()
@@ -329,6 +329,21 @@ def rofizen_config(width, layers, heads, ff, dim=128, vdim=128, experts=8, rank=
                 layers=[dict((gla, both, ret, both)[i % 4], mlp=dense if i % 4 == 0 else routed) for i in range(layers)])
 
 
+def dolutar_config(width, layers, heads, ff, dim=128, vdim=128, window=1024, experts=8, identity=2, top=2, vocab=32768):
+    """Windowed attention with kept first positions and sinks, and a layer that reads the keys and values of the one
+    before it, in turn; the first layer of four with a dense feed-forward of `ff`, the others with routed experts of
+    ff / top values, `top` of them a token, and `identity` more that hand their input on; head sizes, kv heads, window and
+    kept positions as in `katarax_config`."""
+    own = dict(heads=heads, kv_heads=max(1, heads // 4), dim=dim, vdim=vdim, scale=dim ** -0.5, rot=dict(base=10000.0, dims=dim),
+               mask=dict(size=window, keep_first=4))
+    dense = dict(kind="dense", ff=ff, limit=7.0)
+    routed = dict(kind="moe", expert=dict(ff=ff // top), router=dict(experts=experts, identity=identity, top=top))
+    return dict(architecture="Dolutar", vocab=vocab, width=width, norm=dict(eps=1e-6), logit_scale=2.0,
+                embedding=dict(scale=1.0, bigram=dict(buckets=vocab - 1, mul_prev=1021, mul_cur=31)),
+                layers=[dict(type="attention", mixer=own if i % 2 == 0 else dict(own, kv_from=i - 1),
+                             mlp=dense if i % 4 == 0 else routed) for i in range(layers)])
+
+
 def qwen2_like(width, layers, heads, ff, vocab=32768):
     """The Qwen2 decoder of the same width, depth, head count and feed-forward size (head size 128)."""
     return dict(QWEN25_7B, num_hidden_layers=layers, hidden_size=width, num_attention_heads=heads,
@@ -343,9 +358,10 @@ DESIGN_SIZES = {
 
 
 DESIGN_CONFIGS = {"tabezen": tabezen_config, "lagedra": lagedra_config, "nodutar": nodutar_config, "katarax": katarax_config,
-                  "rofizen": rofizen_config, "qwen2": qwen2_like}
+                  "rofizen": rofizen_config, "dolutar": dolutar_config, "qwen2": qwen2_like}
 # the model a design is measured beside
-NEAREST = {"tabezen": "qwen2", "lagedra": "qwen2", "nodutar": "lagedra", "katarax": "nodutar", "rofizen": "nodutar"}
+NEAREST = {"tabezen": "qwen2", "lagedra": "qwen2", "nodutar": "lagedra", "katarax": "nodutar", "rofizen": "nodutar",
+           "dolutar": "katarax"}
 
 
 def traced_step(eng, slots, toks, want):

@@ -63,10 +63,11 @@ __device__ __forceinline__ void load4(const float* __restrict__ p, float (&d)[4]
   d[0] = v.x; d[1] = v.y; d[2] = v.z; d[3] = v.w;
 }
 
-// x [tokens][K] in the run type, router [E][K] float32: a workgroup per token; its four waves form the E
+// x [tokens][K] in the run type, router [E][K] float32: a workgroup per token; its NW waves form the E
 // logits (a wave an expert at a time, lanes over K in runs of 4, sums in 32-bit), then the first wave decides.
-template <typename XT>
-__global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x, const float* __restrict__ router,
+// Few tokens take more waves, so that a token's experts are read side by side.
+template <typename XT, int NW>
+__global__ __launch_bounds__(NW * 64) void moe_route_kernel(const XT* __restrict__ x, const float* __restrict__ router,
                                                        const float* __restrict__ bias, int K,
                                                        float* __restrict__ dense, int* __restrict__ chosen,
                                                        float* __restrict__ weights, int E, int n_groups, int keep,
@@ -75,7 +76,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
   __shared__ float s[MF_MOE_MAX_EXPERTS], ms[MF_MOE_MAX_EXPERTS], gs[MF_MOE_MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const XT* xr = x + (size_t)t * K;
-  for (int e = wv; e < E; e += 4) {
+  for (int e = wv; e < E; e += NW) {
     const float* wr = router + (size_t)e * K;
     float a = 0.f;
     if (K % 4 == 0) {
@@ -113,7 +114,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
   // an expert is chosen by its score plus the correction (the weights take the score alone); what cannot be
   // chosen counts as minus infinity, since corrected scores may be negative
   const int per = E / n_groups;
-  for (int g = lane; g < n_groups; g += 64) {
+  const bool all_kept = keep >= n_groups;        // every group is kept: their scores decide nothing
+  for (int g = all_kept ? n_groups : lane; g < n_groups; g += 64) {
     // the group's `group_top` largest choice scores, summed: each pass takes the best that comes behind the last
     // one taken in the order (larger first, lower index first)
     float total = 0.f, last_v = INFINITY;
@@ -133,9 +135,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const XT* __restrict__ x
     }
     gs[g] = total;
   }
-  for (int e = lane; e < E; e += 64) ms[e] = -INFINITY;
+  for (int e = lane; e < E; e += 64) ms[e] = all_kept ? s[e] + (correction ? correction[e] : 0.f) : -INFINITY;
   MF_WAVE_SYNC();
-  for (int k = 0; k < keep; ++k) {
+  for (int k = all_kept ? keep : 0; k < keep; ++k) {
     float b = -INFINITY;
     int bi = 0x7fffffff;
     for (int g = lane; g < n_groups; g += 64)
@@ -510,12 +512,18 @@ MF_API int mf_moe_route(const void* x, int x_is_bf16, const float* router, const
       top > 64 || top > keep * (E / n_groups) || group_top < 1 ||
       (score_kind != MF_MOE_SCORE_SOFTMAX && score_kind != MF_MOE_SCORE_SIGMOID))
     return (int)hipErrorInvalidValue;
-  if (x_is_bf16)
-    moe_route_kernel<bf16><<<n_tok, 256, 0, stream>>>((const bf16*)x, router, bias, K, dense, chosen, weights, E, n_groups, keep, top,
-                                                      score_kind, correction, group_top, weight_scale, normalize);
-  else
-    moe_route_kernel<float><<<n_tok, 256, 0, stream>>>((const float*)x, router, bias, K, dense, chosen, weights, E, n_groups, keep, top,
-                                                      score_kind, correction, group_top, weight_scale, normalize);
+#define MF_GO(XT, NW)                                                                                                    \
+  moe_route_kernel<XT, NW><<<n_tok, NW * 64, 0, stream>>>((const XT*)x, router, bias, K, dense, chosen, weights, E, n_groups, \
+                                                          keep, top, score_kind, correction, group_top, weight_scale,    \
+                                                          normalize)
+  if (n_tok <= 256 && E > 4) {
+    if (x_is_bf16) MF_GO(bf16, 16);
+    else MF_GO(float, 16);
+  } else {
+    if (x_is_bf16) MF_GO(bf16, 4);
+    else MF_GO(float, 4);
+  }
+#undef MF_GO
   return mf_launch_status();
 }
 

@@ -137,19 +137,28 @@ def clamped_ff(h, w, prefix: str, limit: float):
     return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[prefix + "down"].T
 
 
-def route(h, w, prefix: str, top: int):
-    """(experts, weights) of every token: scores are the softmax over all router outputs; chosen by score plus
-    correction, weighed by the score as it is."""
+def route(h, w, prefix: str, top: int, forced=None):
+    """(experts, weights, margins) of every token: scores are the softmax over all router outputs; chosen by score plus
+    correction, weighed by the score as it is.  The margin is how far the last one chosen lies above the first one left
+    out.  `forced` [tokens][top]: another's choice in its place (weighed by the scores here)."""
     z = h @ w[prefix + "router"].T
     e = np.exp(z - z.max(axis=-1, keepdims=True))
     s = e / e.sum(axis=-1, keepdims=True)
-    order = np.argsort(-(s + w[prefix + "correction"]), axis=-1, kind="stable")[:, :top]
-    return order, np.take_along_axis(s, order, axis=-1)
+    choice = s + w[prefix + "correction"]
+    order = np.argsort(-choice, axis=-1, kind="stable")
+    ranked = np.take_along_axis(choice, order, axis=-1)
+    margins = ranked[:, top - 1] - ranked[:, top] if top < choice.shape[1] else np.full(h.shape[0], np.inf)
+    order = order[:, :top] if forced is None else np.asarray(forced)
+    return order, np.take_along_axis(s, order, axis=-1), margins
 
 
-def mixture(h, w, prefix: str, experts: int, top: int):
-    """The weighted sum of the chosen experts; an expert number from `experts` on hands its input on."""
-    chosen, weight = route(h, w, prefix, top)
+def mixture(h, w, prefix: str, experts: int, top: int, forced=None, seen=None):
+    """The weighted sum of the chosen experts; an expert number from `experts` on hands its input on.  `seen`, where
+    given, gets (choices of the router here, margins)."""
+    if seen is not None:
+        own, _, margins = route(h, w, prefix, top)
+        seen.append((own, margins))
+    chosen, weight, _ = route(h, w, prefix, top, forced)
     out = np.zeros_like(h)
     for t in range(h.shape[0]):
         for e, a in zip(chosen[t], weight[t]):
@@ -162,10 +171,14 @@ def mixture(h, w, prefix: str, experts: int, top: int):
     return out
 
 
-def feed_forward(h, w, prefix: str, mlp):
+def feed_forward(h, w, prefix: str, mlp, forced=None, seen=None):
     if mlp["kind"] == "dense":
         return clamped_ff(h, w, prefix, mlp["limit"])
-    return mixture(h, w, prefix, mlp["router"]["experts"], mlp["router"]["top"])
+    return mixture(h, w, prefix, mlp["router"]["experts"], mlp["router"]["top"], forced, seen)
+
+
+def greedy(logits) -> int:
+    return int(np.argmax(logits))
 
 
 # ------------------------------------------------------------------ the model
@@ -175,8 +188,12 @@ class PlainDolutar:
             self.c = json.load(f)
         self.w = read_safetensors(os.path.join(folder, "model.safetensors"))
 
-    def streams(self, tokens):
-        """The residual stream behind every layer, [layers][tokens][width]."""
+    def routed_layers(self):
+        return [i for i, layer in enumerate(self.c["layers"]) if layer.get("mlp") and layer["mlp"]["kind"] == "moe"]
+
+    def streams(self, tokens, forced=None, seen=None):
+        """The residual stream behind every layer, [layers][tokens][width].  `forced`: {layer: another's choices of
+        experts}; `seen` gets (choices, margins) of every routed layer."""
         c, w, eps = self.c, self.w, self.c["norm"]["eps"]
         x = embed(tokens, w, c.get("embedding") or {})
         kept, out = {}, []
@@ -186,11 +203,11 @@ class PlainDolutar:
             kept[i] = keys_and_values(x, w, p + "mix.", m, eps) if j is None else kept[j]
             x = x + rms_norm(attention(x, kept[i], w, p + "mix.", m, eps), w[p + "norm1"], eps)
             if layer.get("mlp") is not None:
-                x = x + rms_norm(feed_forward(x, w, p + "mlp.", layer["mlp"]), w[p + "norm2"], eps)
+                x = x + rms_norm(feed_forward(x, w, p + "mlp.", layer["mlp"], (forced or {}).get(i), seen), w[p + "norm2"], eps)
             out.append(x)
         return np.stack(out)
 
-    def forward(self, tokens):
+    def forward(self, tokens, forced=None, seen=None):
         """Logits of every position, [tokens][vocab]."""
-        x = rms_norm(self.streams(tokens)[-1], self.w["final.norm"], self.c["norm"]["eps"])
+        x = rms_norm(self.streams(tokens, forced, seen)[-1], self.w["final.norm"], self.c["norm"]["eps"])
         return x @ self.w["head"].T * self.c.get("logit_scale", 1.0)
