@@ -100,19 +100,27 @@ __device__ __forceinline__ void tile_epilogue(floatx16 (&acc)[TM][TN], const flo
   // D[m][n]: lane holds n = lane % 32, m = 8 (r / 4) + 4 (lane / 32) + r % 4
   if (epi == EPI_SWIGLU) {
     if constexpr (TN % 2 == 0) {
+      auto gated = [&](auto act) {
 #pragma unroll
-      for (int i = 0; i < TM; ++i)
+        for (int i = 0; i < TM; ++i)
 #pragma unroll
-        for (int j = 0; j < TN; j += 2) {
-          const int ng = n0 + wn + j * 32 + fr;            // gate column; its up column is ng + 32
-          const int col = (ng >> 6) * 32 + (ng & 63);
-          if (col >= ldc) continue;
+          for (int j = 0; j < TN; j += 2) {
+            const int ng = n0 + wn + j * 32 + fr;            // gate column; its up column is ng + 32
+            const int col = (ng >> 6) * 32 + (ng & 63);
+            if (col >= ldc) continue;
 #pragma unroll
-          for (int r = 0; r < 16; ++r) {
-            const int m = m0 + wm + i * 32 + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
-            if (m < M) ((bf16*)C)[(size_t)m * ldc + col] = (bf16)swiglu_f(acc[i][j][r], acc[i][j + 1][r], bias);
+            for (int r = 0; r < 16; ++r) {
+              const int m = m0 + wm + i * 32 + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
+              if (m < M) ((bf16*)C)[(size_t)m * ldc + col] = (bf16)act(acc[i][j][r], acc[i][j + 1][r]);
+            }
           }
-        }
+      };
+      if (bias) {
+        const float limit = *bias;
+        gated([=](float g, float u) { return clamped_gate(g, u, limit); });
+      } else {
+        gated([](float g, float u) { return swiglu_f(g, u, nullptr); });
+      }
     }
     return;
   }
